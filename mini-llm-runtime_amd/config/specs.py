@@ -18,6 +18,7 @@ class NormSpec:
     size: int
     eps: float
     weight_offset: float = 0.0    # the factor is weight_offset + the stored weight (1: a weight stored around zero)
+    bias: bool = True             # "layernorm": a bias is added
 
 
 @dataclass(frozen=True)
@@ -34,12 +35,24 @@ class FrequencyStretch:
 
 
 @dataclass(frozen=True)
+class FrequencyBands:
+    """Rotation frequencies scaled by bands for contexts beyond the trained one (Llama 3.1): with t = original f / (2 pi)
+    turns over the original length, f stays where t > high, becomes f / factor where t < low, and between them
+    (1 - s) f / factor + s f with s = (t - low) / (high - low)."""
+    factor: float
+    original: float
+    low: float
+    high: float
+
+
+@dataclass(frozen=True)
 class PositionSpec:
     kind: str                 # key in the position registry: "rope_split_half", or "rope" (which reads every field)
     dim: int                  # rotated width (the head size here)
     base: float
     interleaved: bool = False                      # pairs (2 i, 2 i + 1) instead of (i, i + dim / 2)
     stretch: Optional[FrequencyStretch] = None
+    bands: Optional[FrequencyBands] = None
 
 
 @dataclass(frozen=True)
@@ -163,6 +176,28 @@ class SinkAttentionSpec:
 
 
 @dataclass(frozen=True)
+class HeadMixAttentionSpec:
+    """Causal grouped-query attention whose heads' softmax weights are mixed, weights_h <- sum_g talk[h, g] weights_g (a
+    learned [q_heads, q_heads] matrix), before they meet the values of the head's own kv head.  `sink`: one more summand
+    exp(sink) in every denominator -- a number, "learned" (one a head, tensor `sink`) or None; it takes no part in the
+    mixing.  `value_position`: values are turned by their position before they are cached, and a head's output turned
+    back by the query's."""
+    kind: str                 # "head_mix_attention"
+    hidden: int
+    q_heads: int
+    kv_heads: int
+    head_dim: int             # query/key channels of a head
+    value_dim: int
+    scale: float
+    softcap: Optional[float] = None              # score <- softcap * tanh(score / softcap)
+    qk_norm: Optional[NormSpec] = None           # per head, before the rotation
+    position: Optional[PositionSpec] = None      # `dim` of it: how many of a head's first channels turn
+    value_position: Optional[PositionSpec] = None    # dim == value_dim
+    sink: object = None
+    head_gate: Optional[str] = None              # "sigmoid": a head's output times sigmoid(Wg x)[head], Wg [heads, hidden]
+
+
+@dataclass(frozen=True)
 class LatentAttentionSpec:
     """Attention whose keys and values of all heads are made from one latent vector a token (normed, `rank`
     channels) by per-head up-projections, plus one rotated key part (`rot_dim` channels) that all heads share;
@@ -237,15 +272,16 @@ class PlainMlpSpec:
     kind: str                 # "plain_mlp"
     hidden: int
     intermediate: int
-    activation: str = "relu_squared"
+    activation: str = "relu_squared"      # or "gelu_erf": z Phi(z), the normal distribution's function
 
 
 @dataclass(frozen=True)
 class RoutedMlpSpec:
-    """A mixture of `experts` ungated feed-forwards of which a token uses `top`: scores sigmoid(router x); the
-    experts form `group_count` equal groups of neighbours, a group's score is the sum of its two largest scores,
-    only experts of the `group_keep` best groups can be chosen; the chosen experts' scores are their weights as
-    they are (`renormalize` False) or divided by their sum."""
+    """A mixture of `experts` ungated feed-forwards of which a token uses `top`: scores sigmoid(router x) or softmax(router
+    x) over all experts; the experts form `group_count` equal groups of neighbours, a group's score is the sum of its two
+    largest scores (or its largest), only experts of the `group_keep` best groups can be chosen; the chosen experts' scores
+    are their weights as they are (`renormalize` False) or divided by their sum.  `shared`: a feed-forward that every token
+    runs besides, added, with `shared_gate` times sigmoid(sg x), one number a token."""
     kind: str                 # "routed_mlp"
     hidden: int
     intermediate: int         # of one expert
@@ -254,11 +290,16 @@ class RoutedMlpSpec:
     group_count: int = 1
     group_keep: int = 1
     activation: str = "relu_squared"
-    score: str = "sigmoid"
+    score: str = "sigmoid"        # or "softmax"
+    group_score: str = "best_two" # or "best"
     renormalize: bool = False
     gated: bool = False           # an expert is down(act(gate x) * (up x)) with tensors e<i>.gate beside e<i>.up
     correction: bool = False      # the choice goes by s + a stored number an expert (`correction`), the weights by s
     route_scale: float = 1.0      # factor on the chosen weights
+    limit: Optional[float] = None         # activation "clamped": g = min(gate, limit), u = clamp(up, -limit, limit),
+    slope: float = 1.702                  # g sigmoid(slope g) (u + 1)
+    shared: Optional[object] = None       # any feed-forward spec; its tensors are named `shared.<local name>`
+    shared_gate: bool = False
 
 
 @dataclass(frozen=True)
@@ -266,7 +307,8 @@ class LayerSpec:
     kind: str                 # key in the block registry, e.g. "prenorm", "parallel"
     norm1: NormSpec
     mixer: object             # any mixer spec with a `kind`
-    norm2: Optional[NormSpec]     # None with `ffn` None: a layer without a feed-forward
+    norm2: Optional[NormSpec]     # None with `ffn` None: a layer without a feed-forward ("parallel": None with a
+                                  # feed-forward: both sublayers read norm1's output)
     ffn: object               # any feed-forward spec with a `kind`
     norm1_after: Optional[NormSpec] = None    # block "sandwich": the norm of what the mixer gives, before the residual sum
     norm2_after: Optional[NormSpec] = None    # likewise behind the feed-forward
@@ -288,6 +330,7 @@ class EmbedSpec:
     kind: str                 # key in the embed registry, e.g. "token_embedding"
     vocab_size: int
     hidden: int
+    scale: float = 1.0        # factor on the rows
 
 
 @dataclass(frozen=True)

@@ -6,7 +6,7 @@
 // h[m, :] = float(table[ids[m], :]).  An id outside [0, vocab) gives a row of NaN
 // (the host refuses such a batch before anything runs).
 __global__ void embed_gather_kernel(const int32_t* __restrict__ ids, const elem_t* __restrict__ table,
-                                    float* __restrict__ h, int width, int vocab) {
+                                    float* __restrict__ h, int width, int vocab, float scale) {
     const int m = blockIdx.x;
     const int id = ids[m];
     float* out = h + (size_t)m * width;
@@ -15,7 +15,7 @@ __global__ void embed_gather_kernel(const int32_t* __restrict__ ids, const elem_
         return;
     }
     const elem_t* row = table + (size_t)id * width;
-    for (int i = threadIdx.x; i < width; i += blockDim.x) out[i] = to_float(row[i]);
+    for (int i = threadIdx.x; i < width; i += blockDim.x) out[i] = to_float(row[i]) * scale;
 }
 
 __device__ __forceinline__ float block_max(float v, float* scratch) {
@@ -697,29 +697,6 @@ __global__ __launch_bounds__(256) void layernorm_kernel(const elem_t* __restrict
     }
 }
 
-// out = relu(x)^2, element by element (32-bit).
-__global__ void relu_squared_kernel(const elem_t* __restrict__ x, elem_t* __restrict__ out, size_t count) {
-    for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < count; i += (size_t)gridDim.x * blockDim.x) {
-        const float r = fmaxf(to_float(x[i]), 0.f);
-        out[i] = from_float<elem_t>(r * r);
-    }
-}
-
-// out = T(h): the float residual stream as a sublayer's input.
-__global__ void cast_rows_kernel(const float* __restrict__ h, elem_t* __restrict__ out, size_t count) {
-    for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < count; i += (size_t)gridDim.x * blockDim.x)
-        out[i] = from_float<elem_t>(h[i]);
-}
-
-// x *= factor (float values, logits for instance).
-__global__ void scale_float_kernel(float* __restrict__ x, float factor, size_t count) {
-    for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < count; i += (size_t)gridDim.x * blockDim.x)
-        x[i] *= factor;
-}
-
-// ---- a norm without statistics: y = tanh(alpha x) w + b, element by element, 32-bit ---------------------------
-__device__ __forceinline__ float tanh_norm(float x, float alpha, float w, float b) { return __builtin_fmaf(tanhf(alpha * x), w, b); }
-
 // VEC consecutive values in one access where VEC is 4 (the row's width a multiple of 4: 16-byte float accesses, 8- or
 // 16-byte accesses of the engine's element type), else one by one.
 template <int VEC> __device__ __forceinline__ void load_floats(const float* p, float* out) {
@@ -761,6 +738,124 @@ template <int VEC> __device__ __forceinline__ void store_elems(elem_t* p, const 
         p[0] = from_float<elem_t>(in[0]);
     }
 }
+
+// The activation of a feed-forward without a gate, element by element (32-bit): ACT 0 relu(x)^2; ACT 1 the exact gelu,
+// x Phi(x) with the normal distribution's function.  VEC: MLR_VEC values in one access, or 1.
+template <int ACT> __device__ __forceinline__ float plain_act(float x) {
+    if (ACT == 1) return 0.5f * x * (1.0f + erff(x * 0.70710678118654752440f));
+    const float r = fmaxf(x, 0.f);
+    return r * r;
+}
+template <int ACT, int VEC>
+__global__ void plain_act_kernel(const elem_t* __restrict__ x, elem_t* __restrict__ out, size_t count) {
+    for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < count; i += (size_t)gridDim.x * blockDim.x) {
+        if (VEC == 1) {
+            out[i] = from_float<elem_t>(plain_act<ACT>(to_float(x[i])));
+        } else {
+            float v[MLR_VEC];
+            load_vec(x + i * MLR_VEC, v);
+#pragma unroll
+            for (int e = 0; e < MLR_VEC; ++e) v[e] = plain_act<ACT>(v[e]);
+            store_vec(out + i * MLR_VEC, v);
+        }
+    }
+}
+
+// x = h + (d1 + d2) (each may be null), written back to h when one is given; out = layernorm(x) * weight (+ bias): the two
+// branches of a block and the norm that follows in one pass, the row kept in registers (up to 4 VEC LN2_REGS values a
+// lane's share of the row; wider rows are read again).  One workgroup a row; VEC 4: 16-byte float accesses.
+#define LN2_REGS 8
+template <int VEC>
+__global__ __launch_bounds__(256) void add2_layernorm_kernel(float* __restrict__ h, const elem_t* __restrict__ d1,
+                                                             const elem_t* __restrict__ d2, const float* __restrict__ weight,
+                                                             const float* __restrict__ bias, elem_t* __restrict__ out,
+                                                             int width, float eps) {
+    __shared__ float scratch[16];
+    const size_t row = (size_t)blockIdx.x * width;
+    const bool kept = width <= LN2_REGS * VEC * 256;
+    float x[LN2_REGS][VEC];
+    auto read = [&](int c, float* v) {
+        load_floats<VEC>(h + row + c, v);
+        float a[VEC], b[VEC];
+        if (d1 != nullptr) load_elems<VEC>(d1 + row + c, a);
+        if (d2 != nullptr) load_elems<VEC>(d2 + row + c, b);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e)
+            if (d1 != nullptr || d2 != nullptr) v[e] += d2 == nullptr ? a[e] : d1 == nullptr ? b[e] : a[e] + b[e];
+    };
+    float sum = 0.f;
+    auto first = [&](int c, float* v) {
+        read(c, v);
+        if (d1 != nullptr || d2 != nullptr) store_floats<VEC>(h + row + c, v);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) sum += v[e];
+    };
+    if (kept) {
+#pragma unroll
+        for (int j = 0; j < LN2_REGS; ++j) {
+            const int c = (threadIdx.x + j * 256) * VEC;
+            if (c < width) first(c, x[j]);
+        }
+    } else {
+        for (int c = threadIdx.x * VEC; c < width; c += 256 * VEC) first(c, x[0]);
+    }
+    const float mean = block_sum(sum, scratch) / (float)width;
+    float dev = 0.f;
+    auto second = [&](const float* v) {
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) dev += (v[e] - mean) * (v[e] - mean);
+    };
+    if (kept) {
+#pragma unroll
+        for (int j = 0; j < LN2_REGS; ++j)
+            if ((int)(threadIdx.x + j * 256) * VEC < width) second(x[j]);
+    } else {
+        for (int c = threadIdx.x * VEC; c < width; c += 256 * VEC) {
+            load_floats<VEC>(h + row + c, x[0]);           // (this thread's own values: complete)
+            second(x[0]);
+        }
+    }
+    const float inv = 1.0f / sqrtf(block_sum(dev, scratch) / (float)width + eps);
+    auto third = [&](int c, const float* v) {
+        float w[VEC], y[VEC];
+        load_floats<VEC>(weight + c, w);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) y[e] = ((v[e] - mean) * inv) * w[e];
+        if (bias != nullptr) {
+            load_floats<VEC>(bias + c, w);
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) y[e] += w[e];
+        }
+        store_elems<VEC>(out + row + c, y);
+    };
+    if (kept) {
+#pragma unroll
+        for (int j = 0; j < LN2_REGS; ++j) {
+            const int c = (threadIdx.x + j * 256) * VEC;
+            if (c < width) third(c, x[j]);
+        }
+    } else {
+        for (int c = threadIdx.x * VEC; c < width; c += 256 * VEC) {
+            load_floats<VEC>(h + row + c, x[0]);
+            third(c, x[0]);
+        }
+    }
+}
+
+// out = T(h): the float residual stream as a sublayer's input.
+__global__ void cast_rows_kernel(const float* __restrict__ h, elem_t* __restrict__ out, size_t count) {
+    for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < count; i += (size_t)gridDim.x * blockDim.x)
+        out[i] = from_float<elem_t>(h[i]);
+}
+
+// x *= factor (float values, logits for instance).
+__global__ void scale_float_kernel(float* __restrict__ x, float factor, size_t count) {
+    for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < count; i += (size_t)gridDim.x * blockDim.x)
+        x[i] *= factor;
+}
+
+// ---- a norm without statistics: y = tanh(alpha x) w + b, element by element, 32-bit ---------------------------
+__device__ __forceinline__ float tanh_norm(float x, float alpha, float w, float b) { return __builtin_fmaf(tanhf(alpha * x), w, b); }
 
 // x = h[row] + delta[row] (delta may be null; written back to h when write_h), out[r] = norm(x) for row = rows[r]
 // (rows null: r).  One thread takes VEC consecutive elements (width a multiple of VEC).
@@ -875,10 +970,10 @@ template <class... P> static bool aligned16(P... pointers) {
 
 extern "C" {
 
-int mlr_embed_gather(const int32_t* ids, const void* table, float* h, int rows, int width, int vocab,
+int mlr_embed_gather(const int32_t* ids, const void* table, float* h, int rows, int width, int vocab, float scale,
                      hipStream_t stream) {
     if (rows <= 0) return 0;
-    embed_gather_kernel<<<rows, 256, 0, stream>>>(ids, (const elem_t*)table, h, width, vocab);
+    embed_gather_kernel<<<rows, 256, 0, stream>>>(ids, (const elem_t*)table, h, width, vocab, scale);
     return (int)hipGetLastError();
 }
 
@@ -1051,9 +1146,32 @@ int mlr_layernorm(const void* xe, const float* xf, const float* weight, const fl
     return (int)hipGetLastError();
 }
 
-int mlr_relu_squared(const void* x, void* out, size_t count, hipStream_t stream) {
+int mlr_plain_act(const void* x, void* out, size_t count, int act, hipStream_t stream) {
     if (count == 0) return 0;
-    relu_squared_kernel<<<grid_for(count, 256), 256, 0, stream>>>((const elem_t*)x, (elem_t*)out, count);
+    if (act < 0 || act > 1) return -1;
+    const bool vec = count % MLR_VEC == 0 && aligned16(x, out);
+    const size_t n = vec ? count / MLR_VEC : count;
+#define MLR_PLAIN_ACT(ACT)                                                                                              \
+    if (vec) plain_act_kernel<ACT, MLR_VEC><<<grid_for(n, 256), 256, 0, stream>>>((const elem_t*)x, (elem_t*)out, n);    \
+    else plain_act_kernel<ACT, 1><<<grid_for(n, 256), 256, 0, stream>>>((const elem_t*)x, (elem_t*)out, n);
+    if (act == 0) {
+        MLR_PLAIN_ACT(0)
+    } else {
+        MLR_PLAIN_ACT(1)
+    }
+#undef MLR_PLAIN_ACT
+    return (int)hipGetLastError();
+}
+
+int mlr_add2_layernorm(float* h, const void* d1, const void* d2, const float* weight, const float* bias, void* out, int rows,
+                       int width, float eps, hipStream_t stream) {
+    if (rows <= 0) return 0;
+    if (width % 4 == 0 && aligned16(h, d1, d2, weight, bias, out))
+        add2_layernorm_kernel<4><<<rows, 256, 0, stream>>>(h, (const elem_t*)d1, (const elem_t*)d2, weight, bias,
+                                                           (elem_t*)out, width, eps);
+    else
+        add2_layernorm_kernel<1><<<rows, 256, 0, stream>>>(h, (const elem_t*)d1, (const elem_t*)d2, weight, bias,
+                                                           (elem_t*)out, width, eps);
     return (int)hipGetLastError();
 }
 

@@ -6,14 +6,15 @@
 //     out + g * out_group with row strides lda / ldo: one projection per head on slices of wider rows;
 //   offsets != null: group g takes the rows offsets[g] .. offsets[g + 1] - 1 of a list sorted by group (rows of
 //     out; a's row is gather[row] when gather != null): the experts of a routed feed-forward.
-// act: none, or relu(x)^2.  Every output element is one sum over k in ascending order whatever rows lie beside
+// act: none, relu(x)^2, the exact gelu, or one of the gated forms.  Every output element is one sum over k in ascending order whatever rows lie beside
 // it, so a row's result does not depend on the batch.  Accumulation is 32-bit; the bfloat16 engine multiplies on
 // the matrix cores (v_mfma_f32_16x16x32_bf16, operands staged through LDS), the float engine with plain FMAs.
 //
-// Routing (32-bit): `router_topk_kernel` (sigmoid of a token's router logits, the best groups of neighbouring
+// Routing (32-bit): `router_topk_kernel` (sigmoid or softmax of a token's router logits, the best groups of neighbouring
 // experts, the best experts within them), `route_sort_kernel` (the chosen (token, expert) pairs
 // sorted by expert: offsets, the token of every sorted row, the sorted row of every pair),
-// `route_combine_kernel` (a token's output: the weighted sum of its experts' rows, in the order of its choices).
+// `route_combine_kernel` (a token's output: the weighted sum of its experts' rows, in the order of its choices, and what
+// a shared expert gave).
 #include "common.h"
 
 #define ACT_NONE 0
@@ -22,6 +23,9 @@
 // matching 16 of the other ([gate 0..15 | up 0..15 | gate 16..31 | ...]); out[m, f] = act(gate_f) * up_f, N / 2 columns
 #define ACT_GATED_SILU 2
 #define ACT_GATED_GELU_TANH 3
+// the clamped gate: g = min(gate, limit), u = clamp(up, -limit, limit), out = g sigmoid(slope g) (u + 1)
+#define ACT_GATED_CLAMPED 4
+#define ACT_GELU_ERF 5
 
 struct GroupedArgs {
     const elem_t* a; long lda; long a_group;
@@ -29,7 +33,9 @@ struct GroupedArgs {
     void* out; long ldo; long out_group;
     const int32_t* offsets; const int32_t* gather;
     int M, N, K, groups, act, out_float;
+    float limit, slope;                        // of the clamped gate
 };
+__host__ __device__ inline bool gated_form(int act) { return act >= ACT_GATED_SILU && act <= ACT_GATED_CLAMPED; }
 
 #define GBM 64              // rows and columns of the small workgroup tile (the float engine's only one)
 #define GBN 64
@@ -63,12 +69,18 @@ __device__ __forceinline__ float activate(float x, int act) {
         const float r = fmaxf(x, 0.f);
         return r * r;
     }
+    if (act == ACT_GELU_ERF) return 0.5f * x * (1.0f + erff(x * 0.70710678118654752440f));
     return x;
 }
 
-__device__ __forceinline__ float gate_act(float g, int act) {
-    if (act == ACT_GATED_SILU) return g / (1.0f + expf(-g));
-    return 0.5f * g * (1.0f + tanhf(0.79788456080286535588f * (g + 0.044715f * g * g * g)));
+__device__ __forceinline__ float gated(float g, float u, const GroupedArgs& a) {
+    if (a.act == ACT_GATED_SILU) return g / (1.0f + expf(-g)) * u;
+    if (a.act == ACT_GATED_CLAMPED) {
+        g = fminf(g, a.limit);
+        u = fminf(fmaxf(u, -a.limit), a.limit);
+        return g / (1.0f + expf(-a.slope * g)) * (u + 1.0f);
+    }
+    return u * 0.5f * g * (1.0f + tanhf(0.79788456080286535588f * (g + 0.044715f * g * g * g)));
 }
 
 #if !MLR_BF16
@@ -213,7 +225,7 @@ __global__ __launch_bounds__(256) void grouped_gemm_kernel(GroupedArgs g) {
         __syncthreads();
     }
     // accumulator element r of a lane: row (lane / 16) * 4 + r, column lane % 16
-    if (g.act >= ACT_GATED_SILU) {
+    if (gated_form(g.act)) {
         // a wavefront's neighbouring column tiles hold a gate block and its up block: half as many columns leave
 #pragma unroll
         for (int i = 0; i < T; ++i) {
@@ -225,7 +237,7 @@ __global__ __launch_bounds__(256) void grouped_gemm_kernel(GroupedArgs g) {
                 for (int r = 0; r < 4; ++r) {
                     const int m = m0 + (wm * T + i) * 16 + (lane >> 4) * 4 + r;
                     if (m >= m_end) continue;
-                    const float y = gate_act(acc[i][j][r], g.act) * acc[i][j + 1][r];
+                    const float y = gated(acc[i][j][r], acc[i][j + 1][r], g);
                     const size_t at = out_base + (size_t)m * g.ldo + n;
                     if (g.out_float) ((float*)g.out)[at] = y;
                     else ((__bf16*)g.out)[at] = (__bf16)y;
@@ -271,23 +283,34 @@ __device__ __forceinline__ void wave_best(float& value, int& index) {
     }
 }
 
-// One wavefront a token.  s = sigmoid(z), z[m] the token's router logits (float: a product of the framework's own,
-// 32-bit sums).  The experts form `group_count`
+// One wavefront a token.  s = sigmoid(z), or softmax(z) over all experts (`softmax`), z[m * ld ..] the token's router
+// logits (float: a product of the framework's own, 32-bit sums).  The experts form `group_count`
 // equal groups of neighbours; a group's score is the sum of its two largest s (of its only one, when a group is
-// one expert); only experts of the `group_keep` best groups stand; of those the `top` largest s are chosen
+// one expert), or its largest (`group_best`); only experts of the `group_keep` best groups stand; of those the `top` largest s are chosen
 // (ties: the lower index), ids[m][i] in descending order of s with weights[m][i] = s itself.
 // With `correction` [experts] the choice (of groups and of experts) goes by s + correction while the weights stay
 // the plain s; with `renorm` the chosen weights are divided by their sum (+ 1e-20); `out_scale` multiplies them.
-__global__ __launch_bounds__(64) void router_topk_kernel(const float* __restrict__ z, int32_t* __restrict__ ids,
+__global__ __launch_bounds__(64) void router_topk_kernel(const float* __restrict__ z, long ld, int32_t* __restrict__ ids,
                                                          float* __restrict__ weights, int experts, int top,
                                                          int group_count, int group_keep,
-                                                         const float* __restrict__ correction, int renorm, float out_scale) {
+                                                         const float* __restrict__ correction, int renorm, float out_scale,
+                                                         int softmax, int group_best) {
     __shared__ float s_lds[MAX_EXPERTS];      // what the choice goes by
     __shared__ float w_lds[MAX_EXPERTS];      // the plain scores
     __shared__ float g_lds[MAX_EXPERTS];
     const int m = blockIdx.x, lane = threadIdx.x;
+    const float* zr = z + (size_t)m * ld;
+    float z_max = 0.f, z_sum = 1.f;
+    if (softmax) {
+        z_max = -INFINITY;
+        for (int e = lane; e < experts; e += 64) z_max = fmaxf(z_max, zr[e]);
+        z_max = wave_max(z_max);
+        z_sum = 0.f;
+        for (int e = lane; e < experts; e += 64) z_sum += expf(zr[e] - z_max);
+        z_sum = wave_sum(z_sum);
+    }
     for (int e = lane; e < experts; e += 64) {
-        const float sc = 1.0f / (1.0f + expf(-z[(size_t)m * experts + e]));
+        const float sc = softmax ? expf(zr[e] - z_max) / z_sum : 1.0f / (1.0f + expf(-zr[e]));
         w_lds[e] = sc;
         s_lds[e] = correction != nullptr ? sc + correction[e] : sc;
     }
@@ -304,7 +327,7 @@ __global__ __launch_bounds__(64) void router_topk_kernel(const float* __restrict
                 second = v;
             }
         }
-        g_lds[gidx] = per >= 2 ? first + second : first;
+        g_lds[gidx] = per >= 2 && !group_best ? first + second : first;
     }
     __syncthreads();
     // the groups that stand: group_keep times the best of those left; their experts become candidates
@@ -396,14 +419,40 @@ __global__ __launch_bounds__(1024) void route_sort_kernel(const int32_t* __restr
     }
 }
 
-// out[m, :] = sum_i weights[m][i] * y[row_of[m * top + i], :], the sum in 32-bit in the order of the choices.
+// out[m, :] = sum_i weights[m][i] * y[row_of[m * top + i], :], the sum in 32-bit in the order of the choices; with
+// `shared` [rows, width] plus shared[m, :], times sigmoid(shared_gate[m * gate_stride]) when that is given.
+// VEC: MLR_VEC values in one access, or 1.
+template <int VEC>
 __global__ void route_combine_kernel(const elem_t* __restrict__ y, const int32_t* __restrict__ row_of,
-                                     const float* __restrict__ weights, elem_t* __restrict__ out, int width, int top) {
+                                     const float* __restrict__ weights, elem_t* __restrict__ out, int width, int top,
+                                     const elem_t* __restrict__ shared, const float* __restrict__ shared_gate, long gate_stride) {
     const int m = blockIdx.x;
+    const float f = shared_gate != nullptr ? 1.0f / (1.0f + expf(-shared_gate[(size_t)m * gate_stride])) : 1.0f;
+    if (VEC > 1) {
+        for (int c = threadIdx.x * VEC; c < width; c += blockDim.x * VEC) {
+            float sum[MLR_VEC], v[MLR_VEC];
+#pragma unroll
+            for (int e = 0; e < MLR_VEC; ++e) sum[e] = 0.f;
+            for (int i = 0; i < top; ++i) {
+                const float w = weights[(size_t)m * top + i];
+                load_vec(y + (size_t)row_of[(size_t)m * top + i] * width + c, v);
+#pragma unroll
+                for (int e = 0; e < MLR_VEC; ++e) sum[e] = fmaf(w, v[e], sum[e]);
+            }
+            if (shared != nullptr) {
+                load_vec(shared + (size_t)m * width + c, v);
+#pragma unroll
+                for (int e = 0; e < MLR_VEC; ++e) sum[e] = fmaf(f, v[e], sum[e]);
+            }
+            store_vec(out + (size_t)m * width + c, sum);
+        }
+        return;
+    }
     for (int c = threadIdx.x; c < width; c += blockDim.x) {
         float sum = 0.f;
         for (int i = 0; i < top; ++i)
             sum = fmaf(weights[(size_t)m * top + i], to_float(y[(size_t)row_of[(size_t)m * top + i] * width + c]), sum);
+        if (shared != nullptr) sum = fmaf(f, to_float(shared[(size_t)m * width + c]), sum);
         out[(size_t)m * width + c] = from_float<elem_t>(sum);
     }
 }
@@ -412,17 +461,17 @@ extern "C" {
 
 int mlr_grouped_gemm(const void* a, long lda, long a_group, const void* w, long w_group, void* out, long ldo,
                      long out_group, const int32_t* offsets, const int32_t* gather, int M, int N, int K, int groups,
-                     int act, int out_float, hipStream_t stream) {
+                     int act, int out_float, float limit, float slope, hipStream_t stream) {
     if (M <= 0 || N <= 0 || groups <= 0) return 0;
-    if (K <= 0 || act < ACT_NONE || act > ACT_GATED_GELU_TANH) return -1;
+    if (K <= 0 || act < ACT_NONE || act > ACT_GELU_ERF || (act == ACT_GATED_CLAMPED && !(limit > 0.f))) return -1;
 #if !MLR_BF16
-    if (act >= ACT_GATED_SILU) return -3;            // (the gated forms are the matrix-core kernels')
+    if (gated_form(act)) return -3;            // (the gated forms are the matrix-core kernels')
     out_float = 1;
 #else
-    if (act >= ACT_GATED_SILU && N % 32 != 0) return -3;
+    if (gated_form(act) && N % 32 != 0) return -3;
 #endif
     GroupedArgs g{(const elem_t*)a, lda, a_group, (const elem_t*)w, w_group, out, ldo, out_group, offsets, gather,
-                  M, N, K, groups, act, out_float};
+                  M, N, K, groups, act, out_float, limit, slope};
 #if MLR_BF16
     // experts with many rows each: the large tile (310 -> 340 TFLOP/s at 2048 tokens of width 2048, 390 -> 420 at width
     // 4096; the products a head, with inner sizes of 128 to 512, are faster on the small one)
@@ -444,14 +493,15 @@ int mlr_grouped_gemm(const void* a, long lda, long a_group, const void* w, long 
     return (int)hipGetLastError();
 }
 
-int mlr_router_topk(const float* z, int32_t* ids, float* weights, int rows, int experts, int top, int group_count,
-                    int group_keep, const float* correction, int renorm, float out_scale, hipStream_t stream) {
+int mlr_router_topk(const float* z, long ld, int32_t* ids, float* weights, int rows, int experts, int top, int group_count,
+                    int group_keep, const float* correction, int renorm, float out_scale, int softmax, int group_best,
+                    hipStream_t stream) {
     if (rows <= 0) return 0;
-    if (experts < 1 || experts > MAX_EXPERTS || group_count < 1 || experts % group_count != 0 || group_keep < 1 ||
+    if (ld < experts || experts < 1 || experts > MAX_EXPERTS || group_count < 1 || experts % group_count != 0 || group_keep < 1 ||
         group_keep > group_count || top < 1 || top > group_keep * (experts / group_count))
         return -1;
-    router_topk_kernel<<<rows, 64, 0, stream>>>(z, ids, weights, experts, top, group_count, group_keep, correction, renorm,
-                                                out_scale);
+    router_topk_kernel<<<rows, 64, 0, stream>>>(z, ld, ids, weights, experts, top, group_count, group_keep, correction, renorm,
+                                                out_scale, softmax, group_best);
     return (int)hipGetLastError();
 }
 
@@ -464,9 +514,16 @@ int mlr_route_sort(const int32_t* ids, int pairs, int top, int experts, int32_t*
 }
 
 int mlr_route_combine(const void* y, const int32_t* row_of, const float* weights, void* out, int rows, int width,
-                      int top, hipStream_t stream) {
+                      int top, const void* shared, const float* shared_gate, long gate_stride, hipStream_t stream) {
     if (rows <= 0) return 0;
-    route_combine_kernel<<<rows, 256, 0, stream>>>((const elem_t*)y, row_of, weights, (elem_t*)out, width, top);
+    const bool vec = width % MLR_VEC == 0 && ((reinterpret_cast<uintptr_t>(y) | reinterpret_cast<uintptr_t>(out) |
+                                              reinterpret_cast<uintptr_t>(shared)) & 15) == 0;
+    if (vec)
+        route_combine_kernel<MLR_VEC><<<rows, 256, 0, stream>>>((const elem_t*)y, row_of, weights, (elem_t*)out, width, top,
+                                                                (const elem_t*)shared, shared_gate, gate_stride);
+    else
+        route_combine_kernel<1><<<rows, 256, 0, stream>>>((const elem_t*)y, row_of, weights, (elem_t*)out, width, top,
+                                                          (const elem_t*)shared, shared_gate, gate_stride);
     return (int)hipGetLastError();
 }
 

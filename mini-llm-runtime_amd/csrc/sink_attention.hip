@@ -142,7 +142,9 @@ __global__ __launch_bounds__(64) void sink_attention_kernel(SinkArgs a) {
 // heads; null: no weight) before the rotation (norm_mode 1), after it (norm_mode 2) or not at all (0); the first
 // rot_dim channels of a head turned by the token's position with cos = table[p][j], sin = table[p][rot_dim / 2 + j]
 // in pairs (j, j + rot_dim / 2) or, `interleaved`, (2 j, 2 j + 1) (table null: no rotation);
-// q to q_out [m, q_heads * key_dim], k and v into their pages.  One wavefront a head; 32-bit throughout.
+// q to q_out [m, q_heads * key_dim], k and v into their pages.  v_rope, when given, turns ALL channels of a value head by
+// the token's position (its table is value_dim wide, pairs as v_interleaved says); v_transposed: value pages lie
+// [page][kv_head][channel][place] instead of row by row.  One wavefront a head; 32-bit throughout.
 __device__ __forceinline__ float turned_channel(const float* x, int d, const float* cs, int rot_dim, int interleaved) {
     if (cs == nullptr || d >= rot_dim) return x[d];
     const int half = rot_dim >> 1;
@@ -162,7 +164,8 @@ __global__ __launch_bounds__(64) void sink_qkv_prep_kernel(
     const int32_t* __restrict__ block_table, int max_blocks, const int32_t* __restrict__ slots,
     const int32_t* __restrict__ positions, const float* __restrict__ q_norm_w, const float* __restrict__ k_norm_w,
     float eps, const float* __restrict__ rope, int rot_dim, int q_heads, int kv_heads, int key_dim, int value_dim,
-    int page_size, int write_cache, int norm_mode, int interleaved) {
+    int page_size, int write_cache, int norm_mode, int interleaved, const float* __restrict__ v_rope, int v_interleaved,
+    int v_transposed) {
     __shared__ float x_lds[MAX_KEY_DIM];
     const int m = blockIdx.x, unit = blockIdx.y, lane = threadIdx.x;
     const int pos = positions[m], slot = slots[m];
@@ -175,11 +178,23 @@ __global__ __launch_bounds__(64) void sink_qkv_prep_kernel(
         const int kvh = unit < q_heads + kv_heads ? unit - q_heads : unit - q_heads - kv_heads;
         cache_row = ((long long)page * kv_heads + kvh) * page_size + pos % page_size;
     }
-    if (unit >= q_heads + kv_heads) {          // a value head: bias, into its page
+    if (unit >= q_heads + kv_heads) {          // a value head: bias, turn, into its page
         const long off = (long)(q_heads + kv_heads) * key_dim + (long)(unit - q_heads - kv_heads) * value_dim;
+        // (transposed: the head's block of a page starts where row-major rows of value_dim channels would)
+        const int place = pos % page_size;
+        elem_t* dst = v_transposed ? v_pages + (cache_row - place) * value_dim + place : v_pages + cache_row * v_row;
+        const long step = v_transposed ? page_size : 1;
+        const float* vcs = v_rope ? v_rope + (size_t)pos * value_dim : nullptr;
+        if (vcs != nullptr) {
+            for (int c = lane; c < value_dim; c += 64)
+                x_lds[c] = to_float(proj[(size_t)m * ld + off + c]) + (bias ? bias[off + c] : 0.f);
+            __syncthreads();
+            for (int c = lane; c < value_dim; c += 64)
+                dst[c * step] = from_float<elem_t>(turned_channel(x_lds, c, vcs, value_dim, v_interleaved));
+            return;
+        }
         for (int c = lane; c < value_dim; c += 64)
-            v_pages[cache_row * v_row + c] =
-                from_float<elem_t>(to_float(proj[(size_t)m * ld + off + c]) + (bias ? bias[off + c] : 0.f));
+            dst[c * step] = from_float<elem_t>(to_float(proj[(size_t)m * ld + off + c]) + (bias ? bias[off + c] : 0.f));
         return;
     }
     const long off = (long)unit * key_dim;
@@ -591,15 +606,16 @@ int mlr_sink_qkv_prep(const void* proj, long ld, const float* bias, void* q_out,
                       void* v_pages, long v_row, const int32_t* block_table, int max_blocks, const int32_t* slots,
                       const int32_t* positions, const float* q_norm_w, const float* k_norm_w, float eps,
                       const float* rope, int rot_dim, int rows, int q_heads, int kv_heads, int key_dim, int value_dim,
-                      int page_size, int write_cache, int norm_mode, int interleaved, hipStream_t stream) {
+                      int page_size, int write_cache, int norm_mode, int interleaved, const float* v_rope, int v_interleaved,
+                      int v_transposed, hipStream_t stream) {
     if (rows <= 0) return 0;
-    if (key_dim > MAX_KEY_DIM || q_heads + 2 * kv_heads > 65535 || rot_dim > key_dim || (rot_dim & 1) || norm_mode < 0 ||
+    if ((v_rope != nullptr && (value_dim > MAX_KEY_DIM || (value_dim & 1))) || key_dim > MAX_KEY_DIM || q_heads + 2 * kv_heads > 65535 || rot_dim > key_dim || (rot_dim & 1) || norm_mode < 0 ||
         norm_mode > 2)
         return -1;
     sink_qkv_prep_kernel<<<dim3(rows, q_heads + 2 * kv_heads), 64, 0, stream>>>(
         (const elem_t*)proj, ld, bias, (elem_t*)q_out, (elem_t*)k_pages, k_row, (elem_t*)v_pages, v_row, block_table,
         max_blocks, slots, positions, q_norm_w, k_norm_w, eps, rope, rot_dim, q_heads, kv_heads, key_dim, value_dim,
-        page_size, write_cache, norm_mode, interleaved);
+        page_size, write_cache, norm_mode, interleaved, v_rope, v_interleaved, v_transposed);
     return (int)hipGetLastError();
 }
 

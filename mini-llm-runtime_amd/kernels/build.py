@@ -45,6 +45,7 @@ HIP_LIBRARIES = {
     "recurrence": (["recurrence.hip"], ["common.h"], True),
     "diff_attention": (["diff_attention.hip"], ["common.h"], True),
     "sink_attention": (["sink_attention.hip"], ["common.h"], True),
+    "head_mix_attention": (["head_mix_attention.hip"], ["common.h"], True),
     "grouped_gemm": (["grouped_gemm.hip"], ["common.h"], True),
     "attention_tiles": (["attention_tiles.hip"], [], False),      # bfloat16 only by nature
     "sampling": (["sampling.hip"], ["no_alloc.h"], False),

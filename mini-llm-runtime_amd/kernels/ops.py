@@ -111,7 +111,7 @@ def _norm_work(self, h, delta, weight, out, eps, rows=None, write_h=True):
     return moved, 0
 
 
-def _embed_work(self, ids, table, h):
+def _embed_work(self, ids, table, h, scale=1.0):
     return _size(h) + h.numel() * table.element_size(), 0
 
 
@@ -157,15 +157,15 @@ class Kernels:
 
     # -- row-wise ----------------------------------------------------------------------------
     @timed("embed", _embed_work)
-    def embed_gather(self, ids, table, h):
-        """h[m] = float(table[ids[m]])."""
+    def embed_gather(self, ids, table, h, scale=1.0):
+        """h[m] = float(table[ids[m]]) * scale."""
         rows = ids.numel()
         _tensor(ids, "ids", torch.int32, ndim=1)
         _tensor(table, "table", self.dtype, ndim=2)
         vocab, width = table.shape
         _tensor(h, "h", torch.float32, (rows, width))
         fn = self._lib("elementwise").mlr_embed_gather
-        _ok(fn(_p(ids), _p(table), _p(h), _c_int(rows), _c_int(width), _c_int(vocab), _stream()),
+        _ok(fn(_p(ids), _p(table), _p(h), _c_int(rows), _c_int(width), _c_int(vocab), _c_float(scale), _stream()),
             "embed_gather")
 
     @timed("norm", _norm_work)
@@ -1221,6 +1221,21 @@ class Kernels:
                                                    _stream()), "layernorm_add")
 
     @timed("norm", _tensors_work())
+    def add2_layernorm(self, h, d1, d2, weight, bias, out, eps):
+        """x = h + (d1 + d2) (either may be None), written back to h when one is given; out = layernorm(x) * weight (+ bias)."""
+        _tensor(h, "h", torch.float32, ndim=2)
+        m, width = h.shape
+        for name, d in (("d1", d1), ("d2", d2)):
+            if d is not None:
+                _tensor(d, name, self.dtype, (m, width))
+        _tensor(weight, "weight", torch.float32, (width,))
+        if bias is not None:
+            _tensor(bias, "bias", torch.float32, (width,))
+        _tensor(out, "out", self.dtype, (m, width))
+        _ok(self._lib("elementwise").mlr_add2_layernorm(_p(h), _p(d1), _p(d2), _p(weight), _p(bias), _p(out), _c_int(m),
+                                                        _c_int(width), _c_float(eps), _stream()), "add2_layernorm")
+
+    @timed("norm", _tensors_work())
     def tanh_norm_rows(self, h, delta, weight, bias, alpha, out, rows=None, write_h=True):
         """x = h + delta (delta may be None; written back to h when write_h); out[r] = T(tanh(alpha x[rows[r] or r]) *
         weight + bias): a norm that takes no statistics, element by element in 32-bit."""
@@ -1305,12 +1320,21 @@ class Kernels:
                                                    _p(out), _c_int(n_out), _c_int(width), _c_float(eps),
                                                    _c_float(out_scale), _stream()), "layernorm_rows")
 
+    PLAIN_ACTS = {"relu_squared": 0, "gelu_erf": 1}
+
     @timed("activation", _tensors_work())
-    def relu_squared(self, x, out):
-        """out = max(x, 0)^2 (x and out may be the same tensor)."""
+    def plain_act(self, x, out, kind):
+        """out = act(x), element by element (x and out may be the same tensor): "relu_squared" max(x, 0)^2, "gelu_erf"
+        x Phi(x) with the normal distribution's function."""
+        _need(kind in self.PLAIN_ACTS, f"plain_act: activation {kind!r}")
         _tensor(x, "x", self.dtype)
         _tensor(out, "out", self.dtype, tuple(x.shape))
-        _ok(self._lib("elementwise").mlr_relu_squared(_p(x), _p(out), _c_size_t(x.numel()), _stream()), "relu_squared")
+        _ok(self._lib("elementwise").mlr_plain_act(_p(x), _p(out), _c_size_t(x.numel()), _c_int(self.PLAIN_ACTS[kind]),
+                                                   _stream()), "plain_act")
+
+    def relu_squared(self, x, out):
+        """out = max(x, 0)^2 (x and out may be the same tensor)."""
+        self.plain_act(x, out, "relu_squared")
 
     @timed("norm", _tensors_work())
     def cast_rows(self, h, out):
@@ -1341,12 +1365,14 @@ class Kernels:
     @timed("rope_kv", _rope_work)
     def sink_qkv_prep(self, proj, bias, q_out, k_pages, v_pages, block_table, slots, positions, q_norm_w, k_norm_w, eps,
                       rope, q_heads, kv_heads, key_dim, value_dim, page_size, write_cache=True, norm="auto",
-                      interleaved=False):
+                      interleaved=False, v_rope=None, v_interleaved=False, v_transposed=False):
         """From the stacked projection [rows, q_heads * key_dim + kv_heads * (key_dim + value_dim)] (further columns behind these are left alone): bias (float, may be
         None), per-head RMSNorm of q and k, rotation of a head's first rope.shape[1] channels in pairs (j, j + half)
         or, `interleaved`, (2 j, 2 j + 1) (rope float [positions, rot]: cosines | sines; may be None); q to q_out, k
         and v into their row-major pages.  `norm`: "before" the rotation, "after" it, None, or "auto" (before it when
-        weights are given, else none); the weights may be None with any of them (a norm without a weight)."""
+        weights are given, else none); the weights may be None with any of them (a norm without a weight).  `v_rope`
+        (float [positions, value_dim], may be None) turns whole value heads by their position; `v_transposed`: value
+        pages lie [pages, kv_heads, value_dim, page]."""
         total = q_heads * key_dim + kv_heads * (key_dim + value_dim)
         _tensor(proj, "proj", self.dtype, ndim=2)
         rows = proj.shape[0]
@@ -1356,7 +1382,15 @@ class Kernels:
         _tensor(q_out, "q_out", self.dtype, (rows, q_heads * key_dim))
         _need(1 <= key_dim <= self.SINK_MAX_KEY_DIM, f"key_dim {key_dim}: up to {self.SINK_MAX_KEY_DIM}")
         k_row = self._sink_pages(k_pages, "k_pages", kv_heads, page_size, key_dim)
-        v_row = self._sink_pages(v_pages, "v_pages", kv_heads, page_size, value_dim)
+        if v_transposed:
+            _tensor(v_pages, "v_pages", self.dtype, (v_pages.shape[0], kv_heads, value_dim, page_size))
+            v_row = value_dim
+        else:
+            v_row = self._sink_pages(v_pages, "v_pages", kv_heads, page_size, value_dim)
+        if v_rope is not None:
+            _tensor(v_rope, "v_rope", torch.float32, ndim=2)
+            _need(v_rope.shape[1] == value_dim and value_dim % 2 == 0 and value_dim <= self.SINK_MAX_KEY_DIM,
+                  lambda: f"v_rope: expected a width of {value_dim} (even, up to {self.SINK_MAX_KEY_DIM})")
         _tensor(block_table, "block_table", torch.int32, ndim=2)
         _tensor(slots, "slots", torch.int32, (rows,))
         _tensor(positions, "positions", torch.int32, (rows,))
@@ -1377,7 +1411,8 @@ class Kernels:
             ctypes.c_long(v_row), _p(block_table), _c_int(block_table.shape[1]), _p(slots), _p(positions), _p(q_norm_w),
             _p(k_norm_w), _c_float(eps), _p(rope), _c_int(rot), _c_int(rows), _c_int(q_heads), _c_int(kv_heads),
             _c_int(key_dim), _c_int(value_dim), _c_int(page_size), _c_int(1 if write_cache else 0), _c_int(mode),
-            _c_int(1 if interleaved else 0), _stream()), "sink_qkv_prep")
+            _c_int(1 if interleaved else 0), _p(v_rope), _c_int(1 if v_interleaved else 0), _c_int(1 if v_transposed else 0),
+            _stream()), "sink_qkv_prep")
 
     @timed("rope_kv", _rope_work)
     def latent_prep(self, proj, q_out, pages, block_table, slots, positions, norm_w, eps, rope, heads, dim, rot, rank,
@@ -1512,13 +1547,119 @@ class Kernels:
         """Floats that the shares of `splits` key ranges take for `groups` groups of up to `tokens` tokens."""
         return groups * tokens * q_heads * splits * (value_dim + 4)
 
+    # -- attention whose heads' weights are mixed ------------------------------------------------
+    HEAD_MIX_MAX_CAP = 60.0       # of the scores: the matrix-core form takes exp(score) without a running maximum
+
+    def _head_mix_operands(self, q, k_pages, v_pages, block_table, slots, positions, mix, sink, v_rope, gate, out, q_heads,
+                           kv_heads, key_dim, value_dim, page_size):
+        """The arguments both forms share, checked, in the order the kernels take them up to the output."""
+        _tensor(q, "q", self.dtype, ndim=2)
+        rows = q.shape[0]
+        _need(q.shape[1] == q_heads * key_dim, "q: wrong width")
+        _need(kv_heads >= 1 and q_heads % kv_heads == 0, "q_heads must be a multiple of kv_heads")
+        _tensor(k_pages, "k_pages", self.dtype, (k_pages.shape[0], kv_heads, page_size, key_dim))
+        _tensor(v_pages, "v_pages", self.dtype, (k_pages.shape[0], kv_heads, value_dim, page_size))
+        _tensor(block_table, "block_table", torch.int32, ndim=2)
+        _tensor(slots, "slots", torch.int32, (rows,))
+        _tensor(positions, "positions", torch.int32, (rows,))
+        _tensor(mix, "mix", torch.float32, (q_heads, q_heads))
+        kind, value = 0, 0.0
+        if isinstance(sink, torch.Tensor):
+            kind = 2
+            _tensor(sink, "sink", torch.float32, (q_heads,))
+        elif sink is not None:
+            kind, value = 1, float(sink)
+        table, interleaved = v_rope if v_rope is not None else (None, False)
+        if table is not None:
+            _tensor(table, "v_rope", torch.float32, ndim=2)
+            _need(table.shape[1] == value_dim and value_dim % 2 == 0, "v_rope: as wide as a value, which is even")
+        gate_stride = self._columns(gate, "gate", self.dtype, rows, q_heads) if gate is not None else 0
+        _tensor(out, "out", self.dtype, (rows, q_heads * value_dim))
+        return (_p(q), ctypes.c_long(q.shape[1]), _p(k_pages), _p(v_pages), _p(block_table), _c_int(block_table.shape[1]),
+                _p(slots), _p(positions), _p(mix), _p(sink if kind == 2 else None), _c_float(value), _c_int(kind), _p(table),
+                _c_int(1 if interleaved else 0), _p(gate), ctypes.c_long(gate_stride), _p(out), ctypes.c_long(out.shape[1]))
+
+    @timed("attention")
+    def head_mix_attention(self, q, k_pages, v_pages, block_table, slots, positions, mix, sink, v_rope, gate, out, q_heads,
+                           kv_heads, key_dim, value_dim, page_size, scale, softcap=None):
+        """Causal attention with head h's softmax weights replaced by sum_g mix[h, g] weights_g before they meet the
+        values of h's own kv head.  `sink`: None, a number (one more summand exp(number) in every denominator) or a
+        float tensor with one a head; `softcap`: scores <- softcap tanh(scores / softcap); `v_rope` (table float
+        [positions, value_dim], interleaved): every head's output is turned back by the query's position; `gate`
+        (columns [rows, q_heads]): head h's output times sigmoid(gate[:, h]).  Values lie transposed within a page.
+        A workgroup a token; a token's sums follow from its own position alone."""
+        args = self._head_mix_operands(q, k_pages, v_pages, block_table, slots, positions, mix, sink, v_rope, gate, out,
+                                       q_heads, kv_heads, key_dim, value_dim, page_size)
+        _need((2 * q_heads * 64 + q_heads * value_dim + 2 * q_heads) * 4 <= 150 * 1024,
+              f"head_mix_attention: {q_heads} heads of {value_dim} value channels do not fit the workgroup's memory")
+        _ok(self._lib("head_mix_attention").mlr_head_mix_attention(
+            *args, _c_int(q.shape[0]), _c_int(q_heads), _c_int(kv_heads), _c_int(key_dim), _c_int(value_dim),
+            _c_int(page_size), _c_float(scale), _c_float(softcap or 0.0), _stream()), "head_mix_attention")
+
+    @staticmethod
+    def head_mix_layout(q_heads, kv_heads, value_dim):
+        """(places a kv head's query heads take: a power of two; inner size of the product that mixes the heads; the most
+        kv heads a workgroup of the second launch takes), or None where the matrix-core form does not take the sizes."""
+        pad = 1
+        while pad < q_heads // kv_heads:
+            pad *= 2
+        inner = 16 if kv_heads * pad <= 16 else -(-kv_heads * pad // 32) * 32
+        if pad > 32 or inner > 128 or inner % pad != 0 or value_dim % 16 != 0:
+            return None
+        for block in (8, 4, 2, 1):                 # (sums in registers: column tiles x value tiles of a wavefront)
+            if block * pad <= 32 and pad * -(-(value_dim // 16) // (8 // block)) <= 32:
+                return pad, inner, block
+        return None
+
+    def head_mix_tiles_supported(self, q_heads, kv_heads, key_dim, value_dim, page_size, softcap):
+        """Whether the matrix-core form takes these sizes: the bfloat16 engine, keys in multiples of 8 channels up to 256,
+        values in multiples of 16, pages in multiples of 8 places, capped scores, up to 32 query heads a kv head and 128
+        heads in their padded order."""
+        return (self.dtype == torch.bfloat16 and key_dim % 8 == 0 and key_dim <= 256 and page_size % 8 == 0
+                and softcap is not None and 0.0 < softcap <= self.HEAD_MIX_MAX_CAP
+                and self.head_mix_layout(q_heads, kv_heads, value_dim) is not None)
+
+    @timed("attention")
+    def head_mix_tiles(self, q, k_pages, v_pages, block_table, slots, positions, mix, sink, v_rope, gate, out, group_first,
+                       group_count, groups, group_tokens, q_heads, kv_heads, key_dim, value_dim, page_size, scale, softcap,
+                       e, sums, partial, ktiles, score_keys, score_ranges, value_keys, value_ranges, kv_block):
+        """`head_mix_attention` on the matrix cores for `groups` groups of up to `group_tokens` (16 or 1) consecutive tokens
+        of one request each; `ktiles` tiles of 32 keys hold the longest context, and the ranges (score_keys x
+        score_ranges, value_keys x value_ranges) too.  Scratch: e (elements of the engine's type) groups * group_tokens *
+        ktiles * 32 * inner, sums (float) groups * group_tokens * inner * score_ranges, partial (float) groups *
+        group_tokens * q_heads * value_ranges * value_dim, inner as `head_mix_layout` says."""
+        _need(self.head_mix_tiles_supported(q_heads, kv_heads, key_dim, value_dim, page_size, softcap),
+              "head_mix_tiles: sizes that the matrix-core form does not take")
+        args = self._head_mix_operands(q, k_pages, v_pages, block_table, slots, positions, mix, sink, v_rope, gate, out,
+                                       q_heads, kv_heads, key_dim, value_dim, page_size)
+        pad, inner, most = self.head_mix_layout(q_heads, kv_heads, value_dim)
+        _tensor(group_first, "group_first", torch.int32, ndim=1)
+        _tensor(group_count, "group_count", torch.int32, ndim=1)
+        _need(group_first.numel() >= groups and group_count.numel() >= groups, "group vectors too short")
+        _need(group_tokens in (1, 16) and kv_block in (1, 2, 4, 8) and kv_block <= most, "head_mix_tiles: launch shape")
+        keys = ktiles * 32
+        _need(score_keys % 32 == 0 and value_keys % (256 if group_tokens == 1 else 32) == 0 and score_keys * score_ranges >= keys
+              and value_keys * value_ranges >= keys, "head_mix_tiles: key ranges that do not hold the context")
+        rows = groups * group_tokens
+        _tensor(e, "e", self.dtype, ndim=1)
+        _tensor(sums, "sums", torch.float32, ndim=1)
+        _tensor(partial, "partial", torch.float32, ndim=1)
+        _need(e.numel() >= rows * keys * inner and sums.numel() >= rows * inner * score_ranges
+              and partial.numel() >= rows * q_heads * value_ranges * value_dim, "head_mix_tiles: scratch too small")
+        _ok(self._lib("head_mix_attention").mlr_head_mix_tiles(
+            *args, _p(group_first), _p(group_count), _c_int(groups), _c_int(group_tokens), _c_int(q_heads), _c_int(kv_heads),
+            _c_int(key_dim), _c_int(value_dim), _c_int(page_size), _c_float(scale), _c_float(softcap), _p(e), _p(sums),
+            _p(partial), _c_int(ktiles), _c_int(pad), _c_int(inner), _c_int(score_keys), _c_int(score_ranges),
+            _c_int(value_keys), _c_int(value_ranges), _c_int(kv_block), _stream()), "head_mix_tiles")
+
     # -- many small products, routing ----------------------------------------------------------
-    GROUPED_ACTS = {None: 0, "relu_squared": 1, "gated_silu": 2, "gated_gelu_tanh": 3}
+    GROUPED_ACTS = {None: 0, "relu_squared": 1, "gated_silu": 2, "gated_gelu_tanh": 3, "gated_clamped": 4, "gelu_erf": 5}
+    GROUPED_GATED = ("gated_silu", "gated_gelu_tanh", "gated_clamped")
 
     def experts_gated_fused(self, intermediate):
-        """Whether `experts_gemm` takes the gated forms (act "gated_silu" / "gated_gelu_tanh": the weight's rows are a
-        gate's and its up projection's in turn, 16 and 16; half as many columns leave): the bfloat16 engine, inner sizes
-        in multiples of 16."""
+        """Whether `experts_gemm` takes the gated forms (act "gated_silu" / "gated_gelu_tanh" / "gated_clamped": the weight's
+        rows are a gate's and its up projection's in turn, 16 and 16; half as many columns leave): the bfloat16 engine,
+        inner sizes in multiples of 16."""
         return self.dtype == torch.bfloat16 and intermediate % 16 == 0
     MAX_EXPERTS = 256
 
@@ -1533,24 +1674,26 @@ class Kernels:
         rows, groups, k = a.shape
         _need(w.shape[0] == groups and w.shape[2] == k and tuple(out.shape) == (rows, groups, w.shape[1]),
               "heads_gemm: shapes do not fit")
-        _need(act in self.GROUPED_ACTS, f"heads_gemm: activation {act!r}")
+        _need(act in self.GROUPED_ACTS and act not in self.GROUPED_GATED, f"heads_gemm: activation {act!r}")
         n = w.shape[1]
         _ok(self._lib("grouped_gemm").mlr_grouped_gemm(
             _p(a), ctypes.c_long(a.stride(0)), ctypes.c_long(a.stride(1)), _p(w), ctypes.c_long(n * k), _p(out),
             ctypes.c_long(out.stride(0)), ctypes.c_long(out.stride(1)), _ptr(0), _ptr(0), _c_int(rows), _c_int(n), _c_int(k),
-            _c_int(groups), _c_int(self.GROUPED_ACTS[act]), _c_int(0), _stream()), "heads_gemm")
+            _c_int(groups), _c_int(self.GROUPED_ACTS[act]), _c_int(0), _c_float(0.0), _c_float(0.0), _stream()), "heads_gemm")
 
     @timed("gemm")
-    def experts_gemm(self, a, w, out, offsets, gather=None, act=None):
+    def experts_gemm(self, a, w, out, offsets, gather=None, act=None, limit=0.0, slope=0.0):
         """Rows sorted by expert: out[r] = act(a[gather[r] or r] . w[e]^T) for offsets[e] <= r < offsets[e + 1];
-        a [*, K], w [experts, N, K], out [rows, N], offsets int32 [experts + 1] on the device."""
+        a [*, K], w [experts, N, K], out [rows, N], offsets int32 [experts + 1] on the device.  `limit` and `slope` are
+        the clamped gate's."""
         _tensor(a, "a", self.dtype, ndim=2)
         _tensor(w, "w", self.dtype, ndim=3)
         experts, n, k = w.shape
         _need(a.shape[1] == k, "experts_gemm: inner sizes differ")
         _tensor(out, "out", self.dtype, ndim=2)
         rows = out.shape[0]
-        gated = act in ("gated_silu", "gated_gelu_tanh")
+        gated = act in self.GROUPED_GATED
+        _need(act != "gated_clamped" or limit > 0, "experts_gemm: the clamped gate needs a positive limit")
         _need(not gated or (n % 32 == 0 and self.dtype == torch.bfloat16), "experts_gemm: the gated forms take bfloat16 and blocks of 16")
         _need(out.shape[1] == (n // 2 if gated else n), "experts_gemm: out has the wrong width")
         _tensor(offsets, "offsets", torch.int32, (experts + 1,))
@@ -1562,19 +1705,27 @@ class Kernels:
         _ok(self._lib("grouped_gemm").mlr_grouped_gemm(
             _p(a), ctypes.c_long(k), ctypes.c_long(0), _p(w), ctypes.c_long(n * k), _p(out), ctypes.c_long(out.shape[1]),
             ctypes.c_long(0), _p(offsets), _p(gather), _c_int(rows), _c_int(n), _c_int(k), _c_int(experts),
-            _c_int(self.GROUPED_ACTS[act]), _c_int(0), _stream()), "experts_gemm")
+            _c_int(self.GROUPED_ACTS[act]), _c_int(0), _c_float(limit), _c_float(slope), _stream()), "experts_gemm")
+
+    ROUTER_SCORES = {"sigmoid": 0, "softmax": 1}
+    ROUTER_GROUPS = {"best_two": 0, "best": 1}
 
     @timed("activation", _tensors_work())
-    def router_topk(self, logits, ids, weights, group_count=1, group_keep=1, correction=None, renormalize=False, scale=1.0):
-        """Per row of the router logits [rows, experts] (float): s = sigmoid(z); of the group_count equal groups of
-        neighbouring experts the group_keep with the largest sum of their two best s stay; ids [rows, top] int32 the
-        experts with the largest s among those, weights [rows, top] float their s.  With `correction` (float
-        [experts]) every choice goes by s + correction and the weights stay s; `renormalize`: the chosen weights over
-        their sum (+ 1e-20); `scale` multiplies them."""
-        if correction is not None:
-            _tensor(correction, "correction", torch.float32, (logits.shape[1],))
+    def router_topk(self, logits, ids, weights, group_count=1, group_keep=1, correction=None, renormalize=False, scale=1.0,
+                    score="sigmoid", group_score="best_two", experts=None):
+        """Per row of the router logits [rows, >= experts] (float; `experts` None: the whole width): s = sigmoid(z), or
+        softmax(z) over all experts; of the group_count equal groups of neighbouring experts the group_keep with the
+        largest sum of their two best s (`group_score` "best": the largest s) stay; ids [rows, top] int32 the experts with
+        the largest s among those, weights [rows, top] float their s.  With `correction` (float [experts]) every choice
+        goes by s + correction and the weights stay s; `renormalize`: the chosen weights over their sum (+ 1e-20);
+        `scale` multiplies them."""
         _tensor(logits, "logits", torch.float32, ndim=2)
-        rows, experts = logits.shape
+        rows, ld = logits.shape
+        experts = ld if experts is None else experts
+        _need(1 <= experts <= ld, "router_topk: more experts than logits")
+        _need(score in self.ROUTER_SCORES and group_score in self.ROUTER_GROUPS, f"router_topk: {score!r}, {group_score!r}")
+        if correction is not None:
+            _tensor(correction, "correction", torch.float32, (experts,))
         _tensor(ids, "ids", torch.int32, ndim=2)
         top = ids.shape[1]
         _need(ids.shape[0] == rows, "ids: one row a token")
@@ -1582,10 +1733,10 @@ class Kernels:
         _need(1 <= experts <= self.MAX_EXPERTS and group_count >= 1 and experts % group_count == 0
               and 1 <= group_keep <= group_count and 1 <= top <= group_keep * (experts // group_count),
               "router_topk: experts up to 256 in equal groups, and no more choices than the kept groups hold")
-        _ok(self._lib("grouped_gemm").mlr_router_topk(_p(logits), _p(ids), _p(weights), _c_int(rows), _c_int(experts),
-                                                      _c_int(top), _c_int(group_count), _c_int(group_keep), _p(correction),
-                                                      _c_int(1 if renormalize else 0), _c_float(scale), _stream()),
-            "router_topk")
+        _ok(self._lib("grouped_gemm").mlr_router_topk(
+            _p(logits), ctypes.c_long(ld), _p(ids), _p(weights), _c_int(rows), _c_int(experts), _c_int(top),
+            _c_int(group_count), _c_int(group_keep), _p(correction), _c_int(1 if renormalize else 0), _c_float(scale),
+            _c_int(self.ROUTER_SCORES[score]), _c_int(self.ROUTER_GROUPS[group_score]), _stream()), "router_topk")
 
     @timed("gemm")
     def route_sort(self, ids, experts, offsets, token_of, row_of):
@@ -1601,16 +1752,22 @@ class Kernels:
                                                      _p(offsets), _p(token_of), _p(row_of), _stream()), "route_sort")
 
     @timed("activation", _tensors_work())
-    def route_combine(self, y, row_of, weights, out):
-        """out[m] = sum_i weights[m, i] * y[row_of[m * top + i]] (32-bit sums, in the order of the choices)."""
+    def route_combine(self, y, row_of, weights, out, shared=None, shared_gate=None):
+        """out[m] = sum_i weights[m, i] * y[row_of[m * top + i]] (32-bit sums, in the order of the choices), plus
+        shared[m], which `shared_gate` (a float column [rows, 1] of a row-major matrix) multiplies by its sigmoid."""
         _tensor(weights, "weights", torch.float32, ndim=2)
         rows, top = weights.shape
         _tensor(y, "y", self.dtype, ndim=2)
         _need(y.shape[0] == rows * top, "route_combine: one row of y a pair")
         _tensor(row_of, "row_of", torch.int32, (rows * top,))
         _tensor(out, "out", self.dtype, (rows, y.shape[1]))
-        _ok(self._lib("grouped_gemm").mlr_route_combine(_p(y), _p(row_of), _p(weights), _p(out), _c_int(rows),
-                                                        _c_int(y.shape[1]), _c_int(top), _stream()), "route_combine")
+        _need(shared is not None or shared_gate is None, "route_combine: a gate without what it gates")
+        if shared is not None:
+            _tensor(shared, "shared", self.dtype, (rows, y.shape[1]))
+        gate_stride = self._columns(shared_gate, "shared_gate", torch.float32, rows, 1) if shared_gate is not None else 0
+        _ok(self._lib("grouped_gemm").mlr_route_combine(
+            _p(y), _p(row_of), _p(weights), _p(out), _c_int(rows), _c_int(y.shape[1]), _c_int(top), _p(shared),
+            _p(shared_gate), ctypes.c_long(gate_stride), _stream()), "route_combine")
 
     # -- sampling ----------------------------------------------------------------------------
     def sample_scratch(self, rows):

@@ -58,40 +58,53 @@ class PreNormBlock:
 @register_part("block", "parallel")
 class ParallelBlock:
     """Mixer and feed-forward side by side on the same input, each behind a norm of its own:
-    h += mixer(norm1(h)) + ffn(norm2(h)); the sum of the two branches is taken in 32-bit and added to the float
-    residual stream.  `norm2` and `ffn` may be missing (a layer without a feed-forward).  Both norms divide by
-    the same root mean square, so one pass over h serves both (`Kernels.add2_rmsnorm2`), and that pass is the
-    one that adds the branches of the block before: a block ends by norming h for the block that follows
-    (`Normed`) when that one is of this kind too, else it adds its branches itself."""
+    h += mixer(norm1(h)) + ffn(norm2(h)), or (`norm2` missing) both behind the first: h += mixer(x) + ffn(x), x = norm1(h);
+    the sum of the two branches is taken in 32-bit and added to the float residual stream.  Both `norm2` and `ffn` may be
+    missing (a layer without a feed-forward).  RMS norms divide by the same root mean square, so one pass over h serves
+    both (`Kernels.add2_rmsnorm2`), and that pass is the one that adds the branches of the block before; a single norm of
+    another kind may offer the same pass (`norm_sum`).  A block ends by norming h for the block that follows (`Normed`)
+    when that one is of this kind too, else it adds its branches itself."""
     graph_safe = True
     wants_next_block = True
 
     def __init__(self, spec):
         self.norm1 = build_part("norm", spec.norm1)
         self.mixer = build_part("mixer", spec.mixer)
-        if (spec.ffn is None) != (spec.norm2 is None):
-            raise ValueError("a parallel block has a feed-forward and its norm, or neither")
+        if spec.ffn is None and spec.norm2 is not None:
+            raise ValueError("a parallel block's second norm is its feed-forward's")
         self.norm2 = build_part("norm", spec.norm2) if spec.norm2 is not None else None
         self.ffn = build_part("ffn", spec.ffn) if spec.ffn is not None else None
 
     def parts(self):
         out = {"norm1": self.norm1, "mixer": self.mixer}
         if self.ffn is not None:
-            out.update(norm2=self.norm2, ffn=self.ffn)
+            out["ffn"] = self.ffn
+        if self.norm2 is not None:
+            out["norm2"] = self.norm2
         return out
 
     def workspace_plan(self, rows, dtype, limits):
         width = self.norm1.size
-        return {("normed", dtype): rows * width, ("normed2", dtype): rows * width}
+        return {("normed", dtype): rows * width, **({("normed2", dtype): rows * width} if self.norm2 is not None else {})}
+
+    def _norms(self):
+        return (self.norm1,) if self.norm2 is None else (self.norm1, self.norm2)
 
     def _one_pass(self, width):
-        """Whether the block's norms are plain RMSNorms over the whole width with one eps: then they share a pass."""
-        norms = [self.norm1] + ([self.norm2] if self.norm2 is not None else [])
-        return all(getattr(n, "fusable_rmsnorm", False) and n.size == width and n.eps == self.norm1.eps for n in norms)
+        """Whether the sum of the branches and the block's norms are one pass: plain RMSNorms over the whole width with
+        one eps, or a single norm that offers it."""
+        return self._one_norm(width) or all(getattr(n, "fusable_rmsnorm", False) and n.size == width and n.eps == self.norm1.eps
+                                            for n in self._norms())
+
+    def _one_norm(self, width):
+        return self.norm2 is None and hasattr(self.norm1, "norm_sum") and self.norm1.size == width
 
     def _norm_into(self, ctx, h, d1, d2, x1, x2):
         """h += d1 + d2 (either may be None); x1 = norm1(h), x2 = norm2(h)."""
         k = ctx.kernels
+        if self._one_norm(h.shape[1]):
+            self.norm1.norm_sum(ctx, h, d1, d2, x1)
+            return
         if self._one_pass(h.shape[1]):
             k.add2_rmsnorm2(h, d1, d2, self.norm1.weight, self.norm2.weight if self.norm2 is not None else None,
                             x1, x2 if self.norm2 is not None else None, self.norm1.eps)
@@ -107,21 +120,20 @@ class ParallelBlock:
         from .registry import Normed
         shape = tuple(h.shape)
         x1 = ctx.workspace.get("normed", shape, ctx.dtype)
-        x2 = ctx.workspace.get("normed2", shape, ctx.dtype) if self.ffn is not None else None
-        if isinstance(pending, Normed) and pending.norms == ((self.norm1, self.norm2) if self.ffn is not None else (self.norm1,)):
-            x1, x2 = pending.outputs if self.ffn is not None else (pending.outputs[0], None)
+        x2 = ctx.workspace.get("normed2", shape, ctx.dtype) if self.norm2 is not None else None
+        if isinstance(pending, Normed) and pending.norms == self._norms():
+            x1, x2 = pending.outputs if self.norm2 is not None else (pending.outputs[0], None)
         else:
             self._norm_into(ctx, h, None if isinstance(pending, Complete) else pending, None, x1, x2)
         mixed = self.mixer.forward(ctx, x1, cache_id, write_cache)
-        fed = self.ffn.forward(ctx, x2) if self.ffn is not None else None
+        fed = self.ffn.forward(ctx, x2 if x2 is not None else x1) if self.ffn is not None else None
         if isinstance(next_block, ParallelBlock) and next_block._one_pass(h.shape[1]):
             # the branches are added and h is normed for the next block in one pass (its inputs go where this
             # block's own were: both branches have read them)
             n1 = ctx.workspace.get("normed", shape, ctx.dtype)
-            n2 = ctx.workspace.get("normed2", shape, ctx.dtype) if next_block.ffn is not None else None
+            n2 = ctx.workspace.get("normed2", shape, ctx.dtype) if next_block.norm2 is not None else None
             next_block._norm_into(ctx, h, mixed, fed, n1, n2)
-            return Normed((next_block.norm1, next_block.norm2) if next_block.ffn is not None else (next_block.norm1,),
-                          (n1, n2) if next_block.ffn is not None else (n1,))
+            return Normed(next_block._norms(), (n1,) if n2 is None else (n1, n2))
         if fed is None:
             return mixed                                  # (one delta: whoever norms next adds it)
         ctx.kernels.residual_add2(h, mixed, fed)

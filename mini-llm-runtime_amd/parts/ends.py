@@ -43,9 +43,9 @@ class TokenEmbedding:
         return self.weight
 
     def forward(self, ctx):
-        """The float residual stream [B, E] of the step's tokens."""
+        """The float residual stream [B, E] of the step's tokens: the table's rows times the spec's factor."""
         h = ctx.workspace.get("hidden", (ctx.n_tokens, self.spec.hidden), torch.float32)
-        ctx.kernels.embed_gather(ctx.token_ids, self.weight, h)
+        ctx.kernels.embed_gather(ctx.token_ids, self.weight, h, float(getattr(self.spec, "scale", 1.0)))
         return h
 
 

@@ -86,6 +86,7 @@ class ClampedGluMlp:
         if not spec.limit > 0:
             raise PartError("the clamp's limit must be positive")
         self.spec = spec
+        self.out_name = "ffn_out"                         # (a part that runs it beside others gives it a buffer of its own)
         self.gate_up = None
         self.down = None
 
@@ -105,7 +106,7 @@ class ClampedGluMlp:
     def workspace_plan(self, rows, dtype, limits):
         s = self.spec
         return {("act", dtype): rows * s.intermediate, ("gate_up", dtype): rows * 2 * s.intermediate,
-                ("ffn_out", dtype): rows * s.hidden}
+                (self.out_name, dtype): rows * s.hidden}
 
     def forward(self, ctx, x):
         s = self.spec
@@ -118,17 +119,17 @@ class ClampedGluMlp:
             gate_up = ctx.workspace.get("gate_up", (m, 2 * s.intermediate), x.dtype)
             k.gemm(x, self.gate_up, gate_up)
             k.clamped_glu(gate_up, act, float(s.limit), float(s.slope))
-        out = ctx.workspace.get("ffn_out", (m, s.hidden), x.dtype)
+        out = ctx.workspace.get(self.out_name, (m, s.hidden), x.dtype)
         k.gemm(act, self.down, out)
         return out
 
 
-ACTIVATIONS = ("relu_squared",)
+ACTIVATIONS = ("relu_squared", "gelu_erf")
 
 
 @register_part("ffn", "plain_mlp")
 class PlainMlp:
-    """down(act(up(x))) without a gate; act = relu(x)^2."""
+    """down(act(up(x))) without a gate; act = relu(x)^2 or the exact gelu."""
     graph_safe = True
 
     def __init__(self, spec):
@@ -157,7 +158,7 @@ class PlainMlp:
         k = ctx.kernels
         act = ctx.workspace.get("act", (m, s.intermediate), x.dtype)
         k.gemm(x, self.up, act)
-        k.relu_squared(act, act)
+        k.plain_act(act, act, s.activation)
         out = ctx.workspace.get("ffn_out", (m, s.hidden), x.dtype)
         k.gemm(act, self.down, out)
         return out

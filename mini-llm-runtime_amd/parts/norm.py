@@ -85,19 +85,23 @@ class TanhNorm:
 
 @register_part("norm", "layernorm")
 class LayerNorm:
-    """y = (x - mean) / sqrt(var + eps) * weight + bias, var the mean of the squared deviations; 32-bit."""
+    """y = (x - mean) / sqrt(var + eps) * weight + bias (or without a bias), var the mean of the squared deviations;
+    32-bit."""
     graph_safe = True
 
     def __init__(self, spec):
         self.size, self.eps = spec.size, float(spec.eps)
+        self.has_bias = bool(getattr(spec, "bias", True))
         self.weight = self.bias = None
 
     def weight_specs(self):
-        return {"weight": WeightSpec((self.size,), keep_float32=True),
-                "bias": WeightSpec((self.size,), keep_float32=True, init=("normal", 0.0, 0.1))}
+        specs = {"weight": WeightSpec((self.size,), keep_float32=True)}
+        if self.has_bias:
+            specs["bias"] = WeightSpec((self.size,), keep_float32=True, init=("normal", 0.0, 0.1))
+        return specs
 
     def bind(self, weights):
-        self.weight, self.bias = weights["weight"], weights["bias"]
+        self.weight, self.bias = weights["weight"], weights.get("bias")
 
     def libraries(self):
         return ["elementwise"]
@@ -109,6 +113,11 @@ class LayerNorm:
             ctx.kernels.residual_add(h, delta)
         ctx.kernels.layernorm_rows(h, self.weight, self.bias, out, self.eps, rows=rows, out_scale=out_scale)
         return out
+
+    def norm_sum(self, ctx, h, d1, d2, out):
+        """h += d1 + d2 (either may be None); out = norm(h), in one pass: the two branches of a block and the norm of the
+        block that follows."""
+        ctx.kernels.add2_layernorm(h, d1, d2, self.weight, self.bias, out, self.eps)
 
     def add_into(self, ctx, delta, h, cast=None):
         """h += norm(delta): the norm of what a sublayer gave, added to the float residual stream in the same pass;

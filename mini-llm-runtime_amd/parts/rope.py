@@ -39,12 +39,14 @@ class Rope:
     """Rotary positions over the first `dim` channels of a head, in split-half pairs (j, j + dim/2) or interleaved
     ones (2j, 2j + 1), the frequencies base^(-2j/dim) optionally stretched for long contexts
     (`FrequencyStretch`: a ramp between the pairs that turn fast, which keep their frequency, and those that turn
-    slowly, whose frequency is divided by `factor`; cosines and sines are multiplied by 0.1 ln(factor) + 1).
-    Frequencies and angles are 32-bit; the table holds cos in its first half and sin in its second."""
+    slowly, whose frequency is divided by `factor`; cosines and sines are multiplied by 0.1 ln(factor) + 1) or scaled
+    by bands of how often a pair turns over the original length (`FrequencyBands`: fast pairs stay, slow pairs are
+    divided by `factor`, those between are blended).  Frequencies and angles are 32-bit; the table holds cos in its first half and sin in its second."""
 
     def __init__(self, spec):
         self.dim, self.base = spec.dim, float(spec.base)
         self.interleaved, self.stretch = bool(spec.interleaved), spec.stretch
+        self.bands = getattr(spec, "bands", None)
         if self.dim % 2 != 0 or self.dim < 2:
             raise ValueError(f"a rotation turns an even number of channels, not {self.dim}")
         self._tables = {}
@@ -63,6 +65,12 @@ class Rope:
             ramp = np.clip((j - lo) / max(hi - lo, 0.001), 0.0, 1.0)
             freq = freq / st.factor * ramp + freq * (1.0 - ramp)
             amplitude = 0.1 * np.log(st.factor) + 1.0
+        if self.bands is not None:
+            bd = self.bands
+            turns = bd.original * freq / (2.0 * np.pi)
+            s = (turns - bd.low) / (bd.high - bd.low) if bd.high != bd.low else (turns > bd.high).astype(np.float64)
+            freq = np.where(turns > bd.high, freq, np.where(turns < bd.low, freq / bd.factor,
+                                                            (1.0 - s) * freq / bd.factor + s * freq))
         return freq.astype(np.float32), float(amplitude)
 
     def rotation(self, max_positions, device):

@@ -2,19 +2,24 @@
 32-bit (an ordinary product with float output); the experts form equal groups of neighbours, a group's score is the sum of its two largest s, and only
 experts of the best groups can be chosen; of those the `top` largest s win and weigh their experts' outputs (as
 they are, or divided by their sum, and times `route_scale`).  With `correction` the choice goes by s plus a stored
-number an expert while the weights stay the plain s.  An expert is an ungated feed-forward down(act(up(x))) or,
-`gated`, down(act(gate(x)) * up(x)).
+number an expert while the weights stay the plain s.  The scores may be softmax(router . x) over all experts instead,
+a group's score its largest s.  An expert is an ungated feed-forward down(act(up(x))) or, `gated`, down(act(gate(x)) *
+up(x)), or with the activation `clamped` down(g sigmoid(slope g) (u + 1)) of the clamped g and u.  A shared expert (any
+feed-forward part) runs for every token besides and is added by the pass that sums the chosen experts, multiplied by
+sigmoid(sg . x) when `shared_gate` says so: sg is one more row of the router's product.
 
 The step's (token, expert) pairs are sorted by expert on the device, so that every expert's rows lie side by side
 and ONE launch multiplies all of them with their own weights (`Kernels.experts_gemm`, the rows of the first product
 gathered through the sorted list); nothing of it is read on the host, so a step can be captured."""
 from __future__ import annotations
 
+from dataclasses import replace
+
 import torch
 
 from ..weights.loader import WeightSpec, stacked
 from .mlp import ACTIVATIONS
-from .registry import PartError, register_part
+from .registry import PartError, build_part, register_part
 
 
 @register_part("ffn", "routed_mlp")
@@ -25,12 +30,21 @@ class RoutedMlp:
         s = self.spec = spec
         self.gated = bool(getattr(s, "gated", False))
         if self.gated:
-            if s.activation not in ("silu", "gelu_tanh"):
-                raise PartError(f"gated experts: activation {s.activation!r} is not built (silu, gelu_tanh)")
+            if s.activation not in ("silu", "gelu_tanh", "clamped"):
+                raise PartError(f"gated experts: activation {s.activation!r} is not built (silu, gelu_tanh, clamped)")
+            if s.activation == "clamped" and not (s.limit is not None and s.limit > 0):
+                raise PartError("clamped experts need a positive limit")
         elif s.activation not in ACTIVATIONS:
             raise PartError(f"activation {s.activation!r} is not built ({', '.join(ACTIVATIONS)})")
-        if s.score != "sigmoid":
-            raise PartError("routing: sigmoid scores are what is built")
+        if s.score not in ("sigmoid", "softmax") or s.group_score not in ("best_two", "best"):
+            raise PartError(f"routing: scores {s.score!r} (sigmoid, softmax) of groups by {s.group_score!r} (best_two, best)")
+        self.shared = build_part("ffn", s.shared) if s.shared is not None else None
+        if self.shared is not None:
+            if not hasattr(self.shared, "out_name"):
+                raise PartError("the shared expert cannot write to a buffer of its own (`out_name`)")
+            self.shared.out_name = "shared_out"
+        elif s.shared_gate:
+            raise PartError("a gate for a shared expert that is not there")
         self.correction = None
         self.fused_gate = False
         if s.experts % s.group_count != 0 or not 1 <= s.group_keep <= s.group_count or \
@@ -43,7 +57,13 @@ class RoutedMlp:
         s = self.spec
         # (a matrix like the others: its products with the layer's input are exact in 32 bits, and so are their sums'
         # partial results up to rounding: the logits are an ordinary product with float output)
-        specs = {"router": WeightSpec((s.experts, s.hidden), init=("normal", 0.0, 0.05))}
+        gate = bool(s.shared_gate)
+        specs = {"router": WeightSpec((s.experts, s.hidden), init=("normal", 0.0, 0.05), stack="route" if gate else None)}
+        if gate:                                # (one more row of the router's product)
+            specs["shared.sg"] = WeightSpec((1, s.hidden), init=("normal", 0.0, 0.05), stack="route")
+        if self.shared is not None:
+            for local, ws in self.shared.weight_specs().items():
+                specs[f"shared.{local}"] = replace(ws, stack=f"shared.{ws.stack}") if ws.stack is not None else ws
         if getattr(s, "correction", False):
             specs["correction"] = WeightSpec((s.experts,), keep_float32=True, init=("normal", 0.0, 0.05))
         for e in range(s.experts):
@@ -56,7 +76,10 @@ class RoutedMlp:
 
     def bind(self, weights):
         s = self.spec
-        self.router = weights["router"]
+        self.router = stacked([weights["router"], weights["shared.sg"]]) if s.shared_gate else weights["router"]
+        if self.shared is not None:
+            self.shared.bind({name[len("shared."):]: t for name, t in weights.items()
+                              if name.startswith("shared.") and name != "shared.sg"})
         self.correction = weights.get("correction")
         first = [weights[f"e{e}.{n}"] for e in range(s.experts) for n in (("gate", "up") if self.gated else ("up",))]
         self.up = stacked(first).view(s.experts, (2 if self.gated else 1) * s.intermediate, s.hidden)
@@ -76,12 +99,14 @@ class RoutedMlp:
         self.down = stacked([weights[f"e{e}.down"] for e in range(s.experts)]).view(s.experts, s.hidden, s.intermediate)
 
     def libraries(self):
-        return ["gemm", "grouped_gemm"] + (["elementwise"] if self.gated else [])
+        return sorted({"gemm", "grouped_gemm", *(["elementwise"] if self.gated else []),
+                       *(self.shared.libraries() if self.shared is not None else [])})
 
     def workspace_plan(self, rows, dtype, limits):
         s = self.spec
         pairs = rows * s.top
-        return {("route_logits", torch.float32): rows * s.experts, ("route_ids", torch.int32): pairs,
+        return {**(self.shared.workspace_plan(rows, dtype, limits) if self.shared is not None else {}),
+                ("route_logits", torch.float32): rows * (s.experts + (1 if s.shared_gate else 0)), ("route_ids", torch.int32): pairs,
                 ("route_weights", torch.float32): pairs,
                 ("route_offsets", torch.int32): s.experts + 1, ("route_token", torch.int32): pairs,
                 ("route_row", torch.int32): pairs, ("route_act", dtype): pairs * s.intermediate,
@@ -98,22 +123,31 @@ class RoutedMlp:
         offsets = ws.get("route_offsets", (s.experts + 1,), torch.int32)
         token_of = ws.get("route_token", (pairs,), torch.int32)
         row_of = ws.get("route_row", (pairs,), torch.int32)
-        logits = ws.get("route_logits", (m, s.experts), torch.float32)
+        logits = ws.get("route_logits", (m, self.router.shape[0]), torch.float32)
         k.gemm(x, self.router, logits)                   # 32-bit sums of the engine's element type's products
         k.router_topk(logits, ids, weights, s.group_count, s.group_keep, correction=self.correction,
-                      renormalize=bool(s.renormalize), scale=float(getattr(s, "route_scale", 1.0)))
+                      renormalize=bool(s.renormalize), scale=float(getattr(s, "route_scale", 1.0)), score=s.score,
+                      group_score=s.group_score, experts=s.experts)
         k.route_sort(ids, s.experts, offsets, token_of, row_of)
         act = ws.get("route_act", (pairs, s.intermediate), x.dtype)
         if self.fused_gate:
-            k.experts_gemm(x, self.up, act, offsets, gather=token_of, act="gated_" + s.activation)
+            k.experts_gemm(x, self.up, act, offsets, gather=token_of, act="gated_" + s.activation, limit=float(s.limit or 0.0),
+                           slope=float(s.slope))
         elif self.gated:
             both = ws.get("route_gate_up", (pairs, 2 * s.intermediate), x.dtype)
             k.experts_gemm(x, self.up, both, offsets, gather=token_of)
-            k.gated_act_mul(both, act, s.activation)
+            if s.activation == "clamped":
+                k.clamped_glu(both, act, float(s.limit), float(s.slope))
+            else:
+                k.gated_act_mul(both, act, s.activation)
         else:
             k.experts_gemm(x, self.up, act, offsets, gather=token_of, act=s.activation)
         y = ws.get("route_y", (pairs, s.hidden), x.dtype)
         k.experts_gemm(act, self.down, y, offsets)
         out = ws.get("ffn_out", (m, s.hidden), x.dtype)
-        k.route_combine(y, row_of, weights, out)
+        if self.shared is None:
+            k.route_combine(y, row_of, weights, out)
+        else:
+            k.route_combine(y, row_of, weights, out, shared=self.shared.forward(ctx, x),
+                            shared_gate=logits[:, s.experts:] if s.shared_gate else None)
         return out
