@@ -1,0 +1,716 @@
+"""The Nuvorax parts on the GPU against the plain implementation (tests/plain/nuvorax_plain.py): every kernel alone, then
+small random models in every way of cutting requests into steps, in 32-bit and in bfloat16, then generation through the
+scheduler, the command line and the trace tool.  The configurations differ from each other in every size, and hold
+values that a model may happen to make equal or 1 (one head, kv heads = heads, value size = key size, a rotation of the
+whole head, one group of experts, groups of one expert, every expert chosen, no feed-forward, no scaled frequency)."""
+import json
+import os
+
+import numpy as np
+import pytest
+import torch
+
+from helpers import last_one_by_one, make_requests, max_difference, mixed, plain_logits, portions, run_steps, whole
+from plain import nuvorax_plain as P
+
+pytestmark = pytest.mark.gpu
+
+DTYPES = {"float32": torch.float32, "bfloat16": torch.bfloat16}
+
+
+def attention(heads, kv, dim, vdim, rot, cap=30.0, base=10000.0, scale=None, scaling="middle"):
+    bands = {"middle": dict(factor=4.0, low=1.0, high=3.0, original=40), "slow": dict(factor=16.0, low=2.0, high=2.5, original=9),
+             "none": None}[scaling]
+    return dict(type="attention", mixer=dict(heads=heads, kv_heads=kv, dim=dim, vdim=vdim, scale=scale or 2.0 * dim ** -0.5,
+                                             softcap=cap, rot=dict(dims=rot, base=base, **({} if bands is None else dict(scaling=bands)))))
+
+
+def dense(layer, ff):
+    return dict(layer, mlp=None if ff is None else dict(kind="dense", ff=ff))
+
+
+def moe(layer, ff, experts, top, count, keep, shared, limit=1.0, shared_limit=1.5, scale=1.3):
+    return dict(layer, mlp=dict(kind="moe", expert=dict(ff=ff, limit=limit), shared=dict(ff=shared, limit=shared_limit),
+                                router=dict(experts=experts, top=top, scale=scale, groups=dict(count=count, keep=keep))))
+
+
+def model(vocab, width, layers, eps=1e-5, logit_scale=1.0, embed=2.0):
+    return dict(architecture="Nuvorax", vocab=vocab, width=width, norm=dict(eps=eps), embedding=dict(scale=embed),
+                logit_scale=logit_scale, layers=layers)
+
+
+CONFIGS = {
+    # the matrix cores take every layer: two, four and one heads a kv head
+    "mix": model(211, 96, [moe(attention(4, 2, 32, 16, 16), 48, 6, 2, 3, 2, 40), dense(attention(8, 2, 24, 48, 8, base=500.0), 160),
+                           moe(attention(3, 3, 16, 32, 16, cap=15.0, scaling="slow"), 32, 8, 3, 4, 2, 64, limit=0.5)], logit_scale=0.5),
+    # sizes the matrix cores do not take, one head, an expert a group, everything chosen, no feed-forward
+    "odd": model(97, 72, [dense(attention(3, 3, 20, 36, 10, cap=50.0), 50), dense(attention(1, 1, 12, 12, 12, scaling="none"), None),
+                          moe(attention(5, 1, 6, 10, 2, base=30.0), 20, 8, 3, 8, 4, 12, scale=1.0),
+                          moe(attention(10, 5, 8, 6, 4, cap=5.0), 24, 5, 5, 1, 1, 30, limit=2.0, shared_limit=0.25, scale=2.5)],
+                 eps=3e-6, logit_scale=2.0, embed=1.0),
+    # more than sixteen and more than thirty-two heads in the padded order, heads a kv head no power of two
+    "heads": model(64, 64, [dense(attention(20, 4, 8, 16, 8), 96), dense(attention(40, 8, 8, 16, 4), None),
+                            moe(attention(24, 1, 16, 32, 8), 16, 4, 1, 1, 1, 16), dense(attention(6, 6, 32, 64, 32), 32)]),
+    "no_mix_of_experts": model(160, 80, [dense(attention(16, 1, 16, 80, 8), 96), dense(attention(4, 1, 72, 16, 64), 64)], embed=0.7),
+    "wide": model(128, 128, [moe(attention(16, 4, 64, 64, 32), 64, 12, 3, 3, 1, 96), moe(attention(8, 8, 128, 128, 128), 96, 16, 4, 2, 2, 64)],
+                  logit_scale=0.75, embed=3.0),
+}
+LENGTHS = [70, 33, 150, 17, 64, 129, 2, 45]
+LEAST = 25.0                  # of a token's routing margin (see `route_margin`)
+_cache = {}
+
+
+@pytest.fixture(scope="module")
+def folders(tmp_path_factory):
+    from mini_llm_runtime_amd.config import config_from_dict
+    from mini_llm_runtime_amd.weights import write_random_model
+    out = {}
+    for i, (name, cfg) in enumerate(CONFIGS.items()):
+        folder = str(tmp_path_factory.mktemp(f"nuvorax_{name}"))
+        write_random_model(folder, config_from_dict(cfg), seed=170 + i, matrix_std=0.12, norm_std=0.2)
+        out[name] = folder
+    return out
+
+
+def decisive_requests(oracle, vocab, lengths, seed):
+    """Random requests in which no token's choice of experts is a close call: an engine that rounds takes the experts
+    that the plain model takes, and rows can be compared."""
+    rng = np.random.default_rng(2000 + seed)
+    return {rid: oracle.decisive(toks, rng, LEAST) for rid, toks in make_requests(vocab, lengths, seed).items()}
+
+
+def plain(folders, name):
+    if ("plain", name) not in _cache:
+        oracle = P.PlainNuvorax(folders[name])
+        reqs = decisive_requests(oracle, CONFIGS[name]["vocab"], LENGTHS, seed=9)
+        _cache[("plain", name)] = (oracle, reqs, plain_logits(oracle, reqs))
+    return _cache[("plain", name)]
+
+
+def load(folders, name, dtype_name):
+    from mini_llm_runtime_amd.parts import DecoderModel
+    if (name, dtype_name) not in _cache:
+        _cache[(name, dtype_name)] = DecoderModel.load(folders[name], DTYPES[dtype_name])
+    return _cache[(name, dtype_name)]
+
+
+def runner_for(loaded, max_tokens, **kwargs):
+    from mini_llm_runtime_amd.engine import Runner
+    kwargs.setdefault("max_length", 512)
+    kwargs.setdefault("page_size", 8)
+    return Runner(loaded, max_tokens=max_tokens, max_slots=4, **kwargs)
+
+
+def close(got, want, dtype_name, scale, outliers=None):
+    """Rows against float64: the float engine to rounding at every row; the bfloat16 engine to 4 % of the largest logit
+    at the worst place and 1.2 % in the root mean square, where one row in fifty may reach three times that."""
+    assert set(got) == set(want)
+    over = []
+    for key in sorted(want):
+        err = np.abs(got[key] - want[key])
+        assert np.isfinite(got[key]).all(), key
+        if dtype_name == "float32":
+            assert err.max() <= 3e-4 * scale, (key, err.max(), scale)
+        elif not (err.max() <= 0.04 * scale and np.sqrt((err ** 2).mean()) <= 0.012 * scale):
+            assert err.max() <= 0.12 * scale and np.sqrt((err ** 2).mean()) <= 0.036 * scale, (key, err.max(), scale)
+            over.append(key)
+    assert len(over) <= (max(1, len(want) // 50) if outliers is None else outliers), over
+
+
+def idle(r):
+    r.cache.check()
+    assert r.free_slots() == 4
+    for g in range(len(r.cache.group_pages)):
+        assert r.cache.free_pages(g) == r.cache.group_pages[g]
+
+
+def rounded(x, dtype):
+    return torch.from_numpy(np.ascontiguousarray(x)).to(dtype).cuda()
+
+
+def back(t):
+    return t.double().cpu().numpy()
+
+
+def ints(x):
+    return torch.tensor(x, dtype=torch.int32, device="cuda")
+
+
+def tolerance(dtype_name):
+    # (a score near the cap of 30 carries 32-bit rounding of a few 1e-6, and so does its exponential)
+    return dict(rtol=6e-5, atol=6e-5) if dtype_name == "float32" else dict(rtol=3e-2, atol=2e-2)
+
+
+# ---- the kernels alone --------------------------------------------------------------------------------------------
+def paged(keys, values, page, dtype, seed=0):
+    """keys [T, G, D] and values [T, G, V] of ONE request in pages that lie in a shuffled order, values transposed within a
+    page, NaN where nothing was written; (k_pages, v_pages, block table [1, blocks])."""
+    T, G, D = keys.shape
+    V = values.shape[2]
+    blocks = -(-T // page)
+    order = np.random.default_rng(seed).permutation(blocks + 3)[:blocks]
+    kp, vp = np.full((blocks + 3, G, page, D), np.nan), np.full((blocks + 3, G, V, page), np.nan)
+    for t in range(T):
+        kp[order[t // page], :, t % page] = keys[t]
+        vp[order[t // page], :, :, t % page] = values[t]
+    return rounded(kp, dtype), rounded(vp, dtype), ints(order[None].tolist())
+
+
+def plain_attend(q, keys, values, positions, scale, cap, sink, talk, turn_base, gate):
+    """q [M, H, D] at `positions` over keys [T, G, D], values [T, G, V] of one request -> [M, H * V]."""
+    T, G = keys.shape[:2]
+    M, H = q.shape[:2]
+    seen = np.arange(T)[None, :] <= np.asarray(positions)[:, None]
+    weights = []
+    for h in range(H):
+        s = (q[:, h] @ keys[:, h // (H // G)].T) * scale
+        s = np.where(seen, P.capped(s, cap) if cap is not None else s, -np.inf)
+        extra = -np.inf if sink is None else sink[h] if np.ndim(sink) else sink
+        top = np.maximum(s.max(axis=1, keepdims=True), extra)
+        e = np.exp(s - top)
+        weights.append(e / (e.sum(axis=1, keepdims=True) + np.exp(extra - top)))
+    weights = P.mixed_heads(np.stack(weights), talk)
+    out = np.stack([weights[h] @ values[:, h // (H // G)] for h in range(H)], axis=1)
+    if turn_base is not None:
+        out = P.rotate_values(out, positions, turn_base, -1.0)
+    if gate is not None:
+        out = out / (1.0 + np.exp(-gate))[:, :, None]
+    return out.reshape(M, -1)
+
+
+def turn_table(dim, base, positions):
+    from mini_llm_runtime_amd.config.specs import PositionSpec
+    from mini_llm_runtime_amd.parts.rope import Rope
+    return Rope(PositionSpec("rope", dim, base)).rotation(positions, "cuda").table
+
+
+def launch_tiles(k, q, k_pages, v_pages, table, slots, pos, talk, sink, v_rope, gate, heads, kv, dim, vdim, page, scale, cap,
+                 first, count, tokens, context, score_keys, value_keys, kv_block):
+    """The matrix-core form with NaN in every piece of scratch memory."""
+    pad, inner, most = k.head_mix_layout(heads, kv, vdim)
+    ktiles, n = -(-context // 32), len(first)
+    score_ranges, value_ranges = -(-ktiles * 32 // score_keys), -(-ktiles * 32 // value_keys)
+    nan = lambda count, dtype: torch.full((count,), float("nan"), dtype=dtype, device="cuda")
+    rows = n * tokens
+    out = torch.full((q.shape[0], heads * vdim), float("nan"), dtype=q.dtype, device="cuda")
+    k.head_mix_tiles(q, k_pages, v_pages, table, slots, pos, talk, sink, v_rope, gate, out, ints(first), ints(count), n, tokens,
+                     heads, kv, dim, vdim, page, scale, cap, nan(rows * ktiles * 32 * inner, q.dtype),
+                     nan(rows * inner * score_ranges, torch.float32), nan(rows * heads * value_ranges * vdim, torch.float32),
+                     ktiles, score_keys, score_ranges, value_keys, value_ranges, min(kv_block, most))
+    return back(out)
+
+
+SHAPES = [(4, 2, 32, 16, 8), (6, 3, 64, 32, 16), (8, 2, 72, 80, 8), (3, 3, 20, 36, 4), (16, 4, 128, 128, 16), (12, 1, 40, 48, 8),
+          (32, 8, 64, 128, 16), (20, 4, 8, 16, 24), (32, 1, 32, 64, 8), (40, 8, 16, 32, 64), (96, 12, 8, 16, 8), (1, 1, 256, 256, 16)]
+
+
+@pytest.mark.parametrize("dtype_name", DTYPES)
+@pytest.mark.parametrize("heads,kv,dim,vdim,page", SHAPES)
+def test_mixed_heads_find_one_key_wherever_it_lies(dtype_name, heads, kv, dim, vdim, page):
+    """For one query one key among 300 is made to stand out in every second head, the other heads see all keys alike: at
+    the first tokens, at page and tile borders, far back and at the query's own position; a key behind the query, which
+    must not be seen, too.  Both forms, the matrix cores with every query a group of its own, whole and in ranges."""
+    from mini_llm_runtime_amd.kernels import Kernels
+    dtype = DTYPES[dtype_name]
+    k = Kernels(dtype)
+    rng = np.random.default_rng(5)
+    T, cap, base = 300, 30.0, 700.0
+    keys, values = rounded(rng.normal(size=(T, kv, dim)) * 0.3, dtype), rounded(rng.normal(size=(T, kv, vdim)), dtype)
+    keys64, values64 = back(keys), back(values)
+    pairs = sorted({(qp, kp) for qp in (0, 1, 5, page - 1, page, 31, 32, 63, 64, 65, 127, 128, 200, 255, 256, 299)
+                    for kp in (0, 1, qp - 1, qp, qp + 1, qp - 7, qp - page, qp - 32, qp - 64, qp - 150, page - 1, page) if 0 <= kp < T})
+    q = rng.normal(size=(len(pairs), heads, dim)) * 0.02
+    for i, (_, kp) in enumerate(pairs):
+        for h in range(i % 2, heads, 2):
+            key = keys64[kp, h // (heads // kv)]
+            q[i, h] = key * (40.0 / float(np.sum(key ** 2)))
+    q = rounded(q, dtype)
+    positions = [p for p, _ in pairs]
+    m = len(pairs)
+    talk = rounded(rng.normal(size=(heads, heads)) * heads ** -0.5, torch.bfloat16).float()
+    gate = rounded(rng.normal(size=(m, heads)) * 2.0, dtype)
+    k_pages, v_pages, table = paged(keys64, values64, page, dtype, seed=1)
+    slots, pos = torch.zeros(m, dtype=torch.int32, device="cuda"), ints(positions)
+    v_rope = (turn_table(vdim, base, T), False)
+    want = plain_attend(back(q), keys64, values64, positions, 1.0, cap, 0.0, back(talk), base, back(gate))
+    rows = q.view(m, -1)
+    out = torch.empty((m, heads * vdim), dtype=dtype, device="cuda")
+    k.head_mix_attention(rows, k_pages, v_pages, table, slots, pos, talk, 0.0, v_rope, gate, out, heads, kv, dim, vdim, page, 1.0, cap)
+    np.testing.assert_allclose(back(out), want, **tolerance(dtype_name))
+    taken = k.head_mix_tiles_supported(heads, kv, dim, vdim, page, cap)
+    assert taken == (dtype_name == "bfloat16" and (heads, page) != (3, 4))
+    if taken:
+        for tokens, score_keys, value_keys, block in ((1, 320, 512, 8), (16, 320, 320, 8), (1, 128, 256, 1), (16, 96, 64, 1), (16, 32, 160, 2)):
+            got = launch_tiles(k, rows, k_pages, v_pages, table, slots, pos, talk, 0.0, v_rope, gate, heads, kv, dim, vdim, page, 1.0,
+                               cap, list(range(m)), [1] * m, tokens, T, score_keys, value_keys, block)
+            np.testing.assert_allclose(got, want, err_msg=str((tokens, score_keys, value_keys, block)), **tolerance(dtype_name))
+
+
+@pytest.mark.parametrize("sink", [None, 0.0, -1.5, "learned"])
+@pytest.mark.parametrize("heads,kv,dim,vdim,page", [s for s in SHAPES if s[4] != 4])
+def test_groups_of_tokens_on_the_matrix_cores(sink, heads, kv, dim, vdim, page):
+    """Every position of a request of 210 tokens at once, in groups of 16 and of 5 tokens and of one, with and without
+    turned values and gates, for every kind of sink, the scores of every key alive; bfloat16 and, in the other form, 32-bit."""
+    from mini_llm_runtime_amd.kernels import Kernels
+    rng = np.random.default_rng(12)
+    T, cap, scale = 210, 12.0, 0.7
+    for dtype_name, dtype in DTYPES.items():
+        k = Kernels(dtype)
+        keys, values = rounded(rng.normal(size=(T, kv, dim)), dtype), rounded(rng.normal(size=(T, kv, vdim)), dtype)
+        q = rounded(rng.normal(size=(T, heads, dim)), dtype)
+        talk = rounded(rng.normal(size=(heads, heads)) * heads ** -0.5, torch.bfloat16).float()
+        gate = rounded(rng.normal(size=(T, heads)), dtype)
+        sinks = rounded(rng.normal(size=heads), torch.float32) if sink == "learned" else sink
+        k_pages, v_pages, table = paged(back(keys), back(values), page, dtype, seed=3)
+        slots, pos = torch.zeros(T, dtype=torch.int32, device="cuda"), torch.arange(T, dtype=torch.int32, device="cuda")
+        for turned, gated in ((True, True), (False, False)):
+            v_rope = (turn_table(vdim, 50.0, T), False) if turned else None
+            g = gate if gated else None
+            want = plain_attend(back(q), back(keys), back(values), np.arange(T), scale, cap, back(sinks) if sink == "learned" else sink,
+                                back(talk), 50.0 if turned else None, back(gate) if gated else None)
+            if dtype_name == "float32":
+                out = torch.empty((T, heads * vdim), dtype=dtype, device="cuda")
+                k.head_mix_attention(q.view(T, -1), k_pages, v_pages, table, slots, pos, talk, sinks, v_rope, g, out, heads, kv, dim,
+                                     vdim, page, scale, cap)
+                np.testing.assert_allclose(back(out), want, **tolerance(dtype_name))
+                continue
+            for tokens, size, score_keys, value_keys, block in ((16, 16, 224, 224, 8), (16, 5, 128, 64, 1), (1, 1, 128, 256, 4)):
+                first = list(range(0, T, size))
+                count = [min(size, T - f) for f in first]
+                got = launch_tiles(k, q.view(T, -1), k_pages, v_pages, table, slots, pos, talk, sinks, v_rope, g, heads, kv, dim, vdim,
+                                   page, scale, cap, first, count, tokens, T, score_keys, value_keys, block)
+                np.testing.assert_allclose(got, want, err_msg=str((turned, tokens, size)), **tolerance(dtype_name))
+
+
+@pytest.mark.parametrize("dtype_name", DTYPES)
+def test_scores_without_a_cap_and_pairs_of_neighbouring_value_channels(dtype_name):
+    """The form that takes any sizes: no cap, scores far beyond what an unshifted exponential holds, a value rotation
+    in neighbouring pairs."""
+    from mini_llm_runtime_amd.config.specs import PositionSpec
+    from mini_llm_runtime_amd.kernels import Kernels
+    from mini_llm_runtime_amd.parts.rope import Rope
+    dtype = DTYPES[dtype_name]
+    k = Kernels(dtype)
+    rng = np.random.default_rng(3)
+    T, heads, kv, dim, vdim, page = 80, 4, 2, 10, 6, 4
+    keys, values, q = (rounded(rng.normal(size=(T, n, d)), dtype) for n, d in ((kv, dim), (kv, vdim), (heads, dim)))
+    talk = rounded(rng.normal(size=(heads, heads)), torch.float32)
+    k_pages, v_pages, table = paged(back(keys), back(values), page, dtype)
+    out = torch.empty((T, heads * vdim), dtype=dtype, device="cuda")
+    v_rope = (Rope(PositionSpec("rope", vdim, 9.0, interleaved=True)).rotation(T, "cuda").table, True)
+    k.head_mix_attention(q.view(T, -1), k_pages, v_pages, table, torch.zeros(T, dtype=torch.int32, device="cuda"),
+                         torch.arange(T, dtype=torch.int32, device="cuda"), talk, 0.0, v_rope, None, out, heads, kv, dim, vdim, page, 40.0)
+    halves = plain_attend(back(q), back(keys), back(values), np.arange(T), 40.0, None, 0.0, back(talk), None, None).reshape(T, heads, vdim)
+    turned = P.rotate_values(np.concatenate([halves[..., 0::2], halves[..., 1::2]], axis=-1), np.arange(T), 9.0, -1.0)
+    want = np.stack([turned[..., :vdim // 2], turned[..., vdim // 2:]], axis=-1).reshape(T, -1)
+    tol = dict(rtol=2e-4, atol=2e-4) if dtype_name == "float32" else tolerance(dtype_name)
+    np.testing.assert_allclose(back(out), want, **tol)
+
+
+@pytest.mark.parametrize("dtype_name", DTYPES)
+@pytest.mark.parametrize("heads,kv,dim,vdim,rot,page", [(4, 2, 16, 24, 8, 8), (3, 3, 20, 6, 20, 4), (2, 1, 70, 130, 2, 16), (16, 4, 128, 128, 64, 16),
+                                                        (6, 2, 64, 96, 64, 8)])
+def test_keys_are_turned_by_bands_and_values_whole_on_their_way_into_the_pages(dtype_name, heads, kv, dim, vdim, rot, page):
+    from mini_llm_runtime_amd.config.specs import FrequencyBands, PositionSpec
+    from mini_llm_runtime_amd.kernels import Kernels
+    from mini_llm_runtime_amd.parts.rope import Rope
+    dtype = DTYPES[dtype_name]
+    k = Kernels(dtype)
+    rng = np.random.default_rng(7)
+    positions = np.array([0, 1, 2, 7, 8, 9, 30, 31, 32, 100, 101, 5, 6])
+    m, gates = len(positions), heads
+    total = heads * dim + kv * (dim + vdim)
+    proj = rounded(rng.normal(size=(m, total + gates)), dtype)
+    x = back(proj)[:, :total]
+    qw, kw = (rounded(1.0 + 0.3 * rng.normal(size=dim), torch.float32) for _ in range(2))
+    rule = dict(dims=rot, base=300.0, scaling=dict(factor=5.0, low=1.5, high=4.0, original=60))
+    q = P.rotate_keys(P.rms_norm(x[:, :heads * dim].reshape(m, heads, dim), back(qw), 1e-4), positions, rule)
+    kk = P.rotate_keys(P.rms_norm(x[:, heads * dim:(heads + kv) * dim].reshape(m, kv, dim), back(kw), 1e-4), positions, rule)
+    vv = P.rotate_values(x[:, (heads + kv) * dim:].reshape(m, kv, vdim), positions, 300.0)
+    blocks = -(-104 // page)
+    order = np.random.default_rng(1).permutation(blocks + 2)[:blocks]
+    k_pages = torch.full((blocks + 2, kv, page, dim), float("nan"), dtype=dtype, device="cuda")
+    v_pages = torch.full((blocks + 2, kv, vdim, page), float("nan"), dtype=dtype, device="cuda")
+    q_out = torch.empty((m, heads * dim), dtype=dtype, device="cuda")
+    bands = FrequencyBands(factor=5.0, original=60, low=1.5, high=4.0)
+    k.sink_qkv_prep(proj, None, q_out, k_pages, v_pages, ints(order[None].tolist()), torch.zeros(m, dtype=torch.int32, device="cuda"),
+                    ints(positions.tolist()), qw, kw, 1e-4, Rope(PositionSpec("rope", rot, 300.0, bands=bands)).rotation(128, "cuda").table,
+                    heads, kv, dim, vdim, page, v_rope=turn_table(vdim, 300.0, 128), v_transposed=True)
+    tol = tolerance(dtype_name)
+    np.testing.assert_allclose(back(q_out), q.reshape(m, -1), **tol)
+    kp, vp = back(k_pages), back(v_pages)
+    for i, p in enumerate(positions):
+        np.testing.assert_allclose(kp[order[p // page], :, p % page], kk[i], **tol)
+        np.testing.assert_allclose(vp[order[p // page], :, :, p % page], vv[i], **tol)
+    assert np.isfinite(kp).sum() == m * kv * dim and np.isfinite(vp).sum() == m * kv * vdim      # nothing else was touched
+
+
+@pytest.mark.parametrize("dtype_name", DTYPES)
+@pytest.mark.parametrize("rows,width", [(5, 24), (3, 37), (70, 128), (2, 1), (9, 4100), (2, 9000), (1, 2050)])
+def test_branches_are_added_and_normed_in_one_pass(dtype_name, rows, width):
+    from mini_llm_runtime_amd.kernels import Kernels
+    dtype = DTYPES[dtype_name]
+    k = Kernels(dtype)
+    rng = np.random.default_rng(width)
+    h64 = back(rounded(rng.normal(size=(rows, width)) + 3.0, torch.float32))
+    d = [rounded(rng.normal(size=(rows, width)), dtype) for _ in range(2)]
+    w, b = (rounded(rng.normal(size=width), torch.float32) for _ in range(2))
+    for d1, d2, bias in ((d[0], d[1], None), (d[0], None, b), (None, d[1], None), (None, None, None)):
+        h = rounded(h64, torch.float32)
+        out = torch.full((rows, width), float("nan"), dtype=dtype, device="cuda")
+        k.add2_layernorm(h, d1, d2, w, bias, out, 1e-3)
+        total = h64 + sum(back(t) for t in (d1, d2) if t is not None)
+        np.testing.assert_allclose(back(h), total, rtol=1e-6, atol=1e-5)
+        want = P.layer_norm(total, back(w), 1e-3) + (back(bias) if bias is not None else 0.0)
+        np.testing.assert_allclose(back(out), want, **(dict(rtol=1e-4, atol=1e-4) if dtype_name == "float32" else dict(rtol=1e-2, atol=1e-2)))
+
+
+@pytest.mark.parametrize("dtype_name", DTYPES)
+@pytest.mark.parametrize("count", [7, 64, 1000])
+def test_exact_gelu_and_the_embedding_factor(dtype_name, count):
+    from mini_llm_runtime_amd.kernels import Kernels
+    dtype = DTYPES[dtype_name]
+    k = Kernels(dtype)
+    x = rounded(np.random.default_rng(count).normal(size=(3, count)) * 2.5, dtype)
+    out = torch.empty_like(x)
+    k.plain_act(x, out, "gelu_erf")
+    np.testing.assert_allclose(back(out), P.gelu_erf(back(x)), **(dict(rtol=1e-5, atol=1e-6) if dtype_name == "float32" else dict(rtol=1e-2, atol=1e-3)))
+    h = torch.empty((2, count), device="cuda")
+    k.embed_gather(ints([2, 0]), x, h, 2.75)
+    np.testing.assert_allclose(back(h), back(x)[[2, 0]] * 2.75, rtol=1e-6)
+
+
+@pytest.mark.parametrize("experts,top,count,keep,scale", [(8, 2, 4, 2, 1.3), (1, 1, 1, 1, 1.0), (5, 5, 1, 1, 0.5), (70, 3, 7, 2, 2.5),
+                                                          (256, 8, 8, 4, 1.0), (12, 4, 12, 4, 1.0), (16, 3, 2, 1, 1.5)])
+def test_softmax_scores_choose_in_the_best_groups(experts, top, count, keep, scale):
+    """Logits in a wider matrix (one more column behind them); among them rows where the best expert's group loses on the
+    sum of two and wins on its largest, and rows of equal logits (the lowest numbers win)."""
+    from mini_llm_runtime_amd.kernels import Kernels
+    k = Kernels(torch.float32)
+    rng = np.random.default_rng(experts)
+    z = rng.normal(size=(40, experts + 1)) * 2.0
+    z[3] = 0.5
+    if count > 1 and experts // count > 1:
+        per = experts // count
+        z[5] = -3.0
+        z[5, per - 1] = 2.0                                # alone in the first group
+        z[5, per:2 * per] = 1.5                            # a group whose two best sum to more
+    z = rounded(z, torch.float32)
+    ids, weights = torch.empty((40, top), dtype=torch.int32, device="cuda"), torch.empty((40, top), device="cuda")
+    k.router_topk(z, ids, weights, count, keep, renormalize=True, scale=scale, score="softmax", group_score="best", experts=experts)
+    # (route() takes x and a router matrix: the identity makes x the logits)
+    want, ww = P.route(back(z)[:, :experts], dict(router=np.eye(experts)), dict(experts=experts, top=top, scale=scale, groups=dict(count=count, keep=keep)))
+    assert np.array_equal(ids.cpu().numpy(), want)
+    np.testing.assert_allclose(back(weights), ww, rtol=1e-5)
+    if count > 1 and experts // count > 1 and keep == 1:
+        assert want[5, 0] == experts // count - 1
+
+
+@pytest.mark.parametrize("dtype_name", DTYPES)
+@pytest.mark.parametrize("rows,experts,hidden,inter", [(5, 3, 40, 16), (300, 4, 64, 48), (2100, 2, 128, 160), (33, 5, 24, 20)])
+def test_clamped_experts_and_the_gated_shared_expert(dtype_name, rows, experts, hidden, inter):
+    """The part itself against the plain mixture: the grouped product with the clamped gate in its epilogue where it takes
+    the sizes, else the row kernel; inputs that reach both clamps of both limits."""
+    from mini_llm_runtime_amd.config.specs import ClampedGluSpec, RoutedMlpSpec
+    from mini_llm_runtime_amd.engine.context import StepContext, Workspace
+    from mini_llm_runtime_amd.kernels import Kernels
+    from mini_llm_runtime_amd.parts import build_part
+    dtype = DTYPES[dtype_name]
+    k = Kernels(dtype)
+    rng = np.random.default_rng(rows)
+    cfg = dict(kind="moe", expert=dict(ff=inter, limit=0.8), shared=dict(ff=24, limit=1.7),
+               router=dict(experts=experts, top=2, scale=1.4, groups=dict(count=1, keep=1)))
+    spec = RoutedMlpSpec("routed_mlp", hidden, inter, experts, 2, 1, 1, "clamped", "softmax", "best", True, gated=True, limit=0.8,
+                         route_scale=1.4, shared=ClampedGluSpec("clamped_glu", hidden, 24, 1.7), shared_gate=True)
+    part = build_part("ffn", spec)
+    weights = {n: rounded(rng.normal(size=ws.shape) * 1.5 * ws.shape[-1] ** -0.5, dtype) for n, ws in part.weight_specs().items()}
+    w64 = {n: back(t) for n, t in weights.items()}
+    x = rounded(rng.normal(size=(rows, hidden)), dtype)
+    near = np.nonzero(P.route_margin(back(x), w64, cfg["router"]) < 4.0)[0]
+    part.bind(weights)
+    k.prepare(part.libraries())
+    ctx = StepContext(k, None, Workspace("cuda"), dtype, 64, 0, 0)
+    got, want = back(part.forward(ctx, x)), P.moe_ffn(back(x), w64, cfg)
+    keep = np.setdiff1d(np.arange(rows), near) if dtype_name == "bfloat16" else np.arange(rows)
+    assert len(keep) > rows // 2
+    err = np.abs(got - want)[keep]
+    assert err.max() <= (2e-5 if dtype_name == "float32" else 3e-2) * np.abs(want).max(), err.max()
+
+
+# ---- one mechanism a model ----------------------------------------------------------------------------------------
+ONE_LAYER = {
+    "attention": dense(attention(6, 3, 8, 16, 4), None),
+    "attention_one_head": dense(attention(1, 1, 16, 16, 16, scaling="none"), None),
+    "attention_many": dense(attention(18, 6, 24, 32, 24, cap=45.0, scaling="slow"), None),
+    "dense": dense(attention(2, 1, 8, 8, 8), 40),
+    "experts": moe(attention(2, 2, 8, 16, 2), 20, 7, 3, 1, 1, 9, limit=0.3),
+    "experts_in_groups": moe(attention(2, 1, 16, 16, 8), 32, 12, 3, 4, 2, 48, limit=3.0, shared_limit=0.5),
+}
+
+
+@pytest.mark.parametrize("dtype_name", DTYPES)
+@pytest.mark.parametrize("name", ONE_LAYER)
+def test_one_layer_models(tmp_path, dtype_name, name):
+    from mini_llm_runtime_amd.config import config_from_dict
+    from mini_llm_runtime_amd.parts import DecoderModel
+    from mini_llm_runtime_amd.weights import write_random_model
+    cfg = model(50, 48, [ONE_LAYER[name]])
+    folder = str(tmp_path)
+    write_random_model(folder, config_from_dict(cfg), seed=1, matrix_std=0.2, norm_std=0.2)
+    loaded = DecoderModel.load(folder, DTYPES[dtype_name])
+    oracle = P.PlainNuvorax(folder)
+    reqs = decisive_requests(oracle, 50, [90, 3], seed=4)
+    want = plain_logits(oracle, reqs)
+    scale = max(float(np.abs(v).max()) for v in want.values())
+    r = runner_for(loaded, 128)
+    close(run_steps(r, whole(reqs)), want, dtype_name, scale)
+    close(run_steps(r, portions(reqs)), want, dtype_name, scale)
+    close(run_steps(r, last_one_by_one(reqs, tail=40)), want, dtype_name, scale)
+    idle(r)
+
+
+# ---- whole models -------------------------------------------------------------------------------------------------
+@pytest.mark.parametrize("dtype_name", DTYPES)
+@pytest.mark.parametrize("name", CONFIGS)
+def test_every_way_of_cutting_gives_the_plain_logits(folders, name, dtype_name):
+    _, reqs, want = plain(folders, name)
+    scale = max(float(np.abs(v).max()) for v in want.values())
+    loaded = load(folders, name, dtype_name)
+    results = {}
+    r = runner_for(loaded, max_tokens=192)          # one request at a time: 150 tokens -> 192
+    for mode, steps in [("whole", whole(reqs)), ("last50", last_one_by_one(reqs, tail=50)), ("portions", portions(reqs))]:
+        results[mode] = run_steps(r, steps)
+        close(results[mode], want, dtype_name, scale)
+        idle(r)
+    steps, peak = mixed(reqs, seed=5)
+    assert max(len(s["entries"]) for s in steps) == 4
+    assert any(min(len(e["tokens"]) for e in s["entries"]) == 1 and max(len(e["tokens"]) for e in s["entries"]) > 1 for s in steps)
+    assert peak < sum(-(-n // 64) * 64 for n in LENGTHS)        # pages and slots are freed and used again
+    r = runner_for(loaded, max_tokens=peak)
+    results["mixed"] = run_steps(r, steps)
+    close(results["mixed"], want, dtype_name, scale)
+    idle(r)
+    # however a request was cut and whatever ran beside it: the float engine takes every sum in an order that follows
+    # from the token alone, so the logits are the same to the bit
+    limit = 0.0 if dtype_name == "float32" else 0.03 * scale
+    for mode in ("last50", "portions", "mixed"):
+        assert max_difference(results["whole"], results[mode]) <= limit, mode
+
+
+@pytest.mark.parametrize("dtype_name", DTYPES)
+@pytest.mark.parametrize("name", ["mix", "odd", "wide"])
+def test_long_decoding_and_the_first_tokens(folders, name, dtype_name):
+    """Five tokens, then 225 one by one, through captured graphs and without, with pages of 4; requests of one, two and
+    three tokens."""
+    oracle, _, _ = plain(folders, name)
+    loaded = load(folders, name, dtype_name)
+    reqs = decisive_requests(oracle, CONFIGS[name]["vocab"], [230, 1, 2, 3], seed=17)
+    want = plain_logits(oracle, reqs)
+    scale = max(float(np.abs(v).max()) for v in want.values())
+    r = runner_for(loaded, max_tokens=256)
+    close(run_steps(r, last_one_by_one(reqs, tail=225)), want, dtype_name, scale)
+    idle(r)
+    r = runner_for(loaded, max_tokens=256, use_graphs=False, page_size=4)
+    close(run_steps(r, last_one_by_one(reqs, tail=225)), want, dtype_name, scale)
+    close(run_steps(r, portions(reqs, sizes=(1, 1, 2, 1, 3, 2))), want, dtype_name, scale)
+    idle(r)
+
+
+def test_portions_of_a_step_that_the_scratch_memory_does_not_hold_at_once(folders, monkeypatch):
+    """Scratch buffers of one group only, and of a few: the step's groups go through several launches."""
+    from mini_llm_runtime_amd.parts import head_mix_attention as part
+    _, reqs, want = plain(folders, "wide")
+    scale = max(float(np.abs(v).max()) for v in want.values())
+    loaded = load(folders, "wide", "bfloat16")
+    steps, peak = mixed(reqs, seed=6)
+    for cap in (1, 3 * 16 * 512 * 32):
+        monkeypatch.setattr(part, "SCRATCH_CAP", cap)
+        r = runner_for(loaded, max_tokens=max(peak, 192))
+        close(run_steps(r, whole(reqs)), want, "bfloat16", scale)
+        close(run_steps(r, steps), want, "bfloat16", scale)
+        idle(r)
+        assert r.workspace.unplanned_bytes() == 0
+
+
+@pytest.mark.parametrize("dtype_name", DTYPES)
+def test_a_slot_used_again_starts_from_nothing(folders, dtype_name):
+    from mini_llm_runtime_amd.engine import Entry
+    oracle, _, _ = plain(folders, "mix")
+    loaded = load(folders, "mix", dtype_name)
+    reqs = decisive_requests(oracle, CONFIGS["mix"]["vocab"], [60, 44], seed=77)
+    r = runner_for(loaded, max_tokens=64)
+    for _ in range(2):
+        for toks in reqs.values():
+            slot = r.open_request()
+            assert slot == 0
+            got = back(r.step([Entry(slot, toks, list(range(len(toks))))]))
+            want = oracle.logits(toks)
+            close(dict(enumerate(got)), dict(enumerate(want)), dtype_name, np.abs(want).max())
+            r.close_request(slot)
+    idle(r)
+
+
+def test_a_far_key_decides_at_real_distances(tmp_path):
+    """A request of 700 tokens: its prompt whole, its last tokens one by one and in portions beside another's, where the
+    scores are sharp (a large scale): far keys among hundreds decide the logits."""
+    from mini_llm_runtime_amd.config import config_from_dict
+    from mini_llm_runtime_amd.parts import DecoderModel
+    from mini_llm_runtime_amd.weights import write_random_model
+    cfg = model(120, 64, [dense(attention(8, 2, 32, 32, 16, base=1e6, scale=1.2), 64), dense(attention(4, 4, 16, 16, 16, scale=1.5), None)])
+    folder = str(tmp_path)
+    write_random_model(folder, config_from_dict(cfg), seed=8, matrix_std=0.15, norm_std=0.2)
+    oracle = P.PlainNuvorax(folder)
+    reqs = make_requests(120, [700, 650], seed=3)
+    want = plain_logits(oracle, reqs)
+    scale = max(float(np.abs(v).max()) for v in want.values())
+    for dtype_name, dtype in DTYPES.items():
+        r = runner_for(DecoderModel.load(folder, dtype), max_tokens=1536, max_length=768, page_size=16)
+        # (sharp scores: a bfloat16 key moves a score by a tenth and more)
+        few = None if dtype_name == "float32" else len(want) // 5
+        close(run_steps(r, whole(reqs)), want, dtype_name, scale, few)
+        close(run_steps(r, last_one_by_one(reqs, tail=60)), want, dtype_name, scale, few)
+        close(run_steps(r, portions(reqs, sizes=(300, 2, 17, 129))), want, dtype_name, scale, few)
+        idle(r)
+
+
+def test_the_stream_after_every_layer(folders):
+    """The 32-bit engine's residual stream behind every layer against the plain model's."""
+    from mini_llm_runtime_amd.engine import Entry
+    oracle, _, _ = plain(folders, "mix")
+    toks = make_requests(CONFIGS["mix"]["vocab"], [21], seed=2)["r0"]
+    want = oracle.streams(toks)
+    r = runner_for(load(folders, "mix", "float32"), max_tokens=64, check_finite=True, use_graphs=False)
+    seen = []
+    original = r.kernels.finite_check
+
+    def recording(h, delta, layer, status):
+        seen.append(back(h) if delta is None else back(h) + back(delta))
+        original(h, delta, layer, status)
+    r.kernels.finite_check = recording
+    r.step([Entry(r.open_request(), toks, [len(toks) - 1])])
+    assert len(seen) == want.shape[0] == 3
+    for i, (got, w) in enumerate(zip(seen, want)):
+        np.testing.assert_allclose(got, w, atol=3e-5 * np.abs(w).max(), rtol=0, err_msg=f"layer {i}")
+
+
+@pytest.mark.parametrize("dtype_name,name", [("float32", "mix"), ("float32", "odd"), ("bfloat16", "wide"), ("bfloat16", "mix")])
+def test_greedy_generation_through_the_scheduler(folders, dtype_name, name):
+    from mini_llm_runtime_amd.api import LLM
+    oracle, _, _ = plain(folders, name)
+    prompts = list(make_requests(CONFIGS[name]["vocab"], [9, 2, 31, 1, 14, 40], seed=23).values())
+    llm = LLM(folders[name], dtype=dtype_name, context_tokens=256, max_model_len=64, max_active=3, batch_tokens=24,
+              prefill_chunk=8, block_size=8)
+    got = llm.generate(prompts, max_tokens=7)
+    for p, g in zip(prompts, got):
+        w = oracle.greedy(p, 7)
+        if g == w:
+            continue
+        assert dtype_name == "bfloat16", (g, w)
+        i = next(j for j in range(7) if g[j] != w[j])                 # bfloat16 may part at a near tie only
+        row = oracle.logits(p + w[:i], [len(p) + i - 1])[0]
+        top = np.sort(row)[-2:]
+        margins = oracle.routing_margins(p + w[:i])
+        assert top[1] - top[0] < 0.05 * np.abs(row).max() or (margins is not None and margins.min() < LEAST), (g, w)
+    assert llm.runner.free_slots() == 3
+
+
+def test_the_command_line_runs_a_random_model(tmp_path):
+    import subprocess
+    import sys
+    from conftest import ROOT
+    from mini_llm_runtime_amd.config import config_from_dict
+    from mini_llm_runtime_amd.weights import write_random_model
+    cfg = os.path.join(str(tmp_path), "config.json")
+    with open(cfg, "w") as f:
+        json.dump(CONFIGS["odd"], f)
+    out = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "mini-llm"), "--random-weights", cfg, "--seed", "3",
+                          "--prompt-ids", "1,2,3,4,5", "--tokens", "5", "--context", "256", "--dtype", "float32"], capture_output=True,
+                         text=True, timeout=600)
+    assert out.returncode == 0, out.stderr[-2000:]
+    report = json.loads(out.stdout[out.stdout.index("{"):])
+    folder = write_random_model(os.path.join(str(tmp_path), "again"), config_from_dict(CONFIGS["odd"]), 3)
+    assert report["input_token_ids"] == [1, 2, 3, 4, 5] and len(report["token_ids"]) == 5
+    if report["dtype"] == "float32":
+        assert report["token_ids"] == P.PlainNuvorax(folder).greedy([1, 2, 3, 4, 5], 5)
+
+
+def test_the_trace_tool_replays_steps(folders, tmp_path):
+    """bin/trace_run on a folder: portions of two requests beside each other, a request that ends and one that takes
+    its slot, logits written per step."""
+    import subprocess
+    import sys
+    from conftest import ROOT
+    oracle, _, _ = plain(folders, "mix")
+    reqs = make_requests(CONFIGS["mix"]["vocab"], [40, 23, 9], seed=41)
+    a, b, c = reqs["r0"], reqs["r1"], reqs["r2"]
+    steps = [dict(step=0, entries=[dict(id="a", tokens=a[:30], want=[0, 29])], end=[]),
+             dict(step=1, entries=[dict(id="a", tokens=a[30:31], want=[0]), dict(id="b", tokens=b[:20], want=[])], end=[]),
+             dict(step=2, entries=[dict(id="b", tokens=b[20:], want=[0, 2]), dict(id="a", tokens=a[31:], want=[8])], end=["a"]),
+             dict(step=3, entries=[dict(id="c", tokens=c, want=[8])], end=["b", "c"])]
+    out_dir = os.path.join(str(tmp_path), "out")
+    os.makedirs(out_dir)
+    run = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", folders["mix"], "--dtype", "float32",
+                          "--out", out_dir, "--max-tokens", "128"], input="".join(json.dumps(s) + "\n" for s in steps),
+                         capture_output=True, text=True, timeout=900)
+    assert run.returncode == 0, run.stderr[-2000:]
+    assert [line for line in run.stdout.splitlines() if line.startswith("done ")] == [f"done {i}" for i in range(4)]
+    vocab = CONFIGS["mix"]["vocab"]
+    rows = {i: np.fromfile(os.path.join(out_dir, f"{i}.f32"), dtype="<f4").reshape(-1, vocab) for i in range(4)}
+    wa, wb, wc = oracle.logits(a), oracle.logits(b), oracle.logits(c)
+    want = {0: wa[[0, 29]], 1: wa[[30]], 2: np.concatenate([wb[[20, 22]], wa[[39]]]), 3: wc[[8]]}
+    for i in range(4):
+        np.testing.assert_allclose(rows[i], want[i], atol=3e-4 * np.abs(wa).max(), rtol=0)
+
+
+def drawn_config(rng):
+    """A configuration drawn at random: head counts in powers of two and not, head sizes that the matrix cores take or
+    not, any order of dense, routed and missing feed-forwards."""
+    width = int(rng.choice([40, 64, 72, 96, 136]))
+    layers = []
+    for _ in range(int(rng.integers(1, 5))):
+        kv = int(rng.choice([1, 2, 3, 4, 6]))
+        dim = int(rng.choice([8, 16, 20, 32, 48, 64, 96]))
+        layer = attention(kv * int(rng.choice([1, 2, 3, 4, 5])), kv, dim, int(rng.choice([8, 16, 32, 48, 80])),
+                          int(rng.choice([r for r in (2, 4, 8, 16, 20, 32, 64) if r <= dim])), cap=float(rng.choice([10.0, 30.0, 50.0, 80.0])),
+                          base=float(rng.choice([100.0, 1e4, 1e6])), scale=float(rng.uniform(0.05, 0.4)),
+                          scaling=str(rng.choice(["middle", "slow", "none"])))
+        kind = rng.random()
+        if kind < 0.3:
+            layers.append(dense(layer, None if kind < 0.1 else int(rng.choice([24, 64, 100]))))
+            continue
+        count, per = int(rng.choice([1, 2, 4])), int(rng.choice([1, 2, 4]))
+        keep = int(rng.integers(1, count + 1))
+        layers.append(moe(layer, int(rng.choice([16, 20, 64])), count * per, int(rng.integers(1, min(4, keep * per) + 1)), count, keep,
+                          int(rng.choice([8, 33, 64])), limit=float(rng.choice([0.5, 1.0, 4.0])), scale=float(rng.choice([1.0, 1.5, 2.5]))))
+    return model(int(rng.choice([33, 100, 257])), width, layers, eps=float(rng.choice([1e-6, 1e-5, 1e-3])),
+                 logit_scale=float(rng.choice([0.5, 1.0, 3.0])), embed=float(rng.choice([1.0, 2.0, 4.0])))
+
+
+@pytest.mark.parametrize("seed", range(10))
+def test_configurations_drawn_at_random(tmp_path, seed):
+    from mini_llm_runtime_amd.config import config_from_dict
+    from mini_llm_runtime_amd.engine import Runner
+    from mini_llm_runtime_amd.parts import DecoderModel
+    from mini_llm_runtime_amd.weights import write_random_model
+    rng = np.random.default_rng(7000 + seed)
+    cfg = drawn_config(rng)
+    folder = str(tmp_path)
+    write_random_model(folder, config_from_dict(cfg), seed=seed, matrix_std=0.1, norm_std=0.2)
+    oracle = P.PlainNuvorax(folder)
+    reqs = decisive_requests(oracle, cfg["vocab"], [90, 37, 5, 64], seed=seed)
+    want = plain_logits(oracle, reqs)
+    scale = max(float(np.abs(v).max()) for v in want.values())
+    page = int(rng.choice([4, 8, 16, 24, 32]))
+    steps, peak = mixed(reqs, seed=seed)
+    for dtype_name in DTYPES:
+        loaded = DecoderModel.load(folder, DTYPES[dtype_name])
+        results = {}
+        for mode, trace, pool in (("whole", whole(reqs), 128), ("portions", portions(reqs), 128), ("mixed", steps, peak)):
+            r = Runner(loaded, max_tokens=pool, max_slots=4, page_size=page, max_length=256, split_keys=64)
+            results[mode] = run_steps(r, trace)
+            close(results[mode], want, dtype_name, scale)
+            r.cache.check()
+            assert r.free_slots() == 4
+        if dtype_name == "float32":
+            assert max_difference(results["whole"], results["portions"]) == 0.0, cfg
+            assert max_difference(results["whole"], results["mixed"]) == 0.0, cfg
