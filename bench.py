@@ -29,6 +29,9 @@ many gigabytes).  Every runner is built with the product's own defaults.  One JS
   * --only budorax: the same for Budorax models (differential attention in blocks of positions, latent attention with a
     gate a head, the gated delta rule with a decay a head, each between two norms and beside a mixture of gated experts;
     two of the six layers run twice), beside a Tigelorn model of equal sizes.
+  * --only nuvorax: the same for Nuvorax models (attention whose heads' weights are mixed, over turned values, beside a
+    dense feed-forward and a mixture of clamped experts with a shared expert in turn), beside a Pamunex model of equal
+    sizes.
 """
 import argparse
 import json
@@ -731,16 +734,82 @@ class BudoraxBench(Bench):
                     frac=round(step_bytes / (seconds / steps) / HBM_PEAK, 5)), step_bytes, report
 
 
+# `--only nuvorax`: layer sizes that resemble a real model's, for a Nuvorax model of eight layers -- attention with mixed
+# heads beside a dense gelu feed-forward (two matrices of one and a half times the inner size) and beside a mixture of
+# eight clamped experts with a shared expert (an expert a quarter of the inner size, of which a token uses two; the shared
+# one half), in turn, one norm a layer -- and for the closest model the engine had before: a Pamunex model (grouped-query and latent attention with a sink, dense and routed feed-forwards, layer norms) of the same width,
+# feed-forward, heads and layers.
+NUVORAX_SIZES = {
+    "2k": dict(width=2048, ff=5632, vocab=32000, layers=8, heads=16, kv_heads=4),
+    "4k": dict(width=4096, ff=12288, vocab=32000, layers=8, heads=32, kv_heads=8),
+}
+
+
+class NuvoraxBench(Bench):
+    """A Nuvorax model of NUVORAX_SIZES[size] with random weights drawn on the GPU."""
+    EXPERTS, TOP = 8, 2
+
+    def __init__(self, size, args):
+        import torch
+        from mini_llm_runtime_amd.api import parse_dtype
+        from mini_llm_runtime_amd.config import config_from_dict
+        from mini_llm_runtime_amd.parts import DecoderModel, expected_tensors
+        from mini_llm_runtime_amd.weights import random_tensors_on_device
+        d = NUVORAX_SIZES[size]
+        self.torch, self.args, self.size = torch, args, size
+        self.dtype = parse_dtype(args.dtype)
+        self.tag = "bf16" if self.dtype == torch.bfloat16 else "fp32"
+        h, w, ff = d["heads"], d["width"], d["ff"]
+        mixer = dict(heads=h, kv_heads=d["kv_heads"], dim=128, vdim=128, scale=128 ** -0.5, softcap=30.0,
+                     rot=dict(dims=64, base=1000000.0, scaling=dict(factor=8.0, low=1.0, high=4.0, original=8192)))
+        mlps = [dict(kind="dense", ff=ff * 3 // 2),
+                dict(kind="moe", expert=dict(ff=ff // 4, limit=7.0), shared=dict(ff=ff // 2, limit=7.0),
+                     router=dict(experts=self.EXPERTS, top=self.TOP, scale=1.5, groups=dict(count=4, keep=2)))]
+        self.layers = self.full_layers = d["layers"]
+        layers = [dict(type="attention", mixer=mixer, mlp=mlps[i % 2]) for i in range(self.layers)]
+        self.cfg = config_from_dict(dict(architecture="Nuvorax", vocab=d["vocab"], width=w, norm=dict(eps=1e-5),
+                                         embedding=dict(scale=8.0), logit_scale=0.5, layers=layers))
+        self.model = DecoderModel(self.cfg, random_tensors_on_device(expected_tensors(self.cfg), 0, self.dtype, "cuda"),
+                                  self.dtype, "cuda:0")
+        self.weights_from = "drawn on the GPU"
+        self.elem = 2 if self.dtype == torch.bfloat16 else 4
+        n_moe = self.layers // 2
+        expert, shared = 3 * w * (ff // 4), 3 * w * (ff // 2)
+        attention = w * h * 128 + w * d["kv_heads"] * 256 + h * w + w * h * 128
+        self.common = self.layers * attention + (self.layers - n_moe) * 2 * w * (ff * 3 // 2) + n_moe * (shared + self.EXPERTS * w)
+        self.expert, self.n_moe = expert, n_moe
+        self.matrix_params = self.common + n_moe * self.TOP * expert
+        self.weight_bytes = (self.common + n_moe * self.EXPERTS * expert + d["vocab"] * w) * self.elem   # (of the table a row a token)
+        self.kv_bytes_per_token = self.layers * d["kv_heads"] * 256 * self.elem
+        # a pair (query, key): scores and values a head, and the mixing of the heads
+        self.attention_flops = lambda t: self.layers * 2.0 * (t * (t + 1) / 2) * (h * 256 + h * h)
+        self.vocab = d["vocab"]
+        self.g = torch.Generator().manual_seed(0)
+
+    def prefill_flops(self, t):
+        d = NUVORAX_SIZES[self.size]
+        return 2.0 * t * self.matrix_params + self.attention_flops(t) + 2.0 * d["vocab"] * d["width"]
+
+    def decode_point(self, batch, steps, warmup, context=None):
+        d = NUVORAX_SIZES[self.size]
+        seconds, mean_context, report = self.decode(batch, steps, warmup, context)
+        touched = self.EXPERTS * (1.0 - (1.0 - self.TOP / self.EXPERTS) ** batch)      # experts that a step's tokens choose, about
+        weights = (self.common + self.n_moe * touched * self.expert + d["vocab"] * d["width"]) * self.elem
+        step_bytes = weights + batch * mean_context * self.kv_bytes_per_token
+        return dict(tok_s=round(batch * steps / seconds, 1), ms=round(seconds / steps * 1e3, 4),
+                    frac=round(step_bytes / (seconds / steps) / HBM_PEAK, 5)), step_bytes, report
+
+
 def design_block(args):
     """Prefill (2048 tokens in one step) and decode (batch 8 and 64 behind --context tokens) of a design's sizes
     beside the closest model the engine had before it (a Qwen3 dense model of equal width, heads, feed-forward and
-    layers; for Tigelorn a Taletar model of equal sizes); then the same steps once more with events around every
+    layers; for Tigelorn a Taletar model, for Budorax a Tigelorn model, for Nuvorax a Pamunex model of equal sizes); then the same steps once more with events around every
     launch: milliseconds per kernel class."""
     import copy
     out = {}
     design = getattr(args, "design", "taletar")
     table, make_design = {"pamunex": (PAMUNEX_SIZES, PamunexBench), "tigelorn": (TIGELORN_SIZES, TigelornBench),
-                          "budorax": (BUDORAX_SIZES, BudoraxBench)}.get(design, (DESIGN_SIZES, TaletarBench))
+                          "budorax": (BUDORAX_SIZES, BudoraxBench), "nuvorax": (NUVORAX_SIZES, NuvoraxBench)}.get(design, (DESIGN_SIZES, TaletarBench))
     for size in (args.design_sizes.split(",") if args.design_sizes else list(table)):
         d = table[size]
         dense = (d["layers"], dict(hidden_size=d["width"], num_attention_heads=d["heads"], num_key_value_heads=d["kv_heads"],
@@ -750,6 +819,7 @@ def design_block(args):
         block = {}
         beside = ("taletar", lambda a: TaletarBench(size, a)) if design == "tigelorn" else \
             ("tigelorn", lambda a: TigelornBench(size, a)) if design == "budorax" else \
+            ("pamunex", lambda a: PamunexBench(size, a)) if design == "nuvorax" else \
             ("qwen3_dense", lambda a: Bench(size, 0, a, sizes=dense))
         for name, make in ((design, lambda a: make_design(size, a)), beside):
             plain_args, profiled = copy.copy(args), copy.copy(args)
@@ -792,12 +862,13 @@ def main():
                          "tensors drawn on the GPU; auto: folder for the 0.6B sizes, gpu for the larger ones")
     ap.add_argument("--warm-up", type=int, default=0,
                     help="--only engine: 1 captures the decoding steps (Engine.warm_up) before the first burst")
-    ap.add_argument("--only", default="all", choices=["all", "decode", "prefill", "prompt", "engine", "mixed", "taletar", "pamunex", "tigelorn", "budorax"],
+    ap.add_argument("--only", default="all", choices=["all", "decode", "prefill", "prompt", "engine", "mixed", "taletar", "pamunex", "tigelorn", "budorax",
+                                                         "nuvorax"],
                     help="profiling aid: run just the decode steps, just the prefill or just the mixed step; prompt: one "
                          "prompt of --context tokens in portions of 2048; engine: the "
                          "scheduler over a burst of requests (3 x batch requests of 512 prompt and 128 output tokens, "
                          "batch slots), printed as one line of its own")
-    ap.add_argument("--design-sizes", default="", help="--only taletar / pamunex / tigelorn / budorax: which of its sizes (2k, 4k; default both)")
+    ap.add_argument("--design-sizes", default="", help="--only taletar / pamunex / tigelorn / budorax / nuvorax: which of its sizes (2k, 4k; default both)")
     ap.add_argument("--library", type=int, default=1,
                     help="0: every matrix product on the hand-written kernels, none in the vendor library")
     ap.add_argument("--split-keys", type=int, default=256, help="the smallest range of keys of one attention workgroup")
@@ -821,7 +892,7 @@ def main():
     if not args.tune:
         from mini_llm_runtime_amd.kernels import build
         build.load("library_gemm").mlr_library_gemm_tuning(0)
-    if args.only in ("taletar", "pamunex", "tigelorn", "budorax"):
+    if args.only in ("taletar", "pamunex", "tigelorn", "budorax", "nuvorax"):
         args.design = args.only
         print(json.dumps({f"{args.only}_sizes": design_block(args), "context": args.context, "dtype": args.dtype}))
         return 0

@@ -82,7 +82,7 @@ def _mlp(mlp, width, where):
         shared = ClampedGluSpec("clamped_glu", width, _int(sh, "ff", where + ".shared."),
                                 _num(sh, "limit", where + ".shared.", positive=True), GATE_SLOPE)
     return RoutedMlpSpec("routed_mlp", width, _int(expert, "ff", where + ".expert."), experts, top, count, keep, "clamped",
-                         "softmax", "best", True, gated=True, limit=_num(expert, "limit", where + ".expert.", positive=True),
+                         "softmax", True, gated=True, group_score="best", limit=_num(expert, "limit", where + ".expert.", positive=True),
                          slope=GATE_SLOPE, route_scale=_num(router, "scale", where + ".router.", default=1.0), shared=shared,
                          shared_gate=shared is not None)
 

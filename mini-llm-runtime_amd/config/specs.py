@@ -291,11 +291,11 @@ class RoutedMlpSpec:
     group_keep: int = 1
     activation: str = "relu_squared"
     score: str = "sigmoid"        # or "softmax"
-    group_score: str = "best_two" # or "best"
     renormalize: bool = False
     gated: bool = False           # an expert is down(act(gate x) * (up x)) with tensors e<i>.gate beside e<i>.up
     correction: bool = False      # the choice goes by s + a stored number an expert (`correction`), the weights by s
     route_scale: float = 1.0      # factor on the chosen weights
+    group_score: str = "best_two"         # of the two largest scores, or "best": of the largest
     limit: Optional[float] = None         # activation "clamped": g = min(gate, limit), u = clamp(up, -limit, limit),
     slope: float = 1.702                  # g sigmoid(slope g) (u + 1)
     shared: Optional[object] = None       # any feed-forward spec; its tensors are named `shared.<local name>`

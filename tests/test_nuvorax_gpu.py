@@ -420,7 +420,7 @@ def test_clamped_experts_and_the_gated_shared_expert(dtype_name, rows, experts, 
     rng = np.random.default_rng(rows)
     cfg = dict(kind="moe", expert=dict(ff=inter, limit=0.8), shared=dict(ff=24, limit=1.7),
                router=dict(experts=experts, top=2, scale=1.4, groups=dict(count=1, keep=1)))
-    spec = RoutedMlpSpec("routed_mlp", hidden, inter, experts, 2, 1, 1, "clamped", "softmax", "best", True, gated=True, limit=0.8,
+    spec = RoutedMlpSpec("routed_mlp", hidden, inter, experts, 2, 1, 1, "clamped", "softmax", True, gated=True, group_score="best", limit=0.8,
                          route_scale=1.4, shared=ClampedGluSpec("clamped_glu", hidden, 24, 1.7), shared_gate=True)
     part = build_part("ffn", spec)
     weights = {n: rounded(rng.normal(size=ws.shape) * 1.5 * ws.shape[-1] ** -0.5, dtype) for n, ws in part.weight_specs().items()}
