@@ -164,10 +164,20 @@ __global__ __launch_bounds__(256) void head_mix_attention_kernel(HeadMixArgs a) 
 // each half), which is the operand of the product with the values.
 typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8;
 typedef __attribute__((__vector_size__(4 * sizeof(__bf16)))) __bf16 bf16x4;
+typedef __attribute__((__vector_size__(2 * sizeof(__bf16)))) __bf16 bf16x2;
 typedef __attribute__((__vector_size__(4 * sizeof(short)))) short shortx4;
 typedef __attribute__((__vector_size__(4 * sizeof(float)))) float floatx4;
 
 #define TK 32                   // keys in a tile
+
+// The product that mixes the heads: four heads a lane (inner size 16) or eight (32).
+__device__ __forceinline__ floatx4 mixed(bf16x4 p, bf16x8 m, floatx4 d) {
+    const bf16x4 m4 = {m[0], m[1], m[2], m[3]};
+    return __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(__builtin_bit_cast(shortx4, p), __builtin_bit_cast(shortx4, m4), d, 0, 0, 0);
+}
+__device__ __forceinline__ floatx4 mixed(bf16x8 p, bf16x8 m, floatx4 d) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(p, m, d, 0, 0, 0);
+}
 
 struct TileArgs {
     const int32_t* group_first; const int32_t* group_count;
@@ -175,12 +185,9 @@ struct TileArgs {
     __bf16* e;                                 // [groups * NQ][ktiles][...]
     float* sums;                               // [groups * NQ][head_k][score_ranges]
     float* partial;                            // [groups * NQ][q_heads][value_ranges][value_dim]
-    int ktiles, hp_log, head_k, kv_pad;
+    int ktiles, hp_log, head_k, kv_pad, page_log;
     int score_keys, score_ranges, value_keys, value_ranges;      // keys of a range (multiples of 32), ranges
 };
-
-// Elements between the scratch of one key tile and the next of a token row.
-__device__ __forceinline__ size_t tile_elems(int head_k) { return (size_t)TK * head_k; }
 
 // Where heads idx .. of key place i (0..15) of half s of a tile lie, from the tile's first element.
 __device__ __forceinline__ int e_place(int head_k, int idx, int s, int i) {
@@ -188,25 +195,37 @@ __device__ __forceinline__ int e_place(int head_k, int idx, int s, int i) {
     return ((idx >> 5) * 2 + s) * 512 + (((idx >> 3) & 3) * 16 + i) * 8 + (idx & 7);
 }
 
+// Which page a key lies in and its place there; page_log: log2(page_size), or -1 where that is no power of two.
+struct PageOf {
+    int page_size, page_log;
+    __device__ __forceinline__ int block(int key) const { return page_log >= 0 ? key >> page_log : key / page_size; }
+    __device__ __forceinline__ int place(int key) const { return page_log >= 0 ? key & (page_size - 1) : key % page_size; }
+};
+
 // One workgroup: a group's tokens x up to 16 RT rows (token, head of one kv head) x a range of keys; each of the four
 // wavefronts takes every fourth tile of 32 keys.  Rows are the first operand (a lane ends up with four rows of one
-// key: four heads of a token where a kv head has four), keys the second, straight from the pages.
-template <int NKF, int RT>
+// key: four heads of a token where a kv head has four), keys the second, straight from the pages: the next tile's rows
+// are on their way while a tile's exponentials are taken, and the ids of the pages after that.
+// HPL: log2 of the places a kv head's heads take, 2 for all from four on (a lane's four rows are then one token's).
+template <int NKF, int RT, int HPL>
 __global__ __launch_bounds__(256) void head_scores_kernel(HeadMixArgs a, TileArgs t) {
+    constexpr int TOKENS = HPL == 0 ? 4 : HPL == 1 ? 2 : 1, PER = 4 / TOKENS;      // tokens of a lane's four rows; rows a token
     __shared__ float sum_lds[4][RT * 16];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, i16 = lane & 15, b = lane >> 4;
     const int g = (int)gridDim.x - 1 - (int)blockIdx.x;        // (a prompt's last groups have the most keys: first)
     const int kvh = blockIdx.y % t.kv_pad, row0 = (blockIdx.y / t.kv_pad) * RT * 16;
     const int first = t.group_first[g], count = t.group_count[g];
-    const int hp = 1 << t.hp_log, hg = a.q_heads / a.kv_heads, D = a.key_dim, PS = a.page_size;
+    const int hp_log = HPL < 2 ? HPL : t.hp_log, hp = 1 << hp_log, hg = a.q_heads / a.kv_heads, D = a.key_dim;
+    const PageOf pages{a.page_size, t.page_log};
     const int p0 = a.positions[first], kend = p0 + count;
     const int32_t* table = a.block_table + (size_t)a.slots[first] * a.max_blocks;
     const bool real = kvh < a.kv_heads;
+    const bool padded = !real || hg != hp;     // rows that stand for no head
     const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
     bf16x8 qf[RT][NKF];
 #pragma unroll
     for (int r = 0; r < RT; ++r) {
-        const int row = row0 + r * 16 + i16, ti = row >> t.hp_log, hh = row & (hp - 1);
+        const int row = row0 + r * 16 + i16, ti = row >> hp_log, hh = row & (hp - 1);
         const bool ok = real && ti < count && hh < hg;
         const __bf16* src = a.q + (size_t)(first + (ok ? ti : 0)) * a.q_stride + (size_t)(ok ? kvh * hg + hh : 0) * D;
 #pragma unroll
@@ -216,23 +235,43 @@ __global__ __launch_bounds__(256) void head_scores_kernel(HeadMixArgs a, TileArg
             qf[r][kf] = (ok && d < D) ? v : zero8;
         }
     }
+    const int kt_step = t.score_keys / TK;
+    const int kt_end = min((kend + TK - 1) / TK, ((int)blockIdx.z + 1) * kt_step);
+    int kt = (int)blockIdx.z * kt_step + wave;
+    const int te = TK * t.head_k, half = t.head_k == 16 ? 256 : 512;       // elements of a tile, of its half (one step of heads)
+    // where the lane's rows go (tokens beyond the group's have no scratch; padded heads store their zeros)
+    __bf16* dst[RT][TOKENS];
+    bool stored[RT][TOKENS];
+#pragma unroll
+    for (int r = 0; r < RT; ++r)
+#pragma unroll
+        for (int x = 0; x < TOKENS; ++x) {
+            const int row = row0 + r * 16 + 4 * b + x * PER, ti = row >> hp_log;
+            stored[r][x] = ti < count;
+            dst[r][x] = t.e + (((size_t)g * t.group_tokens + ti) * t.ktiles + kt) * te +
+                        e_place(t.head_k, kvh * hp + (row & (hp - 1)), 0, i16);
+        }
     float sums[RT][4];
 #pragma unroll
     for (int r = 0; r < RT; ++r)
 #pragma unroll
         for (int x = 0; x < 4; ++x) sums[r][x] = 0.f;
     // exp(cap tanh(x scale / cap)) = 2^(c1 - 2 c1 / (1 + 2^(x k))), c1 = cap log2(e), k = 2 log2(e) scale / cap
-    const float c1 = a.softcap * 1.4426950408889634f, c2 = 2.0f * c1, kx = 2.0f * 1.4426950408889634f * (a.scale / a.softcap);
-    const int kt_end = min((kend + TK - 1) / TK, ((int)blockIdx.z + 1) * (t.score_keys / TK));
-    const __bf16* kbase = a.k_pages + (size_t)(real ? kvh : 0) * PS * D;
-    const size_t page_elems = (size_t)a.kv_heads * PS * D;
+    const float c1 = a.softcap * 1.4426950408889634f, c2 = -2.0f * c1, kx = 2.0f * 1.4426950408889634f * (a.scale / a.softcap);
+    const __bf16* kbase = a.k_pages + (size_t)(real ? kvh : 0) * a.page_size * D;
+    const size_t page_elems = (size_t)a.kv_heads * a.page_size * D;
+    const int lane_key = 8 * (i16 >> 2) + (i16 & 3);           // of the tile's first half; + 4: of its second
     bf16x8 kreg[2][NKF];
-    auto fetch = [&](int kt) {                 // (clamped addresses: loads that wait for nothing)
+    int page[2];
+    auto ask = [&](int kt) {                   // (clamped: loads behind no branch)
+#pragma unroll
+        for (int s = 0; s < 2; ++s) page[s] = table[pages.block(min(kt * TK + lane_key + 4 * s, kend - 1))];
+    };
+    auto fetch = [&](int kt) {
 #pragma unroll
         for (int s = 0; s < 2; ++s) {
-            const int key = min(kt * TK + 8 * (i16 >> 2) + 4 * s + (i16 & 3), kend - 1);
-            const int page = max(table[key / PS], 0);
-            const __bf16* kr = kbase + (size_t)page * page_elems + (size_t)(key % PS) * D;
+            const int key = min(kt * TK + lane_key + 4 * s, kend - 1);
+            const __bf16* kr = kbase + (size_t)max(page[s], 0) * page_elems + (size_t)pages.place(key) * D;
 #pragma unroll
             for (int kf = 0; kf < NKF; ++kf) {
                 const int d = kf * 32 + b * 8;
@@ -241,8 +280,11 @@ __global__ __launch_bounds__(256) void head_scores_kernel(HeadMixArgs a, TileArg
             }
         }
     };
-    int kt = (int)blockIdx.z * (t.score_keys / TK) + wave;
-    if (kt < kt_end) fetch(kt);
+    if (kt < kt_end) {
+        ask(kt);
+        fetch(kt);
+        ask(kt + 4);
+    }
     for (; kt < kt_end; kt += 4) {
         floatx4 sc[RT][2];
 #pragma unroll
@@ -254,43 +296,45 @@ __global__ __launch_bounds__(256) void head_scores_kernel(HeadMixArgs a, TileArg
                 for (int kf = 0; kf < NKF; ++kf) x = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[r][kf], kreg[s][kf], x, 0, 0, 0);
                 sc[r][s] = x;
             }
-        if (kt + 4 < kt_end) fetch(kt + 4);
+        fetch(kt + 4);
+        ask(kt + 8);
+        // (the same in every lane: a tile that every token sees whole, no rows that stand for nothing)
+        const bool plain = !padded && kt * TK + TK - 1 <= p0;
 #pragma unroll
         for (int r = 0; r < RT; ++r) {
             const int row = row0 + r * 16 + 4 * b;               // the lane's rows row .. row + 3
 #pragma unroll
             for (int s = 0; s < 2; ++s) {
-                const int key = kt * TK + 8 * (i16 >> 2) + 4 * s + (i16 & 3);
+                float e[4];
+#pragma unroll
+                for (int x = 0; x < 4; ++x) {
+                    const float z = __builtin_amdgcn_exp2f(kx * sc[r][s][x]);
+                    e[x] = __builtin_amdgcn_exp2f(__builtin_fmaf(c2, __builtin_amdgcn_rcpf(1.0f + z), c1));
+                }
+                if (!plain) {
+                    const int key = kt * TK + lane_key + 4 * s - p0;
+#pragma unroll
+                    for (int x = 0; x < 4; ++x) {
+                        const bool seen = real && ((row + x) & (hp - 1)) < hg && key <= ((row + x) >> hp_log);
+                        e[x] = __uint_as_float(__float_as_uint(e[x]) & (seen ? 0xffffffffu : 0u));
+                    }
+                }
                 bf16x4 e4;
 #pragma unroll
                 for (int x = 0; x < 4; ++x) {
-                    const int ti = (row + x) >> t.hp_log, hh = (row + x) & (hp - 1);
-                    const bool seen = real && hh < hg && key <= p0 + ti;
-                    const float z = __builtin_amdgcn_exp2f(kx * sc[r][s][x]);
-                    const float e = seen ? __builtin_amdgcn_exp2f(c1 - c2 * __builtin_amdgcn_rcpf(1.0f + z)) : 0.f;
-                    sums[r][x] += e;
-                    e4[x] = (__bf16)e;
+                    sums[r][x] += e[x];
+                    e4[x] = (__bf16)e[x];
                 }
-                // (tokens beyond the group's have no scratch; padded heads store their zeros)
-                const int idx = kvh * hp;
-                auto at = [&](int ti, int hh) {
-                    return t.e + ((size_t)g * t.group_tokens + ti) * t.ktiles * tile_elems(t.head_k) +
-                           (size_t)kt * tile_elems(t.head_k) + e_place(t.head_k, idx + hh, s, i16);
-                };
-                if (hp >= 4) {
-                    const int ti = row >> t.hp_log;
-                    if (ti < count) *reinterpret_cast<bf16x4*>(at(ti, row & (hp - 1))) = e4;
-                } else if (hp == 2) {
-                    const int ti = row >> 1;
-                    typedef __attribute__((__vector_size__(2 * sizeof(__bf16)))) __bf16 bf16x2;
-                    if (ti < count) *reinterpret_cast<bf16x2*>(at(ti, 0)) = bf16x2{e4[0], e4[1]};
-                    if (ti + 1 < count) *reinterpret_cast<bf16x2*>(at(ti + 1, 0)) = bf16x2{e4[2], e4[3]};
-                } else {
 #pragma unroll
-                    for (int x = 0; x < 4; ++x)
-                        if (row + x < count) *at(row + x, 0) = e4[x];
+                for (int x = 0; x < TOKENS; ++x) {
+                    if (!stored[r][x]) continue;
+                    if (PER == 4) *reinterpret_cast<bf16x4*>(dst[r][x] + s * half) = e4;
+                    else if (PER == 2) *reinterpret_cast<bf16x2*>(dst[r][x] + s * half) = bf16x2{e4[(2 * x) & 3], e4[(2 * x + 1) & 3]};
+                    else dst[r][x][s * half] = e4[x];
                 }
             }
+#pragma unroll
+            for (int x = 0; x < TOKENS; ++x) dst[r][x] += 4 * te;
         }
     }
     // a row's sum: over its 16 lanes, then over the wavefronts
@@ -305,7 +349,7 @@ __global__ __launch_bounds__(256) void head_scores_kernel(HeadMixArgs a, TileArg
         }
     __syncthreads();
     for (int r = tid; r < RT * 16; r += 256) {
-        const int row = row0 + r, ti = row >> t.hp_log, hh = row & (hp - 1);
+        const int row = row0 + r, ti = row >> hp_log, hh = row & (hp - 1);
         if (ti < count)
             t.sums[(((size_t)g * t.group_tokens + ti) * t.head_k + kvh * hp + hh) * t.score_ranges + blockIdx.z] =
                 (sum_lds[0][r] + sum_lds[1][r]) + (sum_lds[2][r] + sum_lds[3][r]);
@@ -380,58 +424,76 @@ __global__ __launch_bounds__(512) void head_mix_values_kernel(HeadMixArgs a, Til
         for (int v = 0; v < VT; ++v) acc[c][v] = floatx4{0.f, 0.f, 0.f, 0.f};
     const int kt_first = (int)blockIdx.z * (t.value_keys / TK);
     const int kt_end = min((kend + TK - 1) / TK, kt_first + t.value_keys / TK);
-    const size_t te = tile_elems(head_k);
+    const size_t te = (size_t)TK * head_k;
     const __bf16* e_group = t.e + (size_t)g * t.group_tokens * t.ktiles * te;
+    const PageOf pages{PS, t.page_log};
     const __bf16* vbase = a.v_pages + (size_t)(kvh < a.kv_heads ? kvh : 0) * V * PS;
     const size_t page_elems = (size_t)a.kv_heads * V * PS;
-    const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
 
+    const bool pv = kvh < a.kv_heads;
+    // this lane's eight keys of a tile lie in one page: its id, and the transposed rows from there
+    auto page_of = [&](int kt) { return table[pages.block(min(kt * TK + 8 * b, (kend - 1) & ~7))]; };
+    auto values = [&](int kt, int page, bf16x8 (&vf)[VT]) {
+        const int key = kt * TK + 8 * b;
+        const __bf16* vr = vbase + (size_t)max(page, 0) * page_elems + pages.place(min(key, (kend - 1) & ~7));
+#pragma unroll
+        for (int v = 0; v < VT; ++v) vf[v] = *reinterpret_cast<const bf16x8*>(vr + (size_t)min((vpart + vs * v) * 16 + i16, V - 1) * PS);
+    };
+    // (places behind the last key hold anything)
+    auto cut = [&](int kt, bf16x8 (&vf)[VT]) {
+        if (kt * TK + TK <= kend) return;
+        const int left = kend - (kt * TK + 8 * b);
+#pragma unroll
+        for (int v = 0; v < VT; ++v)
+#pragma unroll
+            for (int j = 0; j < 8; ++j)
+                if (j >= left) vf[v][j] = (__bf16)0.f;
+    };
+    // the scratch of this wavefront's units of a turn (one step of heads: on its way a turn ahead)
+    constexpr int EW = HK == 16 ? 4 : 8;
+    typedef __attribute__((__vector_size__(EW * sizeof(__bf16)))) __bf16 bf16xe;
+    bf16xe ereg[UPW][2];
+    auto exps = [&](int kt0) {
+        if (HK == 0) return;
+#pragma unroll
+        for (int u = 0; u < UPW; ++u) {
+            const int unit = wave * UPW + u, ti = NQ == 16 ? min(unit, count - 1) : 0, kt = min(NQ == 16 ? kt0 : kt0 + unit, kt_end - 1);
+            const __bf16* src = e_group + ((size_t)ti * t.ktiles + kt) * te + lane * EW;
+#pragma unroll
+            for (int s = 0; s < 2; ++s) ereg[u][s] = *reinterpret_cast<const bf16xe*>(src + s * 64 * EW);
+        }
+    };
+    if (kt_first < kt_end) exps(kt_first);
+    int page = kt_first < kt_end ? page_of(kt_first) : 0;
     int turn = 0;
     for (int kt0 = kt_first; kt0 < kt_end; kt0 += KSUB, turn ^= 1) {
         __bf16* wb = w_lds + turn * buffer;
+        bf16x8 vf[VT];
+        values(kt0, page, vf);                 // (on their way while the heads are mixed)
+        if (NQ == 16) page = page_of(kt0 + 1);
 #pragma unroll
         for (int u = 0; u < UPW; ++u) {
             const int unit = wave * UPW + u, ti = NQ == 16 ? unit : 0, kt = NQ == 16 ? kt0 : kt0 + unit;
             if (ti >= count || kt >= kt_end) continue;           // (the same in every lane)
-            const __bf16* src = e_group + ((size_t)ti * t.ktiles + kt) * te;
             floatx4 d[2][2];
 #pragma unroll
             for (int n = 0; n < 2; ++n)
 #pragma unroll
                 for (int s = 0; s < 2; ++s) d[n][s] = floatx4{0.f, 0.f, 0.f, 0.f};
-            if (HK == 16) {
+            for (int st = 0; st < steps; ++st) {
+                float f[PER];
+#pragma unroll
+                for (int j = 0; j < PER; ++j) f[j] = HK == 0 ? inv_lds[ti * head_k + st * 32 + b * 8 + j] : inv[u][j];
 #pragma unroll
                 for (int s = 0; s < 2; ++s) {
-                    const bf16x4 e4 = *reinterpret_cast<const bf16x4*>(src + s * 256 + lane * 4);
-                    bf16x4 p4;
+                    bf16xe ev = ereg[u][s];
+                    if (HK == 0) ev = *reinterpret_cast<const bf16xe*>(e_group + ((size_t)ti * t.ktiles + kt) * te + (st * 2 + s) * 512 + lane * EW);
+                    bf16xe p;
 #pragma unroll
-                    for (int j = 0; j < 4; ++j) p4[j] = (__bf16)((float)e4[j] * inv[u][j]);
+                    for (int j = 0; j < PER; ++j) p[j] = (__bf16)((float)ev[j] * f[j]);
 #pragma unroll
                     for (int n = 0; n < 2; ++n)
-                        if (n * 16 < kv_block * hp) {
-                            const bf16x4 m4 = {mixf[n][0], mixf[n][1], mixf[n][2], mixf[n][3]};
-                            d[n][s] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(__builtin_bit_cast(shortx4, p4),
-                                                                                __builtin_bit_cast(shortx4, m4), d[n][s], 0, 0, 0);
-                        }
-                }
-            } else {
-                for (int st = 0; st < steps; ++st) {
-                    float f[8];
-#pragma unroll
-                    for (int j = 0; j < 8; ++j) f[j] = HK == 0 ? inv_lds[ti * head_k + st * 32 + b * 8 + j] : inv[u][j % PER];
-#pragma unroll
-                    for (int s = 0; s < 2; ++s) {
-                        const bf16x8 e8 = *reinterpret_cast<const bf16x8*>(src + (st * 2 + s) * 512 + lane * 8);
-                        bf16x8 p8;
-#pragma unroll
-                        for (int j = 0; j < 8; ++j) p8[j] = (__bf16)((float)e8[j] * f[j]);
-#pragma unroll
-                        for (int n = 0; n < 2; ++n)
-                            if (n * 16 < kv_block * hp) {
-                                const bf16x8 m8 = HK == 0 ? *reinterpret_cast<const bf16x8*>(mix_lds + ((st * 2 + n) * 64 + lane) * 8) : mixf[n];
-                                d[n][s] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p8, m8, d[n][s], 0, 0, 0);
-                            }
-                    }
+                        if (n * 16 < kv_block * hp) d[n][s] = mixed(p, HK == 0 ? *reinterpret_cast<const bf16x8*>(mix_lds + ((st * 2 + n) * 64 + lane) * 8) : mixf[n], d[n][s]);
                 }
             }
             // lane: head i16 of the column tile, keys 8 b .. 8 b + 7
@@ -447,26 +509,18 @@ __global__ __launch_bounds__(512) void head_mix_values_kernel(HeadMixArgs a, Til
                 }
             }
         }
+        exps(kt0 + KSUB);
         __syncthreads();
-        if (kvh < a.kv_heads) {
+        if (pv) {
 #pragma unroll 1
             for (int sub = 0; sub < KSUB; ++sub) {
                 const int kt = kt0 + sub;
                 if (kt >= kt_end) break;
-                const int key = kt * TK + 8 * b, kc = min(key, (kend - 1) / 8 * 8);      // (eight keys lie in one page)
-                const int page = max(table[kc / PS], 0);
-                const __bf16* vr = vbase + (size_t)page * page_elems + kc % PS;
-                const bool tail = kt * TK + TK > kend;           // (places behind the last key hold anything)
-                bf16x8 vf[VT];
-#pragma unroll
-                for (int v = 0; v < VT; ++v) {
-                    const int ch = (vpart + vs * v) * 16 + i16;
-                    vf[v] = *reinterpret_cast<const bf16x8*>(vr + (size_t)min(ch, V - 1) * PS);
-                    if (tail)
-#pragma unroll
-                        for (int j = 0; j < 8; ++j)
-                            if (key + j >= kend) vf[v][j] = (__bf16)0.f;
+                if (NQ != 16) {
+                    // (single tokens: the next tile's values on their way while this one's are multiplied)
+                    page = page_of(kt + 1);
                 }
+                cut(kt, vf);
                 const __bf16* wr = wb + (gl * block_rows + (NQ == 16 ? 0 : sub * hp)) * TK + 8 * b;
 #pragma unroll
                 for (int c = 0; c < CT; ++c) {
@@ -477,6 +531,7 @@ __global__ __launch_bounds__(512) void head_mix_values_kernel(HeadMixArgs a, Til
                     for (int v = 0; v < VT; ++v)
                         if ((vpart + vs * v) * 16 < V) acc[c][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[v], wf, acc[c][v], 0, 0, 0);
                 }
+                if (NQ != 16 && sub + 1 < KSUB) values(kt + 1, page, vf);
             }
         }
     }
@@ -494,7 +549,8 @@ __global__ __launch_bounds__(512) void head_mix_values_kernel(HeadMixArgs a, Til
     }
 }
 
-// The ranges' shares added in ascending order, turned back, gated: one workgroup a token of a group.
+// The ranges' shares added in ascending order, turned back, gated: a workgroup takes 256 channel pairs of a token of a
+// group.
 __global__ __launch_bounds__(256) void head_mix_finish_kernel(HeadMixArgs a, TileArgs t) {
     const int g = blockIdx.x, ti = blockIdx.y, V = a.value_dim, half = V >> 1;
     if (ti >= t.group_count[g]) return;
@@ -502,7 +558,8 @@ __global__ __launch_bounds__(256) void head_mix_finish_kernel(HeadMixArgs a, Til
     const float* base = t.partial + ((size_t)g * t.group_tokens + ti) * a.q_heads * t.value_ranges * V;
     const int used = min(t.value_ranges, (a.positions[m] + t.value_keys) / t.value_keys);      // ranges that hold a key
     const float* cs = a.v_rope ? a.v_rope + (size_t)a.positions[m] * V : nullptr;
-    for (int o = threadIdx.x; o < a.q_heads * half; o += 256) {
+    const int o = blockIdx.z * 256 + threadIdx.x;
+    if (o < a.q_heads * half) {
         const int h = o / half, j = o % half;
         const int c0 = a.v_interleaved ? 2 * j : j, c1 = a.v_interleaved ? 2 * j + 1 : j + half;
         float u = 0.f, v = 0.f;
@@ -559,9 +616,12 @@ static int launch_scores(const HeadMixArgs& a, const TileArgs& t, hipStream_t st
     const int rt = tiles >= 4 ? 4 : tiles >= 2 ? 2 : 1;
     const dim3 grid(t.groups, t.kv_pad * ((tiles + rt - 1) / rt), t.score_ranges);
     if (grid.y > 65535 || grid.z > 65535) return -2;
-    if (rt == 4) head_scores_kernel<NKF, 4><<<grid, 256, 0, stream>>>(a, t);
-    else if (rt == 2) head_scores_kernel<NKF, 2><<<grid, 256, 0, stream>>>(a, t);
-    else head_scores_kernel<NKF, 1><<<grid, 256, 0, stream>>>(a, t);
+    if (t.hp_log == 0) head_scores_kernel<NKF, 1, 0><<<grid, 256, 0, stream>>>(a, t);
+    else if (t.hp_log == 1 && rt == 1) head_scores_kernel<NKF, 1, 1><<<grid, 256, 0, stream>>>(a, t);
+    else if (t.hp_log == 1) head_scores_kernel<NKF, 2, 1><<<grid, 256, 0, stream>>>(a, t);
+    else if (rt == 4) head_scores_kernel<NKF, 4, 2><<<grid, 256, 0, stream>>>(a, t);
+    else if (rt == 2) head_scores_kernel<NKF, 2, 2><<<grid, 256, 0, stream>>>(a, t);
+    else head_scores_kernel<NKF, 1, 2><<<grid, 256, 0, stream>>>(a, t);
     return (int)hipGetLastError();
 }
 #endif
@@ -631,25 +691,28 @@ int mlr_head_mix_tiles(const void* q, long q_stride, const void* k_pages, const 
     HeadMixArgs a{(const elem_t*)q, q_stride, (const elem_t*)k_pages, (const elem_t*)v_pages, block_table, slots, positions,
                   mix, sink, sink_value, sink_kind, v_rope, v_interleaved, (const elem_t*)gate, gate_stride, (elem_t*)out,
                   out_stride, max_blocks, q_heads, kv_heads, key_dim, value_dim, page_size, scale, softcap};
+    int page_log = 0;
+    while ((1 << page_log) < page_size) ++page_log;
+    if ((1 << page_log) != page_size) page_log = -1;
     TileArgs t{group_first, group_count, groups, group_tokens, (__bf16*)e, sums, partial, ktiles, hp_log, head_k,
-               head_k / head_pad, score_keys, score_ranges, value_keys, value_ranges};
+               head_k / head_pad, page_log, score_keys, score_ranges, value_keys, value_ranges};
     const int ct = group_tokens == 16 ? head_pad : (head_pad + 15) / 16;
     const int vt = (value_dim / 16 + 8 / kv_block - 1) / (8 / kv_block);
-    if (ct * vt > 32) return 1;
+    if (ct * vt > 32 || vt > 8) return 1;
     const int nkf = (key_dim + 31) / 32;
     int rc = nkf <= 2 ? launch_scores<2>(a, t, stream) : nkf <= 4 ? launch_scores<4>(a, t, stream) : launch_scores<8>(a, t, stream);
     if (rc != 0) return rc;
     rc = 1;
 #define MLR_MIX_CLASS(NQ, CT, VT)                                                     \
     if (rc == 1 && group_tokens == NQ && ct == CT && vt <= VT) rc = launch_mix_heads<CT, VT, NQ>(a, t, kv_block, stream);
-    MLR_MIX_CLASS(16, 1, 2) MLR_MIX_CLASS(16, 1, 8) MLR_MIX_CLASS(16, 1, 32)
-    MLR_MIX_CLASS(16, 2, 2) MLR_MIX_CLASS(16, 2, 8) MLR_MIX_CLASS(16, 2, 16)
-    MLR_MIX_CLASS(16, 4, 2) MLR_MIX_CLASS(16, 4, 4) MLR_MIX_CLASS(16, 4, 8)
+    MLR_MIX_CLASS(16, 1, 2) MLR_MIX_CLASS(16, 1, 4) MLR_MIX_CLASS(16, 1, 8)
+    MLR_MIX_CLASS(16, 2, 2) MLR_MIX_CLASS(16, 2, 4) MLR_MIX_CLASS(16, 2, 8)
+    MLR_MIX_CLASS(16, 4, 1) MLR_MIX_CLASS(16, 4, 2) MLR_MIX_CLASS(16, 4, 4)
     MLR_MIX_CLASS(16, 8, 2) MLR_MIX_CLASS(16, 8, 4) MLR_MIX_CLASS(16, 16, 2) MLR_MIX_CLASS(16, 32, 1)
-    MLR_MIX_CLASS(1, 1, 1) MLR_MIX_CLASS(1, 1, 4) MLR_MIX_CLASS(1, 1, 32) MLR_MIX_CLASS(1, 2, 4) MLR_MIX_CLASS(1, 2, 16)
+    MLR_MIX_CLASS(1, 1, 1) MLR_MIX_CLASS(1, 1, 2) MLR_MIX_CLASS(1, 1, 4) MLR_MIX_CLASS(1, 1, 8) MLR_MIX_CLASS(1, 2, 2) MLR_MIX_CLASS(1, 2, 8)
 #undef MLR_MIX_CLASS
     if (rc != 0) return rc;
-    head_mix_finish_kernel<<<dim3(groups, group_tokens), 256, 0, stream>>>(a, t);
+    head_mix_finish_kernel<<<dim3(groups, group_tokens, (q_heads * (value_dim / 2) + 255) / 256), 256, 0, stream>>>(a, t);
     return (int)hipGetLastError();
 #else
     return 1;

@@ -230,6 +230,91 @@ __global__ __launch_bounds__(64) void sink_qkv_prep_kernel(
     }
 }
 
+#if MLR_BF16
+// The same for head sizes of 8 times a power of two (up to 512), split-half pairs whose halves are multiples of 8
+// channels and a norm before the rotation or none: a lane takes eight channels (16-byte accesses), a head is key_dim / 8
+// neighbouring lanes of a wavefront, and what a pair's other half holds comes by a lane exchange.
+__device__ __forceinline__ void turn_eight(float (&x)[8], int li, int half_lanes, const float* cs, int dim) {
+    const int lane = threadIdx.x & 63;
+    const bool low = li < half_lanes, turns = li < 2 * half_lanes;
+    const int other = turns ? (low ? lane + half_lanes : lane - half_lanes) : lane;
+    const int j = turns ? (low ? li : li - half_lanes) * 8 : 0;
+    float c[8], s[8];
+    *reinterpret_cast<float4*>(c) = *reinterpret_cast<const float4*>(cs + j);
+    *reinterpret_cast<float4*>(c + 4) = *reinterpret_cast<const float4*>(cs + j + 4);
+    *reinterpret_cast<float4*>(s) = *reinterpret_cast<const float4*>(cs + dim / 2 + j);
+    *reinterpret_cast<float4*>(s + 4) = *reinterpret_cast<const float4*>(cs + dim / 2 + j + 4);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+        const float o = __shfl(x[e], other, MLR_WAVE);
+        const float y = low ? turn_x(x[e], o, c[e], s[e]) : turn_y(o, x[e], c[e], s[e]);
+        if (turns) x[e] = y;
+    }
+}
+
+__global__ __launch_bounds__(256) void sink_qkv_prep_vec_kernel(
+    const elem_t* __restrict__ proj, long ld, const float* __restrict__ bias, elem_t* __restrict__ q_out,
+    elem_t* __restrict__ k_pages, long k_row, elem_t* __restrict__ v_pages, long v_row,
+    const int32_t* __restrict__ block_table, int max_blocks, const int32_t* __restrict__ slots,
+    const int32_t* __restrict__ positions, const float* __restrict__ q_norm_w, const float* __restrict__ k_norm_w,
+    float eps, const float* __restrict__ rope, int rot_dim, int q_heads, int kv_heads, int key_dim, int value_dim,
+    int page_size, int write_cache, int norm_mode, const float* __restrict__ v_rope, int v_transposed) {
+    const int m = blockIdx.x, at = blockIdx.y * 256 + threadIdx.x;
+    const int k_lanes = key_dim >> 3, v_lanes = value_dim >> 3;      // lanes of a head
+    const int v_start = ((q_heads + kv_heads) * k_lanes + 63) & ~63;
+    const bool value = at >= v_start;                                // (the same in every lane of a wavefront)
+    const int lanes = value ? v_lanes : k_lanes, unit = (value ? at - v_start : at) / lanes;
+    const int li = (value ? at - v_start : at) & (lanes - 1), units = value ? kv_heads : q_heads + kv_heads;
+    const bool ok = unit < units, cached = value || unit >= q_heads;
+    const int pos = positions[m];
+    const long off = (value ? (long)(q_heads + kv_heads) * key_dim + (long)unit * value_dim : (long)unit * key_dim) + li * 8;
+    float x[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) x[e] = 0.f;
+    if (ok) {
+        load_vec(proj + (size_t)m * ld + off, x);
+        if (bias != nullptr)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) x[e] += bias[off + e];
+    }
+    if (!value && norm_mode == 1) {
+        float sum = 0.f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) sum += x[e] * x[e];
+        for (int d = 1; d < lanes; d <<= 1) sum += __shfl_xor(sum, d, MLR_WAVE);
+        const float r = 1.0f / sqrtf(sum / (float)key_dim + eps);
+        const float* w = unit < q_heads ? q_norm_w : k_norm_w;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[e] = (x[e] * r) * (w != nullptr ? w[li * 8 + e] : 1.0f);
+    }
+    if (value) {
+        if (v_rope != nullptr) turn_eight(x, li, v_lanes >> 1, v_rope + (size_t)pos * value_dim, value_dim);
+    } else if (rope != nullptr) {
+        turn_eight(x, li, rot_dim >> 4, rope + (size_t)pos * rot_dim, rot_dim);
+    }
+    if (!ok) return;
+    if (!cached) {
+        store_vec(q_out + (size_t)m * q_heads * key_dim + off, x);
+        return;
+    }
+    const int block = pos / page_size, place = pos % page_size;
+    const int page = write_cache && block < max_blocks ? block_table[(size_t)slots[m] * max_blocks + block] : -1;
+    if (page < 0) return;                      // (no page: nothing is written)
+    const int kvh = value ? unit : unit - q_heads;
+    const long long head_at = ((long long)page * kv_heads + kvh) * page_size;
+    if (!value) {
+        store_vec(k_pages + (head_at + place) * k_row + li * 8, x);
+    } else if (!v_transposed) {
+        store_vec(v_pages + (head_at + place) * v_row + li * 8, x);
+    } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v_pages[head_at * value_dim + (long)(li * 8 + e) * page_size + place] = (elem_t)x[e];
+    }
+}
+
+static bool eight_lanes(int dim) { return dim >= 8 && dim <= 512 && (dim & (dim - 1)) == 0; }
+#endif
+
 // Latent attention's row work.  q_src[m] = [heads * (dim + rot)]: per head `dim` plain and `rot` rotated query
 // channels; kv_src[m] = [rank + rot]: the latent part (`rank` channels) and the one rotated key part all heads
 // share (the two may be column blocks of one projection's output).
@@ -612,6 +697,21 @@ int mlr_sink_qkv_prep(const void* proj, long ld, const float* bias, void* q_out,
     if ((v_rope != nullptr && (value_dim > MAX_KEY_DIM || (value_dim & 1))) || key_dim > MAX_KEY_DIM || q_heads + 2 * kv_heads > 65535 || rot_dim > key_dim || (rot_dim & 1) || norm_mode < 0 ||
         norm_mode > 2)
         return -1;
+#if MLR_BF16
+    const auto aligned = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+    if (norm_mode < 2 && eight_lanes(key_dim) && eight_lanes(value_dim) && ld % 8 == 0 && k_row % 8 == 0 &&
+        (v_transposed || v_row % 8 == 0) && (rope == nullptr || (!interleaved && rot_dim % 16 == 0 && aligned(rope))) &&
+        (v_rope == nullptr || (!v_interleaved && value_dim % 16 == 0 && aligned(v_rope))) && aligned(proj) && aligned(q_out) &&
+        aligned(k_pages) && aligned(v_pages)) {
+        const int v_start = ((q_heads + kv_heads) * (key_dim / 8) + 63) / 64 * 64;
+        const int threads = v_start + kv_heads * (value_dim / 8);
+        sink_qkv_prep_vec_kernel<<<dim3(rows, (threads + 255) / 256), 256, 0, stream>>>(
+            (const elem_t*)proj, ld, bias, (elem_t*)q_out, (elem_t*)k_pages, k_row, (elem_t*)v_pages, v_row, block_table,
+            max_blocks, slots, positions, q_norm_w, k_norm_w, eps, rope, rot_dim, q_heads, kv_heads, key_dim, value_dim,
+            page_size, write_cache, norm_mode, v_rope, v_transposed);
+        return (int)hipGetLastError();
+    }
+#endif
     sink_qkv_prep_kernel<<<dim3(rows, q_heads + 2 * kv_heads), 64, 0, stream>>>(
         (const elem_t*)proj, ld, bias, (elem_t*)q_out, (elem_t*)k_pages, k_row, (elem_t*)v_pages, v_row, block_table,
         max_blocks, slots, positions, q_norm_w, k_norm_w, eps, rope, rot_dim, q_heads, kv_heads, key_dim, value_dim,

@@ -1606,8 +1606,9 @@ class Kernels:
         inner = 16 if kv_heads * pad <= 16 else -(-kv_heads * pad // 32) * 32
         if pad > 32 or inner > 128 or inner % pad != 0 or value_dim % 16 != 0:
             return None
-        for block in (8, 4, 2, 1):                 # (sums in registers: column tiles x value tiles of a wavefront)
-            if block * pad <= 32 and pad * -(-(value_dim // 16) // (8 // block)) <= 32:
+        most = min(8, (16 if pad <= 4 else 32) // pad)      # value tiles of a wavefront: its sums stay in registers
+        for block in (8, 4, 2, 1):
+            if block * pad <= 32 and -(-(value_dim // 16) // (8 // block)) <= most:
                 return pad, inner, block
         return None
 

@@ -25,8 +25,8 @@ SCRATCH_CAP = 144 << 20       # elements of exponentials that one launch may kee
 PARTIAL_CAP = 16 << 20        # floats of the key ranges' shares
 SUMS_CAP = 4 << 20            # floats of the sums
 MOST_RANGES = 64
-SCORE_RANGE = 128             # the narrowest key ranges of a workgroup: of the scores,
-VALUE_RANGE = 256             # and of the values
+RANGE = 256                   # the narrowest range of keys of a workgroup
+WIDE_RANGE = 1024             # and the one that costs nothing
 
 
 def _up(n, unit):
@@ -45,19 +45,24 @@ class LaunchShape:
         # groups a launch: what the scratch buffers hold (at least one)
         self.groups = max(1, min(groups, SCRATCH_CAP // (tokens * row_e), PARTIAL_CAP // (tokens * row_o),
                                  SUMS_CAP // (tokens * inner)))
+        # ranges of keys where the groups alone do not fill the GPU
         tiles = -(-tokens * pad // 16)
         units = self.groups * (inner // pad) * -(-tiles // (4 if tiles >= 4 else 2 if tiles >= 2 else 1))
-        ranges = max(1, min(MOST_RANGES, -(-2 * target // units), keys // SCORE_RANGE,
-                            SUMS_CAP // (self.groups * tokens * inner)))
-        self.score_keys = _up(-(-keys // ranges), SCORE_RANGE)
+        ranges = max(1, min(MOST_RANGES, -(-target // units), keys // RANGE, SUMS_CAP // (self.groups * tokens * inner)))
+        self.score_keys = _up(-(-keys // ranges), 128)
         self.score_ranges = -(-keys // self.score_keys)
-        self.kv_block = most
-        while self.kv_block > 1 and self.groups * -(-s.kv_heads // self.kv_block) < target:
-            self.kv_block //= 2
-        units = self.groups * -(-s.kv_heads // self.kv_block)
-        ranges = max(1, min(MOST_RANGES, -(-target // units), keys // VALUE_RANGE,
-                            PARTIAL_CAP // (self.groups * tokens * row_o)))
-        self.value_keys = _up(-(-keys // ranges), VALUE_RANGE)
+        # the second launch: wide ranges first, then fewer kv heads a workgroup (each mixes for its own), then narrow
+        # ranges (their shares are written and read again), measured in this order
+        room = max(1, PARTIAL_CAP // (self.groups * tokens * row_o))
+        self.kv_block, self.value_keys = most, _up(keys, RANGE)
+        for width, block, enough in ((WIDE_RANGE, most, target), (WIDE_RANGE, 2, target), (RANGE, 2, target), (RANGE, 1, target // 2)):
+            units = self.groups * -(-s.kv_heads // self.kv_block) * -(-keys // self.value_keys)
+            if units >= enough:
+                break
+            self.kv_block = min(self.kv_block, block)
+            units = self.groups * -(-s.kv_heads // self.kv_block)
+            ranges = max(1, min(MOST_RANGES, -(-target // units), keys // width, room))
+            self.value_keys = _up(-(-keys // ranges), RANGE)
         self.value_ranges = -(-keys // self.value_keys)
         rows = self.groups * tokens
         self.e_numel, self.sums_numel = rows * row_e, rows * inner * self.score_ranges
@@ -187,7 +192,7 @@ class HeadMixAttention:
         for (first, count, n), tokens in ((big, GROUP), (small, 1)):
             if n == 0:
                 continue
-            shape = LaunchShape(s, self._layout(), n, tokens, ctx.max_context, ctx.target_workgroups)
+            shape = LaunchShape(s, self._layout(), n, tokens, ctx.max_context, ctx.target_workgroups // 2)
             e = ctx.workspace.get("mix_e", (shape.e_numel,), q.dtype)
             sums = ctx.workspace.get("mix_sums", (shape.sums_numel,), torch.float32)
             partial = ctx.workspace.get("mix_partial", (shape.partial_numel,), torch.float32)
