@@ -211,7 +211,15 @@ struct SkinnyEpilogue {
     int ss_stride;            // floats between the rows of ss_out (its capacity: a strip of 16 a part)
     float glu_limit;          // GATED: > 0: the clamped gate g = min(gate, limit), u = clamp(up, +-limit),
     float glu_slope;          //        y = g sigmoid(slope g) (u + 1); 0: y = silu(gate) up; < 0: y = gelu_tanh(gate) up
+    int plain_act;            // a plain product's activation: 0 none, 1 relu(x)^2, 2 the exact gelu x Phi(x)
 };
+__device__ __forceinline__ float plain_activation(float x, int act) {
+    if (act == 1) {
+        x = fmaxf(x, 0.f);
+        return x * x;
+    }
+    return 0.5f * x * (1.0f + erff(x * 0.70710678118654752440f));
+}
 
 // PAIR: a workgroup owns `cols` (17..32) output columns, two strips side by side, the second one partly
 // used: for a number of columns that deals strips of 16 unevenly to the compute units (384 strips on 256
@@ -447,6 +455,12 @@ __global__ __launch_bounds__(SKINNY_WAVES * 64) void gemm_skinny_kernel(const __
                     y = 0.5f * gg * (1.0f + tanhf(0.7978845608028654f * (gg + 0.044715f * gg * gg * gg))) * v[NW - 1];
                 } else {
                     y = (v[0] / (1.0f + expf(-v[0]))) * v[NW - 1];
+                }
+            }
+            if constexpr (!GATED && !OUT_FLOAT && EPI == EPI_NONE) {
+                if (epi.plain_act) {
+                    y = plain_activation(y, epi.plain_act);
+                    if constexpr (PAIR) v[1] = plain_activation(v[1], epi.plain_act);
                 }
             }
             y4[i][r] = y;
@@ -1010,6 +1024,19 @@ extern "C" int mlr_gemm_gated_gelu_tanh(const void* a, const void* w, void* out,
     if (M <= 16) return launch_skinny<1, true>(a, w, out, M, N, K, 0, stream, epi);
     if (M <= 32) return launch_skinny<2, true>(a, w, out, M, N, K, 0, stream, epi);
     if (M <= 64) return launch_skinny<4, true>(a, w, out, M, N, K, 0, stream, epi);
+    return 1;
+}
+
+// out[M, N] = act(a . w^T), act 1 relu(x)^2 or 2 the exact gelu, as the epilogue of the weight-streaming kernels, up to
+// 64 rows.  Returns 1 for more rows.
+extern "C" int mlr_gemm_act(const void* a, const void* w, void* out, int M, int N, int K, int act, hipStream_t stream) {
+    if (M <= 0 || N <= 0) return 0;
+    if (K <= 0 || act < 1 || act > 2) return -1;
+    SkinnyEpilogue epi{};
+    epi.plain_act = act;
+    if (M <= 16) return launch_skinny<1, false>(a, w, out, M, N, K, 0, stream, epi);
+    if (M <= 32) return launch_skinny<2, false>(a, w, out, M, N, K, 0, stream, epi);
+    if (M <= 64) return launch_skinny<4, false>(a, w, out, M, N, K, 0, stream, epi);
     return 1;
 }
 

@@ -258,13 +258,13 @@ __global__ __launch_bounds__(256) void sink_qkv_prep_vec_kernel(
     const int32_t* __restrict__ block_table, int max_blocks, const int32_t* __restrict__ slots,
     const int32_t* __restrict__ positions, const float* __restrict__ q_norm_w, const float* __restrict__ k_norm_w,
     float eps, const float* __restrict__ rope, int rot_dim, int q_heads, int kv_heads, int key_dim, int value_dim,
-    int page_size, int write_cache, int norm_mode, const float* __restrict__ v_rope, int v_transposed) {
+    int page_size, int write_cache, int norm_mode, const float* __restrict__ v_rope, int v_transposed, int with_values) {
     const int m = blockIdx.x, at = blockIdx.y * 256 + threadIdx.x;
     const int k_lanes = key_dim >> 3, v_lanes = value_dim >> 3;      // lanes of a head
     const int v_start = ((q_heads + kv_heads) * k_lanes + 63) & ~63;
     const bool value = at >= v_start;                                // (the same in every lane of a wavefront)
     const int lanes = value ? v_lanes : k_lanes, unit = (value ? at - v_start : at) / lanes;
-    const int li = (value ? at - v_start : at) & (lanes - 1), units = value ? kv_heads : q_heads + kv_heads;
+    const int li = (value ? at - v_start : at) & (lanes - 1), units = value ? (with_values ? kv_heads : 0) : q_heads + kv_heads;
     const bool ok = unit < units, cached = value || unit >= q_heads;
     const int pos = positions[m];
     const long off = (value ? (long)(q_heads + kv_heads) * key_dim + (long)unit * value_dim : (long)unit * key_dim) + li * 8;
@@ -309,6 +309,54 @@ __global__ __launch_bounds__(256) void sink_qkv_prep_vec_kernel(
     } else {
 #pragma unroll
         for (int e = 0; e < 8; ++e) v_pages[head_at * value_dim + (long)(li * 8 + e) * page_size + place] = (elem_t)x[e];
+    }
+}
+
+// The values of many rows into transposed pages: a workgroup takes 16 rows of the batch and one kv head, turns them, and
+// lays them into LDS channel by channel; eight rows that are consecutive positions of one request and start at a
+// multiple of eight are one 16-byte write a channel, others are written one by one.
+#define VALUE_ROWS 16
+#define VALUE_PITCH (VALUE_ROWS + 8)
+__global__ __launch_bounds__(256) void values_transposed_kernel(
+    const elem_t* __restrict__ proj, long ld, long v_off, const float* __restrict__ bias, elem_t* __restrict__ v_pages,
+    const int32_t* __restrict__ block_table, int max_blocks, const int32_t* __restrict__ slots,
+    const int32_t* __restrict__ positions, int rows, int kv_heads, int value_dim, int page_size,
+    const float* __restrict__ v_rope) {
+    extern __shared__ __attribute__((aligned(16))) unsigned char lds_raw[];
+    __bf16* tile = reinterpret_cast<__bf16*>(lds_raw);               // [value_dim][VALUE_PITCH]
+    const int m0 = blockIdx.x * VALUE_ROWS, kvh = blockIdx.y, tid = threadIdx.x;
+    const int lanes = value_dim >> 3, li = tid & (lanes - 1);
+    const long off = v_off + (long)kvh * value_dim + li * 8;
+    for (int r = tid / lanes; r < VALUE_ROWS; r += 256 / lanes) {
+        const int m = min(m0 + r, rows - 1);
+        float x[8];
+        load_vec(proj + (size_t)m * ld + off, x);
+        if (bias != nullptr)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) x[e] += bias[off + e];
+        if (v_rope != nullptr) turn_eight(x, li, lanes >> 1, v_rope + (size_t)positions[m] * value_dim, value_dim);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) tile[(li * 8 + e) * VALUE_PITCH + r] = (elem_t)x[e];
+    }
+    __syncthreads();
+    for (int i = tid; i < value_dim * 2; i += 256) {
+        const int c = i >> 1, r0 = (i & 1) * 8, m = m0 + r0;
+        if (m >= rows) continue;
+        const int pos = positions[m];
+        const __bf16* src = tile + c * VALUE_PITCH + r0;
+        if ((pos & 7) == 0 && (page_size & 7) == 0 && m + 7 < rows && positions[m + 7] == pos + 7 && slots[m + 7] == slots[m]) {
+            const int block = pos / page_size;
+            const int page = block < max_blocks ? block_table[(size_t)slots[m] * max_blocks + block] : -1;
+            if (page >= 0)
+                *reinterpret_cast<vec16*>(v_pages + (((long long)page * kv_heads + kvh) * value_dim + c) * page_size + pos % page_size) =
+                    *reinterpret_cast<const vec16*>(src);
+            continue;
+        }
+        for (int j = 0; j < 8 && m + j < rows; ++j) {
+            const int p = positions[m + j], block = p / page_size;
+            const int page = block < max_blocks ? block_table[(size_t)slots[m + j] * max_blocks + block] : -1;
+            if (page >= 0) v_pages[(((long long)page * kv_heads + kvh) * value_dim + c) * page_size + p % page_size] = src[j];
+        }
     }
 }
 
@@ -704,11 +752,17 @@ int mlr_sink_qkv_prep(const void* proj, long ld, const float* bias, void* q_out,
         (v_rope == nullptr || (!v_interleaved && value_dim % 16 == 0 && aligned(v_rope))) && aligned(proj) && aligned(q_out) &&
         aligned(k_pages) && aligned(v_pages)) {
         const int v_start = ((q_heads + kv_heads) * (key_dim / 8) + 63) / 64 * 64;
-        const int threads = v_start + kv_heads * (value_dim / 8);
+        const bool values_apart = v_transposed && rows >= 64 && write_cache && kv_heads <= 65535;
+        const int threads = values_apart ? v_start : v_start + kv_heads * (value_dim / 8);
         sink_qkv_prep_vec_kernel<<<dim3(rows, (threads + 255) / 256), 256, 0, stream>>>(
             (const elem_t*)proj, ld, bias, (elem_t*)q_out, (elem_t*)k_pages, k_row, (elem_t*)v_pages, v_row, block_table,
             max_blocks, slots, positions, q_norm_w, k_norm_w, eps, rope, rot_dim, q_heads, kv_heads, key_dim, value_dim,
-            page_size, write_cache, norm_mode, v_rope, v_transposed);
+            page_size, write_cache, norm_mode, v_rope, v_transposed, values_apart ? 0 : 1);
+        if (values_apart)
+            values_transposed_kernel<<<dim3((rows + VALUE_ROWS - 1) / VALUE_ROWS, kv_heads), 256,
+                                       (size_t)value_dim * VALUE_PITCH * sizeof(elem_t), stream>>>(
+                (const elem_t*)proj, ld, (long)(q_heads + kv_heads) * key_dim, bias, (elem_t*)v_pages, block_table, max_blocks,
+                slots, positions, rows, kv_heads, value_dim, page_size, v_rope);
         return (int)hipGetLastError();
     }
 #endif

@@ -401,6 +401,21 @@ class Kernels:
         _ok(self._lib("gemm").mlr_gemm_gated_gelu_tanh(_p(a), _p(w), _p(out), _c_int(m), _c_int(two_n // 2), _c_int(k),
                                                        _stream()), "gemm_gated_gelu_tanh")
 
+    @timed("gemm", _gemm_work)
+    def gemm_act(self, a, w, out, kind):
+        """out[M, N] = act(a . w^T), act as `plain_act`'s, fused into the weight-streaming projection, up to 64 rows
+        (bfloat16)."""
+        _need(self.dtype == torch.bfloat16 and a.shape[0] <= 64, "gemm_act: bfloat16, up to 64 rows")
+        _need(kind in self.PLAIN_ACTS, f"gemm_act: activation {kind!r}")
+        _tensor(a, "a", self.dtype, ndim=2)
+        _tensor(w, "w", self.dtype, ndim=2)
+        m, k = a.shape
+        n, k2 = w.shape
+        _need(k == k2, "gemm_act: inner sizes differ")
+        _tensor(out, "out", self.dtype, (m, n))
+        _ok(self._lib("gemm").mlr_gemm_act(_p(a), _p(w), _p(out), _c_int(m), _c_int(n), _c_int(k),
+                                           _c_int(1 + self.PLAIN_ACTS[kind]), _stream()), "gemm_act")
+
     # -- an RMSNorm handed from one projection to the next (few rows) ------------------------------
     HANDOFF_MAX_ROWS = 16
 

@@ -157,8 +157,11 @@ class PlainMlp:
         m = x.shape[0]
         k = ctx.kernels
         act = ctx.workspace.get("act", (m, s.intermediate), x.dtype)
-        k.gemm(x, self.up, act)
-        k.plain_act(act, act, s.activation)
+        if m <= 64 and k.streams_weight(m, s.hidden):      # few rows: the activation rides on the projection
+            k.gemm_act(x, self.up, act, s.activation)
+        else:
+            k.gemm(x, self.up, act)
+            k.plain_act(act, act, s.activation)
         out = ctx.workspace.get("ffn_out", (m, s.hidden), x.dtype)
         k.gemm(act, self.down, out)
         return out

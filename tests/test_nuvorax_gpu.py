@@ -346,6 +346,59 @@ def test_keys_are_turned_by_bands_and_values_whole_on_their_way_into_the_pages(d
 
 
 @pytest.mark.parametrize("dtype_name", DTYPES)
+@pytest.mark.parametrize("heads,kv,dim,vdim,rot,page", [(4, 2, 64, 32, 32, 8), (2, 2, 128, 128, 128, 16), (3, 1, 8, 16, 4, 4), (1, 1, 512, 256, 16, 24),
+                                                        (5, 1, 40, 48, 8, 8)])
+def test_rows_of_several_requests_reach_their_pages(dtype_name, heads, kv, dim, vdim, rot, page):
+    """Enough rows that values go to their pages in blocks: two portions that start at odd positions, single tokens
+    between them, a portion that starts at a multiple of eight."""
+    from mini_llm_runtime_amd.config.specs import PositionSpec
+    from mini_llm_runtime_amd.kernels import Kernels
+    from mini_llm_runtime_amd.parts.rope import Rope
+    dtype = DTYPES[dtype_name]
+    k = Kernels(dtype)
+    rng = np.random.default_rng(8)
+    places = [(0, p) for p in range(5, 66)] + [(1, 17), (2, 40)] + [(3, p) for p in range(8, 50)] + [(4, p) for p in range(3)]
+    slots, positions = [s for s, _ in places], np.array([p for _, p in places])
+    m, total = len(places), heads * dim + kv * (dim + vdim)
+    proj = rounded(rng.normal(size=(m, total)), dtype)
+    x = back(proj)
+    qw, kw = (rounded(1.0 + 0.3 * rng.normal(size=dim), torch.float32) for _ in range(2))
+    rule = dict(dims=rot, base=300.0)
+    q = P.rotate_keys(P.rms_norm(x[:, :heads * dim].reshape(m, heads, dim), back(qw), 1e-4), positions, rule)
+    kk = P.rotate_keys(P.rms_norm(x[:, heads * dim:(heads + kv) * dim].reshape(m, kv, dim), back(kw), 1e-4), positions, rule)
+    vv = P.rotate_values(x[:, (heads + kv) * dim:].reshape(m, kv, vdim), positions, 300.0)
+    blocks = -(-72 // page)
+    table = np.random.default_rng(1).permutation(5 * blocks).reshape(5, blocks)
+    k_pages = torch.full((5 * blocks, kv, page, dim), float("nan"), dtype=dtype, device="cuda")
+    v_pages = torch.full((5 * blocks, kv, vdim, page), float("nan"), dtype=dtype, device="cuda")
+    q_out = torch.empty((m, heads * dim), dtype=dtype, device="cuda")
+    k.sink_qkv_prep(proj, None, q_out, k_pages, v_pages, ints(table.tolist()), ints(slots), ints(positions.tolist()), qw, kw, 1e-4,
+                    Rope(PositionSpec("rope", rot, 300.0)).rotation(128, "cuda").table, heads, kv, dim, vdim, page,
+                    v_rope=turn_table(vdim, 300.0, 128), v_transposed=True)
+    tol = tolerance(dtype_name)
+    np.testing.assert_allclose(back(q_out), q.reshape(m, -1), **tol)
+    kp, vp = back(k_pages), back(v_pages)
+    for i, (s, p) in enumerate(places):
+        np.testing.assert_allclose(kp[table[s, p // page], :, p % page], kk[i], **tol)
+        np.testing.assert_allclose(vp[table[s, p // page], :, :, p % page], vv[i], **tol)
+    assert np.isfinite(kp).sum() == m * kv * dim and np.isfinite(vp).sum() == m * kv * vdim      # nothing else was touched
+
+
+@pytest.mark.parametrize("rows", [1, 7, 16, 20, 33, 64])
+@pytest.mark.parametrize("hidden,inter", [(64, 48), (128, 6200), (40, 100), (2048, 20)])
+def test_the_activation_rides_on_the_projection_of_few_rows(rows, hidden, inter):
+    from mini_llm_runtime_amd.kernels import Kernels
+    k = Kernels(torch.bfloat16)
+    rng = np.random.default_rng(hidden)
+    x, w = rounded(rng.normal(size=(rows, hidden)), torch.bfloat16), rounded(rng.normal(size=(inter, hidden)) * 1.5 * hidden ** -0.5, torch.bfloat16)
+    z = back(x) @ back(w).T
+    for kind, want in (("gelu_erf", P.gelu_erf(z)), ("relu_squared", np.maximum(z, 0.0) ** 2)):
+        out = torch.full((rows, inter), float("nan"), dtype=torch.bfloat16, device="cuda")
+        k.gemm_act(x, w, out, kind)
+        np.testing.assert_allclose(back(out), want, rtol=1e-2, atol=2e-3)
+
+
+@pytest.mark.parametrize("dtype_name", DTYPES)
 @pytest.mark.parametrize("rows,width", [(5, 24), (3, 37), (70, 128), (2, 1), (9, 4100), (2, 9000), (1, 2050)])
 def test_branches_are_added_and_normed_in_one_pass(dtype_name, rows, width):
     from mini_llm_runtime_amd.kernels import Kernels
