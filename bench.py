@@ -737,8 +737,9 @@ class BudoraxBench(Bench):
 # `--only nuvorax`: layer sizes that resemble a real model's, for a Nuvorax model of eight layers -- attention with mixed
 # heads beside a dense gelu feed-forward (two matrices of one and a half times the inner size) and beside a mixture of
 # eight clamped experts with a shared expert (an expert a quarter of the inner size, of which a token uses two; the shared
-# one half), in turn, one norm a layer -- and for the closest model the engine had before: a Pamunex model (grouped-query and latent attention with a sink, dense and routed feed-forwards, layer norms) of the same width,
-# feed-forward, heads and layers.
+# one half), in turn, one norm a layer -- and for the closest model the engine had before: a Pamunex model (grouped-query and
+# latent attention with a sink, dense and routed feed-forwards, layer norms) of the same width, feed-forward, heads and
+# layers.
 NUVORAX_SIZES = {
     "2k": dict(width=2048, ff=5632, vocab=32000, layers=8, heads=16, kv_heads=4),
     "4k": dict(width=4096, ff=12288, vocab=32000, layers=8, heads=32, kv_heads=8),
@@ -803,8 +804,8 @@ class NuvoraxBench(Bench):
 def design_block(args):
     """Prefill (2048 tokens in one step) and decode (batch 8 and 64 behind --context tokens) of a design's sizes
     beside the closest model the engine had before it (a Qwen3 dense model of equal width, heads, feed-forward and
-    layers; for Tigelorn a Taletar model, for Budorax a Tigelorn model, for Nuvorax a Pamunex model of equal sizes); then the same steps once more with events around every
-    launch: milliseconds per kernel class."""
+    layers; for Tigelorn a Taletar model, for Budorax a Tigelorn model, for Nuvorax a Pamunex model of equal sizes); then
+    the same steps once more with events around every launch: milliseconds per kernel class."""
     import copy
     out = {}
     design = getattr(args, "design", "taletar")

@@ -41,7 +41,8 @@ class Rope:
     (`FrequencyStretch`: a ramp between the pairs that turn fast, which keep their frequency, and those that turn
     slowly, whose frequency is divided by `factor`; cosines and sines are multiplied by 0.1 ln(factor) + 1) or scaled
     by bands of how often a pair turns over the original length (`FrequencyBands`: fast pairs stay, slow pairs are
-    divided by `factor`, those between are blended).  Frequencies and angles are 32-bit; the table holds cos in its first half and sin in its second."""
+    divided by `factor`, those between are blended).  Frequencies and angles are 32-bit; the table holds cos in its
+    first half and sin in its second."""
 
     def __init__(self, spec):
         self.dim, self.base = spec.dim, float(spec.base)
