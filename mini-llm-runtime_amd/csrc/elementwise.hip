@@ -3,8 +3,9 @@
 // activation and the residual sum are computed in 32-bit.
 #include "common.h"
 
-// h[m, :] = float(table[ids[m], :]).  An id outside [0, vocab) gives a row of NaN
-// (the host refuses such a batch before anything runs).
+// h[m, :] = float(table[ids[m], :]) * scale; without a factor (SCALED false) every bit of a value survives.  An id
+// outside [0, vocab) gives a row of NaN (the host refuses such a batch before anything runs).
+template <bool SCALED>
 __global__ void embed_gather_kernel(const int32_t* __restrict__ ids, const elem_t* __restrict__ table,
                                     float* __restrict__ h, int width, int vocab, float scale) {
     const int m = blockIdx.x;
@@ -15,7 +16,7 @@ __global__ void embed_gather_kernel(const int32_t* __restrict__ ids, const elem_
         return;
     }
     const elem_t* row = table + (size_t)id * width;
-    for (int i = threadIdx.x; i < width; i += blockDim.x) out[i] = to_float(row[i]) * scale;
+    for (int i = threadIdx.x; i < width; i += blockDim.x) out[i] = SCALED ? to_float(row[i]) * scale : to_float(row[i]);
 }
 
 __device__ __forceinline__ float block_max(float v, float* scratch) {
@@ -973,7 +974,8 @@ extern "C" {
 int mlr_embed_gather(const int32_t* ids, const void* table, float* h, int rows, int width, int vocab, float scale,
                      hipStream_t stream) {
     if (rows <= 0) return 0;
-    embed_gather_kernel<<<rows, 256, 0, stream>>>(ids, (const elem_t*)table, h, width, vocab, scale);
+    if (scale == 1.0f) embed_gather_kernel<false><<<rows, 256, 0, stream>>>(ids, (const elem_t*)table, h, width, vocab, scale);
+    else embed_gather_kernel<true><<<rows, 256, 0, stream>>>(ids, (const elem_t*)table, h, width, vocab, scale);
     return (int)hipGetLastError();
 }
 
