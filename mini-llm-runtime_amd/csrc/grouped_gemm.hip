@@ -6,8 +6,8 @@
 //     out + g * out_group with row strides lda / ldo: one projection per head on slices of wider rows;
 //   offsets != null: group g takes the rows offsets[g] .. offsets[g + 1] - 1 of a list sorted by group (rows of
 //     out; a's row is gather[row] when gather != null): the experts of a routed feed-forward.
-// act: none, relu(x)^2, the exact gelu, or one of the gated forms.  Every output element is one sum over k in ascending order whatever rows lie beside
-// it, so a row's result does not depend on the batch.  Accumulation is 32-bit; the bfloat16 engine multiplies on
+// act: none, relu(x)^2, the exact gelu, or one of the gated forms.  Every output element is one sum over k in
+// ascending order whatever rows lie beside it, so a row's result does not depend on the batch.  Accumulation is 32-bit; the bfloat16 engine multiplies on
 // the matrix cores (v_mfma_f32_16x16x32_bf16, operands staged through LDS), the float engine with plain FMAs.
 //
 // Routing (32-bit): `router_topk_kernel` (sigmoid or softmax of a token's router logits, the best groups of neighbouring
@@ -286,8 +286,8 @@ __device__ __forceinline__ void wave_best(float& value, int& index) {
 // One wavefront a token.  s = sigmoid(z), or softmax(z) over all experts (`softmax`), z[m * ld ..] the token's router
 // logits (float: a product of the framework's own, 32-bit sums).  The experts form `group_count`
 // equal groups of neighbours; a group's score is the sum of its two largest s (of its only one, when a group is
-// one expert), or its largest (`group_best`); only experts of the `group_keep` best groups stand; of those the `top` largest s are chosen
-// (ties: the lower index), ids[m][i] in descending order of s with weights[m][i] = s itself.
+// one expert), or its largest (`group_best`); only experts of the `group_keep` best groups stand; of
+// those the `top` largest s are chosen (ties: the lower index), ids[m][i] in descending order of s with weights[m][i] = s itself.
 // With `correction` [experts] the choice (of groups and of experts) goes by s + correction while the weights stay
 // the plain s; with `renorm` the chosen weights are divided by their sum (+ 1e-20); `out_scale` multiplies them.
 __global__ __launch_bounds__(64) void router_topk_kernel(const float* __restrict__ z, long ld, int32_t* __restrict__ ids,

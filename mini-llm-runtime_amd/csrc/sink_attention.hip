@@ -742,7 +742,8 @@ int mlr_sink_qkv_prep(const void* proj, long ld, const float* bias, void* q_out,
                       int page_size, int write_cache, int norm_mode, int interleaved, const float* v_rope, int v_interleaved,
                       int v_transposed, hipStream_t stream) {
     if (rows <= 0) return 0;
-    if ((v_rope != nullptr && (value_dim > MAX_KEY_DIM || (value_dim & 1))) || key_dim > MAX_KEY_DIM || q_heads + 2 * kv_heads > 65535 || rot_dim > key_dim || (rot_dim & 1) || norm_mode < 0 ||
+    if ((v_rope != nullptr && (value_dim > MAX_KEY_DIM || (value_dim & 1))) || key_dim > MAX_KEY_DIM ||
+        q_heads + 2 * kv_heads > 65535 || rot_dim > key_dim || (rot_dim & 1) || norm_mode < 0 ||
         norm_mode > 2)
         return -1;
 #if MLR_BF16
