@@ -8,7 +8,7 @@ layer without memory.  What a page holds is the mixer's business: the spec names
 and their shape within a page, the manager only multiplies them out.  Entries with equal specs
 form a group; a group has its own pool of pages (one page id is valid in every entry of the
 group), its own page size, its own block tables and its own rule for giving pages back (all
-tokens kept, or only a window).  The bookkeeping itself (free lists, tables, lengths, invariants) is native code in
+tokens kept, or only a window, optionally with the first tokens).  The bookkeeping itself (free lists, tables, lengths, invariants) is native code in
 csrc/host/cache_manager.cpp; this module owns the device memory and keeps the device copies
 of the block tables current.
 
@@ -51,6 +51,7 @@ class PagedSpec:
     window: Optional[int] = None      # None: all tokens are kept
     page_size: Optional[int] = None
     dtype: Optional[torch.dtype] = None
+    keep_first: int = 0               # with a window: the first tokens of a request that stay as well
 
     def shape_of(self, name, page_size):
         for n, shape in self.tensors:
@@ -120,7 +121,7 @@ def _host_lib():
         lib.mlr_cache_create.argtypes = [ctypes.c_int, ctypes.c_int]
         lib.mlr_cache_destroy.argtypes = [ctypes.c_void_p]
         lib.mlr_cache_destroy.restype = None
-        lib.mlr_cache_add_group.argtypes = [ctypes.c_void_p, ctypes.c_int, ctypes.c_int, ctypes.c_int]
+        lib.mlr_cache_add_group.argtypes = [ctypes.c_void_p, ctypes.c_int, ctypes.c_int, ctypes.c_int, ctypes.c_int]
         lib.mlr_cache_max_blocks.argtypes = [ctypes.c_void_p, ctypes.c_int]
         lib.mlr_cache_free_pages.argtypes = [ctypes.c_void_p, ctypes.c_int]
         lib.mlr_cache_free_slots.argtypes = [ctypes.c_void_p]
@@ -162,8 +163,8 @@ class PageBook:
         if h:
             self._lib.mlr_cache_destroy(h)
 
-    def add_group(self, page_size, num_pages, window=None):
-        g = self._lib.mlr_cache_add_group(self._h, page_size, num_pages, window or 0)
+    def add_group(self, page_size, num_pages, window=None, keep_first=0):
+        g = self._lib.mlr_cache_add_group(self._h, page_size, num_pages, window or 0, keep_first)
         if g < 0:
             raise CacheError("page_size and num_pages must be positive")
         self.groups.append((page_size, num_pages, window))
@@ -333,7 +334,7 @@ class CacheManager:
                 if size <= 0:
                     raise CacheError("a group's page size must be positive")
                 pages = (max_tokens + size - 1) // size
-                self._group_of_spec[paged] = self.book.add_group(size, pages, paged.window)
+                self._group_of_spec[paged] = self.book.add_group(size, pages, paged.window, paged.keep_first)
                 members.append([])
                 self.group_specs.append(paged)
                 self.group_page_size.append(size)

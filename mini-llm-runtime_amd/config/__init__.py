@@ -8,8 +8,10 @@ from .pamunex import PamunexConfig
 from .tigelorn import TigelornConfig
 from .budorax import BudoraxConfig
 from .nuvorax import NuvoraxConfig
+from .sagopel import SagopelConfig
 
 __all__ = ["ConfigError", "config_class", "config_from_dict", "known_architectures", "load_config",
            "register_architecture", "AttentionSpec", "LayerRun", "LayerSpec", "MlpSpec",
            "ModelSpec", "NormSpec", "PositionSpec", "Qwen3Config", "ClampedGluSpec", "DiffAttentionSpec", "GlaSpec",
-           "Mamba2Spec", "QueryTemperature", "TaletarConfig", "PamunexConfig", "TigelornConfig", "BudoraxConfig", "NuvoraxConfig"]
+           "Mamba2Spec", "QueryTemperature", "TaletarConfig", "PamunexConfig", "TigelornConfig", "BudoraxConfig", "NuvoraxConfig",
+           "SagopelConfig"]

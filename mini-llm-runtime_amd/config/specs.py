@@ -73,7 +73,7 @@ class MlpSpec:
     kind: str                 # key in the feed-forward registry, e.g. "swiglu"
     hidden: int
     intermediate: int
-    activation: str = "silu"  # of the gate: silu, gelu_tanh
+    activation: str = "silu"  # of the gate: silu, gelu_tanh, relu
 
 
 @dataclass(frozen=True)
@@ -147,9 +147,11 @@ class ClampedGluSpec:
 @dataclass(frozen=True)
 class MaskSpec:
     """Which keys a query at position p sees besides "none after it": `window`: the last `size` positions
-    (itself and the size - 1 before it); `chunk`: the positions of its own block floor(p / size)."""
+    (itself and the size - 1 before it); `chunk`: the positions of its own block floor(p / size).  `keep_first`: a
+    window's queries see the request's first tokens as well, however far back they lie."""
     kind: str                 # "window" | "chunk"
     size: int
+    keep_first: int = 0
 
 
 @dataclass(frozen=True)
@@ -173,6 +175,7 @@ class SinkAttentionSpec:
     qk_norm_weight: bool = True                  # False: q and k are only divided by their root mean square
     qk_norm_after_rotation: bool = False         # the norm follows the rotation instead of preceding it
     gate: Optional[str] = None                   # "sigmoid": the heads side by side times sigmoid(Wg x) before Wo
+    softcap: Optional[float] = None              # score <- softcap * tanh(score / softcap)
 
 
 @dataclass(frozen=True)
@@ -221,9 +224,10 @@ class LatentAttentionSpec:
 
 @dataclass(frozen=True)
 class DecayedLinearAttentionSpec:
-    """Linear attention with ONE constant decay a head: q, k, v = act(W x); per head S_t = decay S_(t-1) + k_t v_t^T,
-    o_t = S_t^T q_t; the heads side by side are RMS-normed as one row (a weight as wide as the row), multiplied by
-    gate(Wg x) and projected by Wo."""
+    """Linear attention with ONE constant decay a head: q, k, v = act(W x), q and k optionally turned by their position and
+    k multiplied by `k_scale`; per head S_t = decay S_(t-1) + k_t v_t^T, o_t = S_t^T q_t; the heads side by side are
+    RMS-normed as one row (a weight as wide as the row) or, `norm` "heads", each head's o is divided by its own root
+    mean square (no weight); then multiplied by gate(Wg x) and projected by Wo."""
     kind: str                 # "decayed_linear_attention"
     hidden: int
     heads: int
@@ -231,8 +235,11 @@ class DecayedLinearAttentionSpec:
     value_dim: int
     decay: Tuple[float, ...]  # one number in (0, 1] a head
     eps: float
-    activation: str = "silu"
+    activation: Optional[str] = "silu"
     gate: str = "sigmoid"
+    position: Optional[PositionSpec] = None      # `dim` of it: how many of a head's first channels turn
+    k_scale: float = 1.0
+    norm: str = "row"                            # or "heads"
 
 
 @dataclass(frozen=True)
@@ -259,11 +266,13 @@ class DeltaRuleSpec:
 
 @dataclass(frozen=True)
 class MixerSumSpec:
-    """Several mixers side by side on the same input: the output is sum_i scale_i mixer_i(x).  `mixers`: (name, spec,
-    scale) each; a mixer's tensors are named `<name>.<its local name>`, and each keeps a cache entry of its own."""
+    """Several mixers side by side on the same input: the output is sum_i scale_i mixer_i(x), or with `out_norm_eps`
+    sum_i scale_i norm_i(mixer_i(x)), an RMS norm over the model's width with a weight a mixer (`<name>.out`).  `mixers`:
+    (name, spec, scale) each; a mixer's tensors are named `<name>.<its local name>`, and each keeps a cache entry of its own."""
     kind: str                 # "mixer_sum"
     hidden: int
     mixers: Tuple[Tuple[str, object, float], ...]
+    out_norm_eps: Optional[float] = None
 
 
 @dataclass(frozen=True)
@@ -300,6 +309,8 @@ class RoutedMlpSpec:
     slope: float = 1.702                  # g sigmoid(slope g) (u + 1)
     shared: Optional[object] = None       # any feed-forward spec; its tensors are named `shared.<local name>`
     shared_gate: bool = False
+    identity: int = 0                     # further router outputs behind the experts' that stand for experts without
+                                          # tensors: their output is the layer's input
 
 
 @dataclass(frozen=True)
@@ -312,6 +323,7 @@ class LayerSpec:
     ffn: object               # any feed-forward spec with a `kind`
     norm1_after: Optional[NormSpec] = None    # block "sandwich": the norm of what the mixer gives, before the residual sum
     norm2_after: Optional[NormSpec] = None    # likewise behind the feed-forward
+    residual_scale: float = 1.0       # block "prenorm": factor on what each sublayer adds to the stream
 
 
 @dataclass(frozen=True)
@@ -323,6 +335,8 @@ class LayerRun:
     write_cache: bool = True
     add_embedding: bool = False   # the embedding's output (the stream as it was before the first run) is added to
                                   # the stream right before this run: the start of a further pass over looped layers
+    add_vector: Optional[int] = None  # this row of the model's run vectors is added to the stream (every token's) right
+                                      # before this run: the start of a pass that has a vector of its own
 
 
 @dataclass(frozen=True)
@@ -343,6 +357,14 @@ class PairEmbedSpec:
     buckets: int
     mul_prev: int
     mul_cur: int
+
+
+@dataclass(frozen=True)
+class RunVectorsSpec:
+    """Learned vectors as wide as the model, [count, hidden], that runs of the schedule add to the stream (`add_vector`)."""
+    kind: str                 # key in the embed registry: "run_vectors"
+    count: int
+    hidden: int
 
 
 @dataclass(frozen=True)
@@ -368,6 +390,7 @@ class ModelSpec:
     eos_token_ids: Tuple[int, ...] = field(default_factory=tuple)
     embed: Optional[object] = None      # any embed spec with a `kind`; None: a plain table [vocab_size, hidden]
     head: Optional[object] = None       # any head spec with a `kind`; None: a plain projection, tied as `tie_embeddings` says
+    run_vectors: Optional[RunVectorsSpec] = None
 
     def embed_spec(self):
         return self.embed if self.embed is not None else EmbedSpec("token_embedding", self.vocab_size, self.hidden)

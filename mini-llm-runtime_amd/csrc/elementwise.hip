@@ -30,21 +30,50 @@ __device__ __forceinline__ float block_max(float v, float* scratch) {
     return total;
 }
 
+// What a row of the residual stream still lacks: `factor` times a row of a sublayer's output (in the engine's element
+// type) plus a vector that joins every row; either may be null.  (A factor of 1 gives the plain sum's bits.)
+struct RowAddend {
+    const elem_t* delta; float factor;
+    const float* vector;
+    __device__ __forceinline__ bool any() const { return delta != nullptr || vector != nullptr; }
+    __device__ __forceinline__ RowAddend of_row(size_t row, int width) const {
+        return RowAddend{delta ? delta + row * width : nullptr, factor, vector};
+    }
+    __device__ __forceinline__ float to(float x, int i) const {
+        if (delta) x = fmaf(factor, to_float(delta[i]), x);
+        if (vector) x += vector[i];
+        return x;
+    }
+    // MLR_VEC values from channel c on
+    __device__ __forceinline__ void to_vec(float* x, int c) const {
+        if (delta) {
+            float dv[MLR_VEC];
+            load_vec(delta + c, dv);
+#pragma unroll
+            for (int e = 0; e < MLR_VEC; ++e) x[e] = fmaf(factor, dv[e], x[e]);
+        }
+        if (vector) {
+#pragma unroll
+            for (int e = 0; e < MLR_VEC; ++e) x[e] += vector[c + e];
+        }
+    }
+};
+
 // A row whose sum of squares does not fit 32 bits (elements beyond about 1e19) or is no number: the
 // reference's way of norming (src/minillm/cuda/ops.cu:87-126), the row divided by its largest element before
 // it is squared, and eps scaled alike: largest = max(max |x|, sqrt(eps)), den = sqrt(mean((x / largest)^2) +
 // eps / largest^2), y = ((x / largest) / den) * w; a row with an infinity or a NaN comes out as NaN.  The usual
-// row never gets here, so it keeps its one pass and its bits.  x = hrow + drow (drow: what is still to be
-// added, or null).  WAVE: one wavefront serves the row, else the whole workgroup (every thread of it must
+// row never gets here, so it keeps its one pass and its bits.  x = hrow + what is still to be
+// added (`more`).  WAVE: one wavefront serves the row, else the whole workgroup (every thread of it must
 // call, `scratch` holds 16 floats of LDS).
 template <bool WAVE>
-__device__ void norm_row_rescaled(const float* hrow, const elem_t* drow, const float* __restrict__ weight,
+__device__ void norm_row_rescaled(const float* hrow, const RowAddend more, const float* __restrict__ weight,
                                   elem_t* __restrict__ orow, int width, float eps, float* scratch) {
     __threadfence_block();                     // (the row may have been written back by other lanes just now)
     const int t = WAVE ? (int)(threadIdx.x & 63) : (int)threadIdx.x, step = WAVE ? 64 : (int)blockDim.x;
     float largest = 0.f;
     for (int i = t; i < width; i += step) {
-        const float x = hrow[i] + (drow ? to_float(drow[i]) : 0.f);
+        const float x = more.to(hrow[i], i);
         largest = fmaxf(largest, isfinite(x) ? fabsf(x) : INFINITY);
     }
     largest = WAVE ? wave_max(largest) : block_max(largest, scratch);
@@ -55,21 +84,21 @@ __device__ void norm_row_rescaled(const float* hrow, const elem_t* drow, const f
     }
     float sum = 0.f;
     for (int i = t; i < width; i += step) {
-        const float scaled = (hrow[i] + (drow ? to_float(drow[i]) : 0.f)) / largest;
+        const float scaled = more.to(hrow[i], i) / largest;
         sum += scaled * scaled;
     }
     sum = WAVE ? wave_sum(sum) : block_sum(sum, scratch);
     const float den = sqrtf(sum / (float)width + (eps / largest) / largest);
     for (int i = t; i < width; i += step) {
-        const float x = hrow[i] + (drow ? to_float(drow[i]) : 0.f);
+        const float x = more.to(hrow[i], i);
         orow[i] = from_float<elem_t>(((x / largest) / den) * weight[i]);
     }
 }
 
-// For output row r: src = rows ? rows[r] : r;  x = h[src] + (delta ? delta[src] : 0);
+// For output row r: src = rows ? rows[r] : r;  x = h[src] + what is still to be added to it;
 // if write_h: h[src] = x;  out[r] = (x * rsqrt(mean(x^2) + eps)) * weight.
 // One workgroup per row; the sum of squares is taken over the row in a fixed order.
-__global__ void add_rmsnorm_kernel(float* __restrict__ h, const elem_t* __restrict__ delta,
+__global__ void add_rmsnorm_kernel(float* __restrict__ h, const RowAddend addend,
                                    const float* __restrict__ weight, elem_t* __restrict__ out,
                                    const int32_t* __restrict__ rows, int width, float eps,
                                    int write_h) {
@@ -77,12 +106,12 @@ __global__ void add_rmsnorm_kernel(float* __restrict__ h, const elem_t* __restri
     const int r = blockIdx.x;
     const size_t src = rows ? (size_t)rows[r] : (size_t)r;
     float* hrow = h + src * width;
-    const elem_t* drow = delta ? delta + src * width : nullptr;
+    const RowAddend more = addend.of_row(src, width);
     float sum = 0.f;
     for (int i = threadIdx.x; i < width; i += blockDim.x) {
         float x = hrow[i];
-        if (drow) {
-            x += to_float(drow[i]);
+        if (more.any()) {
+            x = more.to(x, i);
             if (write_h) hrow[i] = x;
         }
         sum += x * x;
@@ -90,20 +119,20 @@ __global__ void add_rmsnorm_kernel(float* __restrict__ h, const elem_t* __restri
     sum = block_sum(sum, scratch);
     elem_t* orow = out + (size_t)r * width;
     if (!isfinite(sum)) {                      // (the same in every thread of the workgroup)
-        norm_row_rescaled<false>(hrow, (drow && !write_h) ? drow : nullptr, weight, orow, width, eps, scratch);
+        norm_row_rescaled<false>(hrow, write_h ? RowAddend{nullptr, 1.f, nullptr} : more, weight, orow, width, eps, scratch);
         return;
     }
     const float scale = 1.0f / sqrtf(sum / (float)width + eps);
     for (int i = threadIdx.x; i < width; i += blockDim.x) {
         float x = hrow[i];
-        if (drow && !write_h) x += to_float(drow[i]);
+        if (!write_h) x = more.to(x, i);
         orow[i] = from_float<elem_t>((x * scale) * weight[i]);
     }
 }
 
 // One workgroup per row as above, 16 bytes per thread and access (width a multiple of MLR_VEC): for few
 // rows of the bfloat16 engine, where the scalar kernel's latency would show.
-__global__ __launch_bounds__(256) void add_rmsnorm_row_vec_kernel(float* __restrict__ h, const elem_t* __restrict__ delta,
+__global__ __launch_bounds__(256) void add_rmsnorm_row_vec_kernel(float* __restrict__ h, const RowAddend addend,
                                                                   const float* __restrict__ weight,
                                                                   elem_t* __restrict__ out, const int32_t* __restrict__ rows,
                                                                   int width, float eps, int write_h) {
@@ -111,7 +140,7 @@ __global__ __launch_bounds__(256) void add_rmsnorm_row_vec_kernel(float* __restr
     const int r = blockIdx.x;
     const size_t src = rows ? (size_t)rows[r] : (size_t)r;
     float* hrow = h + src * width;
-    const elem_t* drow = delta ? delta + src * width : nullptr;
+    const RowAddend more = addend.of_row(src, width);
     float sum = 0.f;
     for (int c = threadIdx.x * MLR_VEC; c < width; c += 256 * MLR_VEC) {
         float x[MLR_VEC];
@@ -120,11 +149,8 @@ __global__ __launch_bounds__(256) void add_rmsnorm_row_vec_kernel(float* __restr
             const float4 v = *reinterpret_cast<const float4*>(hrow + c + e);
             x[e] = v.x; x[e + 1] = v.y; x[e + 2] = v.z; x[e + 3] = v.w;
         }
-        if (drow) {
-            float dv[MLR_VEC];
-            load_vec(drow + c, dv);
-#pragma unroll
-            for (int e = 0; e < MLR_VEC; ++e) x[e] += dv[e];
+        if (more.any()) {
+            more.to_vec(x, c);
             if (write_h) {
 #pragma unroll
                 for (int e = 0; e < MLR_VEC; e += 4)
@@ -137,7 +163,7 @@ __global__ __launch_bounds__(256) void add_rmsnorm_row_vec_kernel(float* __restr
     sum = block_sum(sum, scratch);
     elem_t* orow = out + (size_t)r * width;
     if (!isfinite(sum)) {
-        norm_row_rescaled<false>(hrow, (drow && !write_h) ? drow : nullptr, weight, orow, width, eps, scratch);
+        norm_row_rescaled<false>(hrow, write_h ? RowAddend{nullptr, 1.f, nullptr} : more, weight, orow, width, eps, scratch);
         return;
     }
     const float scale = 1.0f / sqrtf(sum / (float)width + eps);
@@ -148,12 +174,7 @@ __global__ __launch_bounds__(256) void add_rmsnorm_row_vec_kernel(float* __restr
             const float4 v = *reinterpret_cast<const float4*>(hrow + c + e);
             x[e] = v.x; x[e + 1] = v.y; x[e + 2] = v.z; x[e + 3] = v.w;
         }
-        if (drow && !write_h) {
-            float dv[MLR_VEC];
-            load_vec(drow + c, dv);
-#pragma unroll
-            for (int e = 0; e < MLR_VEC; ++e) x[e] += dv[e];
-        }
+        if (!write_h) more.to_vec(x, c);
 #pragma unroll
         for (int e = 0; e < MLR_VEC; e += 4) {
             const float4 w = *reinterpret_cast<const float4*>(weight + c + e);
@@ -170,7 +191,7 @@ __global__ __launch_bounds__(256) void add_rmsnorm_row_vec_kernel(float* __restr
 // one wavefront per row, four rows per workgroup, the row kept in registers between the two passes
 // when it fits (width <= 64 * MLR_VEC * ROW_REGS), else re-read.
 #define ROW_REGS 4
-__global__ __launch_bounds__(256) void add_rmsnorm_vec_kernel(float* __restrict__ h, const elem_t* __restrict__ delta,
+__global__ __launch_bounds__(256) void add_rmsnorm_vec_kernel(float* __restrict__ h, const RowAddend addend,
                                                               const float* __restrict__ weight,
                                                               elem_t* __restrict__ out, const int32_t* __restrict__ rows,
                                                               int n_out, int width, float eps, int write_h) {
@@ -179,7 +200,7 @@ __global__ __launch_bounds__(256) void add_rmsnorm_vec_kernel(float* __restrict_
     if (r >= n_out) return;
     const size_t src = rows ? (size_t)rows[r] : (size_t)r;
     float* hrow = h + src * width;
-    const elem_t* drow = delta ? delta + src * width : nullptr;
+    const RowAddend more = addend.of_row(src, width);
     float x[ROW_REGS][MLR_VEC];
     float sum = 0.f;
 #pragma unroll
@@ -191,11 +212,8 @@ __global__ __launch_bounds__(256) void add_rmsnorm_vec_kernel(float* __restrict_
                 const float4 v = *reinterpret_cast<const float4*>(hrow + c + e);
                 x[i][e] = v.x; x[i][e + 1] = v.y; x[i][e + 2] = v.z; x[i][e + 3] = v.w;
             }
-            if (drow) {
-                float dv[MLR_VEC];
-                load_vec(drow + c, dv);
-#pragma unroll
-                for (int e = 0; e < MLR_VEC; ++e) x[i][e] += dv[e];
+            if (more.any()) {
+                more.to_vec(x[i], c);
                 if (write_h) {
 #pragma unroll
                     for (int e = 0; e < MLR_VEC; e += 4)
@@ -209,7 +227,7 @@ __global__ __launch_bounds__(256) void add_rmsnorm_vec_kernel(float* __restrict_
     sum = wave_sum(sum);
     elem_t* orow = out + (size_t)r * width;
     if (!isfinite(sum)) {                      // (the same in every lane of the wavefront, which serves this row alone)
-        norm_row_rescaled<true>(hrow, (drow && !write_h) ? drow : nullptr, weight, orow, width, eps, nullptr);
+        norm_row_rescaled<true>(hrow, write_h ? RowAddend{nullptr, 1.f, nullptr} : more, weight, orow, width, eps, nullptr);
         return;
     }
     const float scale = 1.0f / sqrtf(sum / (float)width + eps);
@@ -231,18 +249,22 @@ __global__ __launch_bounds__(256) void add_rmsnorm_vec_kernel(float* __restrict_
     }
 }
 
-// h[m, :] += delta[m, :] (the last residual sum when nothing is normed afterwards).
-__global__ void residual_add_kernel(float* __restrict__ h, const elem_t* __restrict__ delta, size_t count) {
+// h[m, :] += factor * delta[m, :] + vector (the last residual sum when nothing is normed afterwards).
+__global__ void residual_add_kernel(float* __restrict__ h, const RowAddend addend, int width, size_t count) {
     for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < count;
          i += (size_t)gridDim.x * blockDim.x) {
-        h[i] += to_float(delta[i]);
+        float x = h[i];
+        if (addend.delta) x = fmaf(addend.factor, to_float(addend.delta[i]), x);
+        if (addend.vector) x += addend.vector[i % width];
+        h[i] = x;
     }
 }
 
 // The activation of a gated feed-forward's gate: ACT 0 silu(g) = g / (1 + exp(-g)); ACT 1 the tanh form of gelu,
-// 0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3))).  32-bit.
+// 0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3))); ACT 2 max(g, 0).  32-bit.
 template <int ACT>
 __device__ __forceinline__ float gate_act(float g) {
+    if (ACT == 2) return fmaxf(g, 0.f);
     if (ACT == 1) return 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
     return g / (1.0f + expf(-g));
 }
@@ -345,6 +367,40 @@ __global__ void scaled_sum_kernel(const elem_t* __restrict__ a, const elem_t* __
         out[i] = from_float<elem_t>(sa * to_float(a[i]) + sb * to_float(b[i]));
 }
 
+// out[m] = sa * norm(a[m]) + sb * norm(b[m]): two sublayers' rows, each over its own root mean square times a weight as wide
+// as the row (a null weight: the row as it is, not normed), added in 32-bit.  One workgroup a row; VEC: MLR_VEC values in
+// one access, or 1.
+template <int VEC>
+__global__ __launch_bounds__(256) void normed_sum_kernel(const elem_t* __restrict__ a, const elem_t* __restrict__ b,
+                                                         const float* __restrict__ wa, const float* __restrict__ wb,
+                                                         elem_t* __restrict__ out, float sa, float sb, int width, float eps) {
+    __shared__ float scratch[16];
+    const elem_t* arow = a + (size_t)blockIdx.x * width;
+    const elem_t* brow = b + (size_t)blockIdx.x * width;
+    float suma = 0.f, sumb = 0.f;
+    for (int c = threadIdx.x * VEC; c < width; c += 256 * VEC) {
+        float x[MLR_VEC], y[MLR_VEC];
+        if (VEC > 1) { load_vec(arow + c, x); load_vec(brow + c, y); }
+        else { x[0] = to_float(arow[c]); y[0] = to_float(brow[c]); }
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) { suma += x[e] * x[e]; sumb += y[e] * y[e]; }
+    }
+    suma = block_sum(suma, scratch);
+    sumb = block_sum(sumb, scratch);
+    const float fa = wa ? sa / sqrtf(suma / (float)width + eps) : sa, fb = wb ? sb / sqrtf(sumb / (float)width + eps) : sb;
+    elem_t* orow = out + (size_t)blockIdx.x * width;
+    for (int c = threadIdx.x * VEC; c < width; c += 256 * VEC) {
+        float x[MLR_VEC], y[MLR_VEC];
+        if (VEC > 1) { load_vec(arow + c, x); load_vec(brow + c, y); }
+        else { x[0] = to_float(arow[c]); y[0] = to_float(brow[c]); }
+#pragma unroll
+        for (int e = 0; e < VEC; ++e)
+            x[e] = (x[e] * fa) * (wa ? wa[c + e] : 1.f) + (y[e] * fb) * (wb ? wb[c + e] : 1.f);
+        if (VEC > 1) store_vec(orow + c, x);
+        else orow[c] = from_float<elem_t>(x[0]);
+    }
+}
+
 // The first half of an RMSNorm whose scale is applied by the projection that follows (few rows): x = h + delta
 // (delta may be null; written back to h when write_h), out = elem(x * weight) WITHOUT the scale, and the row's
 // sum of squares ss[r] (one "partial" sum a row).  One workgroup per row, sums in a fixed order.
@@ -380,15 +436,15 @@ __global__ void status_reset_kernel(int32_t* __restrict__ status) {
     }
 }
 
-// One workgroup per row of x = h + delta (delta may be null): which kinds of non-finite values it holds.
-__global__ void finite_check_kernel(const float* __restrict__ h, const elem_t* __restrict__ delta, int width, int layer,
+// One workgroup per row of x = h + factor * delta (delta may be null): which kinds of non-finite values it holds.
+__global__ void finite_check_kernel(const float* __restrict__ h, const elem_t* __restrict__ delta, float factor, int width, int layer,
                                     int32_t* __restrict__ status) {
     const int r = blockIdx.x;
     const float* hrow = h + (size_t)r * width;
     const elem_t* drow = delta ? delta + (size_t)r * width : nullptr;
     int bits = 0;
     for (int i = threadIdx.x; i < width; i += blockDim.x) {
-        const float x = hrow[i] + (drow ? to_float(drow[i]) : 0.f);
+        const float x = hrow[i] + (drow ? factor * to_float(drow[i]) : 0.f);
         const uint32_t u = __float_as_uint(x) & 0x7fffffffu;
         if (u > 0x7f800000u) bits |= 1;
         else if (u == 0x7f800000u) bits |= 2;
@@ -489,7 +545,7 @@ __global__ __launch_bounds__(256) void gated_part_norm_kernel(const float* __res
         const int c = c0 + i;
         float v = yrow[c];
         if (gate_first) v *= gate_of(c);
-        v = (v * scale) * weight[c % period];
+        v = (v * scale) * (weight ? weight[c % period] : 1.f);
         if (!gate_first) v *= gate_of(c);
         out[m * width + c] = from_float<elem_t>(v);
     }
@@ -616,14 +672,14 @@ __global__ __launch_bounds__(256) void gated_part_norm_vec_kernel(const float* _
         if (gate_first) {
             gated(c, v, true);
 #pragma unroll
-            for (int e = 0; e < 8; ++e) o[e] = (v[e] * scale) * weight[(c + e) % period];
+            for (int e = 0; e < 8; ++e) o[e] = (v[e] * scale) * (weight ? weight[(c + e) % period] : 1.f);
         } else {
             float gt[8];
             gated(c, gt, false);
             const float4 lo = *reinterpret_cast<const float4*>(yrow + c), hi = *reinterpret_cast<const float4*>(yrow + c + 4);
             v[0] = lo.x; v[1] = lo.y; v[2] = lo.z; v[3] = lo.w; v[4] = hi.x; v[5] = hi.y; v[6] = hi.z; v[7] = hi.w;
 #pragma unroll
-            for (int e = 0; e < 8; ++e) o[e] = ((v[e] * scale) * weight[(c + e) % period]) * gt[e];
+            for (int e = 0; e < 8; ++e) o[e] = ((v[e] * scale) * (weight ? weight[(c + e) % period] : 1.f)) * gt[e];
         }
         store_vec(out + m * width + c, o);
     }
@@ -979,21 +1035,22 @@ int mlr_embed_gather(const int32_t* ids, const void* table, float* h, int rows, 
     return (int)hipGetLastError();
 }
 
-int mlr_add_rmsnorm(float* h, const void* delta, const float* weight, void* out, const int32_t* rows,
-                    int n_out, int width, float eps, int write_h, hipStream_t stream) {
+int mlr_add_rmsnorm(float* h, const void* delta, float factor, const float* vector, const float* weight, void* out,
+                    const int32_t* rows, int n_out, int width, float eps, int write_h, hipStream_t stream) {
     if (n_out <= 0) return 0;
+    const RowAddend addend{(const elem_t*)delta, factor, vector};
     // (the float engine keeps its one order of additions for every batch size)
     if (MLR_BF16 && width % MLR_VEC == 0 && width <= 64 * MLR_VEC * ROW_REGS && n_out >= 64) {
-        add_rmsnorm_vec_kernel<<<(n_out + 3) / 4, 256, 0, stream>>>(h, (const elem_t*)delta, weight, (elem_t*)out,
+        add_rmsnorm_vec_kernel<<<(n_out + 3) / 4, 256, 0, stream>>>(h, addend, weight, (elem_t*)out,
                                                                      rows, n_out, width, eps, write_h);
         return (int)hipGetLastError();
     }
     if (MLR_BF16 && width % MLR_VEC == 0) {
-        add_rmsnorm_row_vec_kernel<<<n_out, 256, 0, stream>>>(h, (const elem_t*)delta, weight, (elem_t*)out, rows,
+        add_rmsnorm_row_vec_kernel<<<n_out, 256, 0, stream>>>(h, addend, weight, (elem_t*)out, rows,
                                                               width, eps, write_h);
         return (int)hipGetLastError();
     }
-    add_rmsnorm_kernel<<<n_out, 256, 0, stream>>>(h, (const elem_t*)delta, weight, (elem_t*)out, rows,
+    add_rmsnorm_kernel<<<n_out, 256, 0, stream>>>(h, addend, weight, (elem_t*)out, rows,
                                                   width, eps, write_h);
     return (int)hipGetLastError();
 }
@@ -1010,17 +1067,19 @@ int mlr_status_reset(int32_t* status, hipStream_t stream) {
     return (int)hipGetLastError();
 }
 
-int mlr_finite_check(const float* h, const void* delta, int rows, int width, int layer, int32_t* status,
+int mlr_finite_check(const float* h, const void* delta, float factor, int rows, int width, int layer, int32_t* status,
                      hipStream_t stream) {
     if (rows <= 0) return 0;
     if (layer < 0 || layer >= 2047) return -1;
-    finite_check_kernel<<<rows, 256, 0, stream>>>(h, (const elem_t*)delta, width, layer, status);
+    finite_check_kernel<<<rows, 256, 0, stream>>>(h, (const elem_t*)delta, factor, width, layer, status);
     return (int)hipGetLastError();
 }
 
-int mlr_residual_add(float* h, const void* delta, size_t count, hipStream_t stream) {
+int mlr_residual_add(float* h, const void* delta, float factor, const float* vector, int width, size_t count,
+                     hipStream_t stream) {
     if (count == 0) return 0;
-    residual_add_kernel<<<grid_for(count, 256), 256, 0, stream>>>(h, (const elem_t*)delta, count);
+    if (width < 1) return -1;
+    residual_add_kernel<<<grid_for(count, 256), 256, 0, stream>>>(h, RowAddend{(const elem_t*)delta, factor, vector}, width, count);
     return (int)hipGetLastError();
 }
 
@@ -1029,11 +1088,12 @@ int mlr_silu_mul(const void* gate_up, void* act, int rows, int inter, hipStream_
     return launch_gated<0>(gate_up, act, rows, inter, stream);
 }
 
-// act = activation(gate) * up; kind 0: silu, 1: the tanh form of gelu
+// act = activation(gate) * up; kind 0: silu, 1: the tanh form of gelu, 2: relu
 int mlr_gated_act_mul(const void* gate_up, void* act, int rows, int inter, int kind, hipStream_t stream) {
     if (rows <= 0) return 0;
     if (kind == 0) return launch_gated<0>(gate_up, act, rows, inter, stream);
     if (kind == 1) return launch_gated<1>(gate_up, act, rows, inter, stream);
+    if (kind == 2) return launch_gated<2>(gate_up, act, rows, inter, stream);
     return -1;
 }
 
@@ -1073,6 +1133,16 @@ int mlr_rmsnorm_columns(const void* x, long x_stride, const float* weight, void*
 int mlr_scaled_sum(const void* a, const void* b, void* out, float sa, float sb, size_t count, hipStream_t stream) {
     if (count == 0) return 0;
     scaled_sum_kernel<<<grid_for(count, 256), 256, 0, stream>>>((const elem_t*)a, (const elem_t*)b, (elem_t*)out, sa, sb, count);
+    return (int)hipGetLastError();
+}
+
+int mlr_normed_sum(const void* a, const void* b, const float* wa, const float* wb, void* out, float sa, float sb, int rows,
+                   int width, float eps, hipStream_t stream) {
+    if (rows <= 0) return 0;
+    if (MLR_BF16 && width % MLR_VEC == 0 && aligned16(a, b, out))
+        normed_sum_kernel<MLR_VEC><<<rows, 256, 0, stream>>>((const elem_t*)a, (const elem_t*)b, wa, wb, (elem_t*)out, sa, sb, width, eps);
+    else
+        normed_sum_kernel<1><<<rows, 256, 0, stream>>>((const elem_t*)a, (const elem_t*)b, wa, wb, (elem_t*)out, sa, sb, width, eps);
     return (int)hipGetLastError();
 }
 

@@ -210,7 +210,7 @@ struct SkinnyEpilogue {
     int cols;                 // PAIR: the output columns of a workgroup, 17..32 (otherwise 16, whatever this says)
     int ss_stride;            // floats between the rows of ss_out (its capacity: a strip of 16 a part)
     float glu_limit;          // GATED: > 0: the clamped gate g = min(gate, limit), u = clamp(up, +-limit),
-    float glu_slope;          //        y = g sigmoid(slope g) (u + 1); 0: y = silu(gate) up; < 0: y = gelu_tanh(gate) up
+    float glu_slope;          //        y = g sigmoid(slope g) (u + 1); 0: y = silu(gate) up; -1: gelu_tanh(gate) up; -2: relu(gate) up
     int plain_act;            // a plain product's activation: 0 none, 1 relu(x)^2, 2 the exact gelu x Phi(x)
 };
 __device__ __forceinline__ float plain_activation(float x, int act) {
@@ -450,6 +450,8 @@ __global__ __launch_bounds__(SKINNY_WAVES * 64) void gemm_skinny_kernel(const __
                     const float gg = fminf(v[0], epi.glu_limit);
                     const float uu = fminf(fmaxf(v[NW - 1], -epi.glu_limit), epi.glu_limit);
                     y = (gg / (1.0f + expf(-epi.glu_slope * gg))) * (uu + 1.0f);
+                } else if (epi.glu_limit < -1.5f) {
+                    y = fmaxf(v[0], 0.f) * v[NW - 1];
                 } else if (epi.glu_limit < 0.f) {
                     const float gg = v[0];
                     y = 0.5f * gg * (1.0f + tanhf(0.7978845608028654f * (gg + 0.044715f * gg * gg * gg))) * v[NW - 1];
@@ -1014,13 +1016,13 @@ extern "C" int mlr_gemm_gated_clamped(const void* a, const void* w, void* out, i
     return 1;
 }
 
-// out[M, N] = gelu_tanh(a . w[0:N]^T) * (a . w[N:2N]^T), gelu_tanh(g) = 0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3))):
-// the gate as the epilogue of the weight-streaming kernels, up to 64 rows.  Returns 1 for more rows.
-extern "C" int mlr_gemm_gated_gelu_tanh(const void* a, const void* w, void* out, int M, int N, int K, hipStream_t stream) {
+// out[M, N] = act(a . w[0:N]^T) * (a . w[N:2N]^T), act 1 the tanh form of gelu, 0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715
+// g^3))), or 2 relu: the gate as the epilogue of the weight-streaming kernels, up to 64 rows.  Returns 1 for more rows.
+extern "C" int mlr_gemm_gated_act(const void* a, const void* w, void* out, int M, int N, int K, int act, hipStream_t stream) {
     if (M <= 0 || N <= 0) return 0;
-    if (K <= 0) return -1;
+    if (K <= 0 || act < 1 || act > 2) return -1;
     SkinnyEpilogue epi{};
-    epi.glu_limit = -1.0f;
+    epi.glu_limit = -(float)act;
     if (M <= 16) return launch_skinny<1, true>(a, w, out, M, N, K, 0, stream, epi);
     if (M <= 32) return launch_skinny<2, true>(a, w, out, M, N, K, 0, stream, epi);
     if (M <= 64) return launch_skinny<4, true>(a, w, out, M, N, K, 0, stream, epi);

@@ -420,13 +420,20 @@ __global__ __launch_bounds__(1024) void route_sort_kernel(const int32_t* __restr
 }
 
 // out[m, :] = sum_i weights[m][i] * y[row_of[m * top + i], :], the sum in 32-bit in the order of the choices; with
-// `shared` [rows, width] plus shared[m, :], times sigmoid(shared_gate[m * gate_stride]) when that is given.
+// `shared` [rows, width] plus shared[m, :], times sigmoid(shared_gate[m * gate_stride]) when that is given.  With `ids`
+// [rows, top] a choice ids[m * top + i] >= experts stands for an expert that gives its input back: x[m, :] takes its row's
+// place (no row of y was computed for it).
 // VEC: MLR_VEC values in one access, or 1.
 template <int VEC>
 __global__ void route_combine_kernel(const elem_t* __restrict__ y, const int32_t* __restrict__ row_of,
                                      const float* __restrict__ weights, elem_t* __restrict__ out, int width, int top,
-                                     const elem_t* __restrict__ shared, const float* __restrict__ shared_gate, long gate_stride) {
+                                     const elem_t* __restrict__ shared, const float* __restrict__ shared_gate, long gate_stride,
+                                     const int32_t* __restrict__ ids, int experts, const elem_t* __restrict__ x) {
     const int m = blockIdx.x;
+    auto source = [&](int i) {
+        if (ids != nullptr && ids[(size_t)m * top + i] >= experts) return x + (size_t)m * width;
+        return y + (size_t)row_of[(size_t)m * top + i] * width;
+    };
     const float f = shared_gate != nullptr ? 1.0f / (1.0f + expf(-shared_gate[(size_t)m * gate_stride])) : 1.0f;
     if (VEC > 1) {
         for (int c = threadIdx.x * VEC; c < width; c += blockDim.x * VEC) {
@@ -435,7 +442,7 @@ __global__ void route_combine_kernel(const elem_t* __restrict__ y, const int32_t
             for (int e = 0; e < MLR_VEC; ++e) sum[e] = 0.f;
             for (int i = 0; i < top; ++i) {
                 const float w = weights[(size_t)m * top + i];
-                load_vec(y + (size_t)row_of[(size_t)m * top + i] * width + c, v);
+                load_vec(source(i) + c, v);
 #pragma unroll
                 for (int e = 0; e < MLR_VEC; ++e) sum[e] = fmaf(w, v[e], sum[e]);
             }
@@ -451,7 +458,7 @@ __global__ void route_combine_kernel(const elem_t* __restrict__ y, const int32_t
     for (int c = threadIdx.x; c < width; c += blockDim.x) {
         float sum = 0.f;
         for (int i = 0; i < top; ++i)
-            sum = fmaf(weights[(size_t)m * top + i], to_float(y[(size_t)row_of[(size_t)m * top + i] * width + c]), sum);
+            sum = fmaf(weights[(size_t)m * top + i], to_float(source(i)[c]), sum);
         if (shared != nullptr) sum = fmaf(f, to_float(shared[(size_t)m * width + c]), sum);
         out[(size_t)m * width + c] = from_float<elem_t>(sum);
     }
@@ -514,16 +521,20 @@ int mlr_route_sort(const int32_t* ids, int pairs, int top, int experts, int32_t*
 }
 
 int mlr_route_combine(const void* y, const int32_t* row_of, const float* weights, void* out, int rows, int width,
-                      int top, const void* shared, const float* shared_gate, long gate_stride, hipStream_t stream) {
+                      int top, const void* shared, const float* shared_gate, long gate_stride, const int32_t* ids, int experts,
+                      const void* x, hipStream_t stream) {
     if (rows <= 0) return 0;
+    if ((ids == nullptr) != (x == nullptr)) return -1;
     const bool vec = width % MLR_VEC == 0 && ((reinterpret_cast<uintptr_t>(y) | reinterpret_cast<uintptr_t>(out) |
-                                              reinterpret_cast<uintptr_t>(shared)) & 15) == 0;
+                                              reinterpret_cast<uintptr_t>(shared) | reinterpret_cast<uintptr_t>(x)) & 15) == 0;
     if (vec)
         route_combine_kernel<MLR_VEC><<<rows, 256, 0, stream>>>((const elem_t*)y, row_of, weights, (elem_t*)out, width, top,
-                                                                (const elem_t*)shared, shared_gate, gate_stride);
+                                                                (const elem_t*)shared, shared_gate, gate_stride, ids, experts,
+                                                                (const elem_t*)x);
     else
         route_combine_kernel<1><<<rows, 256, 0, stream>>>((const elem_t*)y, row_of, weights, (elem_t*)out, width, top,
-                                                          (const elem_t*)shared, shared_gate, gate_stride);
+                                                          (const elem_t*)shared, shared_gate, gate_stride, ids, experts,
+                                                          (const elem_t*)x);
     return (int)hipGetLastError();
 }
 

@@ -18,6 +18,7 @@ namespace {
 
 struct Group {
     int page_size = 0, num_pages = 0, window = 0, max_blocks = 0;
+    int keep_blocks = 0;                     // a window gives back no page below this block: the first tokens stay
     std::vector<int32_t> free_list;          // LIFO: the page freed last is taken first
     std::vector<int32_t> table;              // [slots][max_blocks]
     std::vector<int32_t> owner;              // [num_pages]: slot or -1
@@ -66,14 +67,16 @@ void* mlr_cache_create(int max_slots, int max_length) {
 
 void mlr_cache_destroy(void* h) { delete static_cast<Cache*>(h); }
 
-// window <= 0: every key is kept.  Returns the group's index or -1.
-int mlr_cache_add_group(void* h, int page_size, int num_pages, int window) {
+// window <= 0: every key is kept.  keep_first: with a window, the sequence's first tokens stay as well.  Returns the
+// group's index or -1.
+int mlr_cache_add_group(void* h, int page_size, int num_pages, int window, int keep_first) {
     auto* c = static_cast<Cache*>(h);
     if (page_size <= 0 || num_pages <= 0) return -1;
     Group g;
     g.page_size = page_size;
     g.num_pages = num_pages;
     g.window = window > 0 ? window : 0;
+    g.keep_blocks = keep_first > 0 ? blocks_for(keep_first, page_size) : 0;
     g.max_blocks = blocks_for(c->max_length, page_size);
     // A fresh pool hands its pages out in a fixed shuffled order.  In ascending order, requests of equal
     // length that start together lie a power of two apart, and the workgroups that read block i of each of
@@ -201,7 +204,7 @@ int mlr_cache_commit_first(void* h, const int32_t* slots, const int32_t* counts,
 }
 
 // After the step ran: in groups with a window, pages whose keys no later query can see go
-// back to the pool.  A query at position >= length sees keys > position - window.
+// back to the pool.  A query at position >= length sees keys > position - window (and the group's first tokens).
 int mlr_cache_retire(void* h, const int32_t* slots, int n) {
     auto* c = static_cast<Cache*>(h);
     int freed = 0;
@@ -213,7 +216,7 @@ int mlr_cache_retire(void* h, const int32_t* slots, int n) {
             const int first_needed = std::max(0, c->length[s] - g.window + 1);   // lowest key still seen
             const int keep_from = first_needed / g.page_size;
             int32_t* row = g.table.data() + (size_t)s * g.max_blocks;
-            for (int b = g.first_block[s]; b < keep_from; ++b) {
+            for (int b = std::max(g.first_block[s], g.keep_blocks); b < keep_from; ++b) {
                 if (row[b] >= 0) {
                     g.owner[row[b]] = -1;
                     g.free_list.push_back(row[b]);
@@ -258,7 +261,7 @@ int mlr_cache_check(void* h) {
             for (int b = 0; b < g.max_blocks; ++b) {
                 const int p = row[b];
                 if (p < 0) {
-                    if (b < used && b >= g.first_block[s]) return 2;       // a needed page is missing
+                    if (b < used && (b >= g.first_block[s] || b < g.keep_blocks)) return 2;       // a needed page is missing
                     continue;
                 }
                 if (b >= used || p >= g.num_pages || seen[p]++ || g.owner[p] != s) return 3;

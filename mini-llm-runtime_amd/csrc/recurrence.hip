@@ -108,6 +108,9 @@ struct ScanArgs {
     int heads, heads_per_group, N, V, decay_per_channel, write_state;
     float q_scale;
     int silu;                                  // q, k and v pass silu as they are read (before the factors)
+    // q and k are turned as they are read (null: not): the first rot_dim channels of a head by the token's position, in
+    // pairs (i, i + rot_dim / 2), rope [positions][rot_dim] holding cosines, then sines; 32-bit
+    const float* rope; const int32_t* positions; int rot_dim;
     float* piece_state;                        // [pieces][heads][N][V]: L_c after the first pass, S_c after the second
     float* piece_decay;                        // [pieces][heads][N]: A_c
 };
@@ -160,6 +163,16 @@ __global__ __launch_bounds__(256) void linear_recurrence_kernel(ScanArgs a) {
                 dk = to_float(a.k[row * a.k_stride + qk_head * N + i]);
                 dq = to_float(a.q[row * a.q_stride + qk_head * N + i]);
                 if (a.silu) { dk = silu_f(dk); dq = silu_f(dq); }
+                if (i < a.rot_dim) {
+                    const int half = a.rot_dim >> 1, j = i < half ? i : i - half, other = i < half ? i + half : i - half;
+                    const float* cs = a.rope + (size_t)a.positions[row] * a.rot_dim;
+                    float ok = to_float(a.k[row * a.k_stride + qk_head * N + other]);
+                    float oq = to_float(a.q[row * a.q_stride + qk_head * N + other]);
+                    if (a.silu) { ok = silu_f(ok); oq = silu_f(oq); }
+                    const float c = cs[j], s = cs[half + j];
+                    dk = i < half ? turn_x(dk, ok, c, s) : turn_y(ok, dk, c, s);
+                    dq = i < half ? turn_x(dq, oq, c, s) : turn_y(oq, dq, c, s);
+                }
                 dq *= a.q_scale;
             }
             a_lds[idx] = da; k_lds[idx] = dk; q_lds[idx] = dq;
@@ -709,14 +722,17 @@ int mlr_linear_recurrence(const void* q, long q_stride, const void* k, long k_st
                           long v_scale_stride, const float* skip, float q_scale, float* out, const float* live, float* stage,
                           long state_stride, const int32_t* seg_first, const int32_t* seg_count, const int32_t* slots,
                           int segments, int heads, int heads_per_group, int n_keys, int n_values, int write_state,
-                          float* piece_state, float* piece_decay, int silu, hipStream_t stream) {
+                          float* piece_state, float* piece_decay, int silu, const float* rope, const int32_t* positions,
+                          int rot_dim, hipStream_t stream) {
     // piece_state, piece_decay given: `seg_first`/`seg_count` name pieces of requests (a request's pieces one after
     // the other), run side by side in three passes; [segments][heads][n_keys][n_values] and [segments][heads][n_keys]
     if (segments <= 0) return 0;
     if (n_keys < 1 || n_keys > 256 || n_values < 1 || heads < 1 || heads_per_group < 1 || heads % heads_per_group) return -1;
+    if (rot_dim < 0 || rot_dim > n_keys || (rot_dim & 1) || (rot_dim > 0 && (rope == nullptr || positions == nullptr))) return -1;
     ScanArgs a{(const elem_t*)q, q_stride, (const elem_t*)k, k_stride, (const elem_t*)v, v_stride, log_decay, decay_stride,
                v_scale, v_scale_stride, skip, out, live, stage, state_stride, seg_first, seg_count, slots, heads,
-               heads_per_group, n_keys, n_values, decay_per_channel, write_state, q_scale, silu, piece_state, piece_decay};
+               heads_per_group, n_keys, n_values, decay_per_channel, write_state, q_scale, silu, rope, positions, rot_dim, piece_state,
+               piece_decay};
     if ((piece_state == nullptr) != (piece_decay == nullptr)) return -2;
     const int nr = (n_keys + SCAN_PARTS - 1) / SCAN_PARTS;
     if (nr <= 8) return launch_scan<8, 16>(a, segments, stream);

@@ -5,9 +5,10 @@
 //   MASK_ALL     lo = 0
 //   MASK_WINDOW  lo = max(0, p - size + 1)         (itself and the size - 1 tokens before it)
 //   MASK_CHUNK   lo = floor(p / size) * size        (the keys of its own block of `size` positions)
+// and besides (keep_first > 0) the request's first keep_first keys, as far as they lie at or before p;
 // positions counted from the request's first token, never from where a step cut it.  The softmax's denominator
 // holds one more summand, exp(sink[head]) (no key, no value, not scaled); sink == null: none.
-// score = (q . k) * scale.  Scores, the softmax and its sums are 32-bit.
+// score = (q . k) * scale, with a cap c tanh(score / c) (softcap 0: none).  Scores, the softmax and its sums are 32-bit.
 //
 // Cache of one layer: key rows k_pages[page][kv_head][place in page][k_row] of which the first key_dim channels
 // are the key, value rows v_pages[page][kv_head][place][v_row] of which the first value_dim channels are the
@@ -38,8 +39,8 @@ struct SinkArgs {
     const int32_t* block_table; const int32_t* slots; const int32_t* positions;
     const float* sink;                         // [q_heads] or null
     elem_t* out; long out_stride;              // out[m * out_stride + head * value_dim + c]
-    int max_blocks, q_heads, kv_heads, key_dim, value_dim, page_size, mask_kind, mask_size;
-    float scale;
+    int max_blocks, q_heads, kv_heads, key_dim, value_dim, page_size, mask_kind, mask_size, keep_first;
+    float scale, softcap;
     // key ranges over several workgroups (the matrix-core kernel): workgroup z of a group takes split_keys keys from
     // the group's first tile on and leaves (unnormalised values, maximum, sum) in partial[((g * tokens + i) * q_heads +
     // head) * splits + z][value_dim + 4] for token i of group g; null: one workgroup walks every key and writes out
@@ -62,17 +63,20 @@ __global__ __launch_bounds__(64) void sink_attention_kernel(SinkArgs a) {
     const int kvh = head / (a.q_heads / a.kv_heads);
     const int pos = a.positions[m], slot = a.slots[m];
     const int kbegin = first_seen(pos, a.mask_kind, a.mask_size), kend = pos + 1;
+    // the tiles below kept_end hold the first keys; those between them and the range's own first tile are passed over
+    const int range_tile = (kbegin / TILE_KEYS) * TILE_KEYS, kept_end = min(min(a.keep_first, kend), range_tile);
     for (int i = lane; i < D; i += 64) q_lds[i] = to_float(a.q[(size_t)m * a.q_stride + (size_t)head * D + i]);
     float run_max = -INFINITY, run_sum = 0.f, acc[MAX_V_REGS];
 #pragma unroll
     for (int i = 0; i < MAX_V_REGS; ++i) acc[i] = 0.f;
     const int32_t* table = a.block_table + (size_t)slot * a.max_blocks;
-    for (int t0 = (kbegin / TILE_KEYS) * TILE_KEYS; t0 < kend; t0 += TILE_KEYS) {
+    for (int t0 = kept_end > 0 ? 0 : range_tile; t0 < kend; t0 += TILE_KEYS) {
+        if (t0 >= kept_end && t0 < range_tile) t0 = range_tile;
         __syncthreads();
         {
             const int kp = t0 + lane;
             long long r = -1;
-            if (kp >= kbegin && kp < kend) {
+            if ((kp >= kbegin || kp < a.keep_first) && kp < kend) {
                 const int block = kp / a.page_size;
                 const int page = block < a.max_blocks ? table[block] : -1;
                 if (page >= 0) r = ((long long)page * a.kv_heads + kvh) * a.page_size + kp % a.page_size;
@@ -95,7 +99,9 @@ __global__ __launch_bounds__(64) void sink_attention_kernel(SinkArgs a) {
             s += part;
         }
         const bool valid = row_of[lane] >= 0;
-        s = valid ? s * a.scale : -INFINITY;
+        s *= a.scale;
+        if (a.softcap > 0.f) s = a.softcap * tanhf(s / a.softcap);
+        if (!valid) s = -INFINITY;
         const float new_max = fmaxf(run_max, wave_max(s));
         const float p = (valid && new_max > -INFINITY) ? expf(s - new_max) : 0.f;
         const float corr = new_max > -INFINITY ? expf(run_max - new_max) : 1.f;
@@ -418,7 +424,8 @@ __global__ __launch_bounds__(64) void latent_prep_kernel(
 //
 // A workgroup (4 wavefronts) serves ONE group of consecutive tokens of a request and up to `head_block` query heads
 // of one kv head: 64 columns (token, head), token = column / head_block.  It walks the keys that its tokens see,
-// from the first key of the group's first token to the last token's own position, in tiles of 32 keys at absolute
+// from the first key of the group's first token to the last token's own position, before them the tiles of the
+// request's first keys where a mask keeps those (what lies between is passed over), in tiles of 32 keys at absolute
 // multiples of 32; a tile's key rows are staged once through LDS for all its columns (row-major for the scores,
 // and the value channels transposed, [channel][key], for the second product: 16-byte reads of eight keys of one
 // channel), the next tile's rows on their way from memory into registers meanwhile.  A thread stages 16 bytes (eight
@@ -458,11 +465,16 @@ __global__ __launch_bounds__(256) void sink_attention_tiles_kernel(SinkArgs a, c
     const int D = a.key_dim, V = a.value_dim;
     const bool shared_rows = a.v_pages == a.k_pages;
     const int p0 = a.positions[first], slot = a.slots[first];
-    int kbegin = first_seen(p0, a.mask_kind, a.mask_size), kend = p0 + count;
-    if (a.partial != nullptr) {                // this workgroup's share of the keys, from the group's first tile on
-        const int base = (kbegin / TK) * TK + (int)blockIdx.z * a.split_keys;
-        kbegin = max(kbegin, base);
-        kend = min(kend, base + a.split_keys);
+    const int kbegin = first_seen(p0, a.mask_kind, a.mask_size), kend = p0 + count;
+    // The group's tiles are counted without those between the kept first keys and the range: number i lies at tile i below
+    // `kept`, at tile i + gap from there on (kept = 0 where nothing lies between).
+    int kept = (min(a.keep_first, kend) + TK - 1) / TK;
+    const int gap = max(0, kbegin / TK - kept);
+    if (gap == 0) kept = 0;
+    int i_first = 0, i_end = (kend + TK - 1) / TK - gap;
+    if (a.partial != nullptr) {                // this workgroup's share of them
+        i_first = (int)blockIdx.z * (a.split_keys / TK);
+        i_end = min(i_end, i_first + a.split_keys / TK);
     }
     const int32_t* table = a.block_table + (size_t)slot * a.max_blocks;
 
@@ -487,11 +499,22 @@ __global__ __launch_bounds__(256) void sink_attention_tiles_kernel(SinkArgs a, c
     for (int j = 0; j < NACC; ++j) acc[j] = floatx4{0.f, 0.f, 0.f, 0.f};
     float run_max = -INFINITY, run_sum = 0.f;
     const float scale2 = a.scale * 1.4426950408889634f;
+    const bool capped = a.softcap > 0.f;
+    const float cap2 = a.softcap * 1.4426950408889634f, cap_slope = capped ? 2.0f * scale2 / a.softcap : 0.f;
 
-    // the page ids of the workgroup's key range, once
-    const int block0 = kbegin / a.page_size;
-    const int n_blocks = kend > kbegin ? min((kend - 1) / a.page_size - block0 + 1, TILES_MAX_BLOCKS) : 0;
-    for (int i = tid; i < n_blocks; i += 256) page_lds[i] = block0 + i < a.max_blocks ? table[block0 + i] : -1;
+    // the page ids of the workgroup's keys, once: those of its kept tiles, behind them those of its others
+    const int lead_end = min(i_end, kept) * TK;                                   // its kept keys end here
+    const int lead0 = (i_first * TK) / a.page_size;
+    const int n_lead = lead_end > i_first * TK ? (lead_end - 1) / a.page_size - lead0 + 1 : 0;
+    const int main_first = max((max(i_first, kept) + gap) * TK, a.keep_first > 0 ? 0 : kbegin);
+    const int main_end = min(kend, (i_end + gap) * TK);
+    const int block0 = main_first / a.page_size;
+    const int n_main = main_end > main_first ? (main_end - 1) / a.page_size - block0 + 1 : 0;
+    const int n_blocks = min(n_lead + n_main, TILES_MAX_BLOCKS);
+    for (int i = tid; i < n_blocks; i += 256) {
+        const int blk = i < n_lead ? lead0 + i : block0 + i - n_lead;
+        page_lds[i] = blk < a.max_blocks ? table[blk] : -1;
+    }
     __syncthreads();
 
     // A thread stages the same key of every tile (key = thread % 32: 256 is a multiple of it) and the chunks
@@ -501,9 +524,10 @@ __global__ __launch_bounds__(256) void sink_attention_tiles_kernel(SinkArgs a, c
     const int my_key = tid & 31, my_chunk = tid >> 5;
     auto fetch = [&](int t0, bf16x8 (&kreg)[NSK], bf16x8 (&vreg)[NSV]) {
         const int kp = t0 + my_key;
-        const bool inside = kp >= kbegin && kp < kend;
-        const int blk = inside ? kp / a.page_size - block0 : 0;
-        const int page = (inside && blk < n_blocks) ? page_lds[blk] : -1;
+        const bool lead = t0 < lead_end;
+        const bool inside = (kp >= kbegin || kp < a.keep_first) && kp < (lead ? lead_end : main_end);
+        const int rel = inside ? kp / a.page_size - (lead ? lead0 : block0) : -1, blk = lead ? rel : n_lead + rel;
+        const int page = (rel >= 0 && blk < n_blocks) ? page_lds[blk] : -1;
         const bool have = page >= 0;
         const long long r = have ? ((long long)page * a.kv_heads + kvh) * a.page_size + kp % a.page_size : 0;
         const __bf16* krow = a.k_pages + r * a.k_row;
@@ -574,13 +598,16 @@ __global__ __launch_bounds__(256) void sink_attention_tiles_kernel(SinkArgs a, c
         float sc[8];
         float tile_max = -INFINITY;
         // a tile that every token of the group sees whole needs no comparisons (the same in every thread)
-        const bool whole = t0 >= last_lo && t0 + TK - 1 <= p0;
+        const bool whole = (t0 >= last_lo || t0 + TK <= a.keep_first) && t0 + TK - 1 <= p0;
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
             const int kp = t0 + 8 * b + e;
             const float raw = e < 4 ? s0[e] : s1[e - 4];
-            const bool seen = col_ok && (whole || (kp >= qlo && kp <= qpos));
-            sc[e] = seen ? raw * scale2 : -INFINITY;
+            const bool seen = col_ok && (whole || ((kp >= qlo || kp < a.keep_first) && kp <= qpos));
+            // (capped: c tanh(s / c) = c - 2 c / (1 + e^(2 s / c)), here in base 2; an exponent beyond 32 bits gives c)
+            const float s2 = capped ? cap2 - 2.0f * cap2 * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(raw * cap_slope))
+                                    : raw * scale2;
+            sc[e] = seen ? s2 : -INFINITY;
             tile_max = fmaxf(tile_max, sc[e]);
         }
         tile_max = fmaxf(tile_max, __shfl_xor(tile_max, 16, MLR_WAVE));
@@ -615,13 +642,13 @@ __global__ __launch_bounds__(256) void sink_attention_tiles_kernel(SinkArgs a, c
     // The next tile's rows are asked for before this tile's products, unconditionally (beyond the range the rows come
     // out as zeros): a load behind a branch would make the loop wait for it where the branches join, before the
     // products it is meant to hide behind.
-    const int t_first = (kbegin / TK) * TK;
-    fetch(t_first, kreg_a, vreg_a);
-    for (int t0 = t_first; t0 < kend; t0 += TK) {
+    const auto tile_at = [&](int i) { return (i < kept ? i : i + gap) * TK; };
+    fetch(tile_at(i_first), kreg_a, vreg_a);
+    for (int i = i_first; i < i_end; ++i) {
         stage(kreg_a, vreg_a);
         __syncthreads();
-        fetch(t0 + TK, kreg_a, vreg_a);
-        tile(t0);
+        fetch(tile_at(i + 1), kreg_a, vreg_a);
+        tile(tile_at(i));
         __syncthreads();
     }
     if (a.partial != nullptr) {                // this range's share: the merge kernel finishes the column
@@ -723,14 +750,15 @@ extern "C" {
 int mlr_sink_attention(const void* q, long q_stride, const void* k_pages, long k_row, const void* v_pages, long v_row,
                        const int32_t* block_table, int max_blocks, const int32_t* slots, const int32_t* positions,
                        const float* sink, void* out, long out_stride, int rows, int q_heads, int kv_heads, int key_dim,
-                       int value_dim, int page_size, int mask_kind, int mask_size, float scale, hipStream_t stream) {
+                       int value_dim, int page_size, int mask_kind, int mask_size, int keep_first, float softcap, float scale,
+                       hipStream_t stream) {
     if (rows <= 0) return 0;
     if (key_dim > MAX_KEY_DIM || value_dim > 64 * MAX_V_REGS || q_heads > 65535 || kv_heads <= 0 ||
-        q_heads % kv_heads != 0 || (mask_kind != MASK_ALL && mask_size <= 0))
+        q_heads % kv_heads != 0 || (mask_kind != MASK_ALL && mask_size <= 0) || keep_first < 0 || !(softcap >= 0.f))
         return -1;
     SinkArgs a{(const elem_t*)q, q_stride, (const elem_t*)k_pages, k_row, (const elem_t*)v_pages, v_row, block_table,
                slots, positions, sink, (elem_t*)out, out_stride, max_blocks, q_heads, kv_heads, key_dim, value_dim,
-               page_size, mask_kind, mask_size, scale, nullptr, 0, 1, 1};
+               page_size, mask_kind, mask_size, keep_first, scale, softcap, nullptr, 0, 1, 1};
     sink_attention_kernel<<<dim3(rows, q_heads), 64, 0, stream>>>(a);
     return (int)hipGetLastError();
 }
@@ -799,26 +827,26 @@ int mlr_sink_attention_tiles(const void* q, long q_stride, const void* k_pages, 
                              const int32_t* positions, const float* sink, void* out, long out_stride,
                              const int32_t* group_first, const int32_t* group_count, int groups, int head_block,
                              int split_values, int q_heads, int kv_heads, int key_dim, int value_dim, int page_size,
-                             int mask_kind, int mask_size, int max_context, float scale, float* partial, int split_keys,
-                             int splits, hipStream_t stream) {
+                             int mask_kind, int mask_size, int keep_first, float softcap, int max_context, float scale,
+                             float* partial, int split_keys, int splits, hipStream_t stream) {
 #if MLR_BF16
     if (groups <= 0) return 0;
     {
         // the keys that one workgroup may have to walk: its page ids must fit what it keeps of them
-        const long reach = mask_kind == MASK_ALL ? (long)max_context : (long)mask_size + 64;
-        if (reach / page_size + 2 > TILES_MAX_BLOCKS) return 1;
+        const long reach = mask_kind == MASK_ALL ? (long)max_context : (long)mask_size + 64 + (keep_first > 0 ? keep_first + 96 : 0);
+        if (reach / page_size + (keep_first > 0 ? 4 : 2) > TILES_MAX_BLOCKS) return 1;
     }
     if (key_dim % 8 != 0 || value_dim % 16 != 0 || key_dim > 576 || value_dim > 512 || k_row % 8 != 0 || v_row % 8 != 0 ||
         q_stride % 8 != 0 || out_stride % 4 != 0 || kv_heads <= 0 || q_heads % kv_heads != 0)
         return 1;
     if (head_block < 1 || head_block > (split_values ? 16 : 64) || (head_block & (head_block - 1)) != 0 ||
-        (mask_kind != MASK_ALL && mask_size <= 0))
+        (mask_kind != MASK_ALL && mask_size <= 0) || keep_first < 0 || !(softcap >= 0.f))
         return -1;
     const int hg = q_heads / kv_heads, head_blocks = (hg + head_block - 1) / head_block;
     if ((long)kv_heads * head_blocks > 65535) return -2;
     SinkArgs a{(const elem_t*)q, q_stride, (const elem_t*)k_pages, k_row, (const elem_t*)v_pages, v_row, block_table,
                slots, positions, sink, (elem_t*)out, out_stride, max_blocks, q_heads, kv_heads, key_dim, value_dim,
-               page_size, mask_kind, mask_size, scale, splits > 1 ? partial : nullptr, split_keys, splits > 1 ? splits : 1,
+               page_size, mask_kind, mask_size, keep_first, scale, softcap, splits > 1 ? partial : nullptr, split_keys, splits > 1 ? splits : 1,
                (split_values ? 16 : 64) / head_block};
     if (splits > 1 && (partial == nullptr || split_keys <= 0 || split_keys % TK != 0 || splits > 65535 || a.group_tokens > 65535))
         return -1;

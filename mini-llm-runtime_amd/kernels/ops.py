@@ -103,7 +103,7 @@ def _residual_work(self, a, w, h, *rest, **kw):
     return _size(a) + _size(w) + 2 * _size(h), 2 * a.shape[0] * w.shape[0] * w.shape[1]
 
 
-def _norm_work(self, h, delta, weight, out, eps, rows=None, write_h=True):
+def _norm_work(self, h, delta, weight, out, eps, rows=None, write_h=True, factor=1.0, vector=None):
     n, width = out.shape[0], h.shape[1]
     moved = n * width * 4 + _size(out)
     if delta is not None:
@@ -169,9 +169,9 @@ class Kernels:
             "embed_gather")
 
     @timed("norm", _norm_work)
-    def add_rmsnorm(self, h, delta, weight, out, eps, rows=None, write_h=True):
-        """x = h[src] + delta[src] (delta may be None); h[src] = x when write_h; out[r] =
-        rmsnorm(x) * weight, src = rows[r] or r."""
+    def add_rmsnorm(self, h, delta, weight, out, eps, rows=None, write_h=True, factor=1.0, vector=None):
+        """x = h[src] + factor * delta[src] + vector (delta and the float vector [width] may be None); h[src] = x when
+        write_h; out[r] = rmsnorm(x) * weight, src = rows[r] or r."""
         _tensor(h, "h", torch.float32, ndim=2)
         m, width = h.shape
         if delta is not None:
@@ -182,10 +182,13 @@ class Kernels:
             n_out = rows.numel()
         else:
             n_out = m
+        if vector is not None:
+            _tensor(vector, "vector", torch.float32, (width,))
         _tensor(out, "out", self.dtype, (n_out, width))
         fn = self._lib("elementwise").mlr_add_rmsnorm
-        _ok(fn(_p(h), _p(delta), _p(weight), _p(out), _p(rows), _c_int(n_out), _c_int(width),
-               _c_float(eps), _c_int(1 if (write_h and delta is not None) else 0), _stream()),
+        changes = delta is not None or vector is not None
+        _ok(fn(_p(h), _p(delta), _c_float(factor), _p(vector), _p(weight), _p(out), _p(rows), _c_int(n_out), _c_int(width),
+               _c_float(eps), _c_int(1 if (write_h and changes) else 0), _stream()),
             "add_rmsnorm")
 
     @timed("check")
@@ -195,8 +198,8 @@ class Kernels:
         _ok(self._lib("elementwise").mlr_status_reset(_p(status), _stream()), "status_reset")
 
     @timed("check")
-    def finite_check(self, h, delta, layer, status):
-        """ORs into status[0] which kinds of non-finite values h + delta holds (1: NaN, 2: infinity) and keeps
+    def finite_check(self, h, delta, layer, status, factor=1.0):
+        """ORs into status[0] which kinds of non-finite values h + factor * delta holds (1: NaN, 2: infinity) and keeps
         in status[1] the smallest (layer << 20 | row) that held one."""
         _tensor(h, "h", torch.float32, ndim=2)
         m, width = h.shape
@@ -204,15 +207,19 @@ class Kernels:
             _tensor(delta, "delta", self.dtype, (m, width))
         _tensor(status, "status", torch.int32, (2,))
         _need(0 <= layer < 2047, "finite_check: layer index out of range")
-        _ok(self._lib("elementwise").mlr_finite_check(_p(h), _p(delta), _c_int(m), _c_int(width), _c_int(layer),
-                                                      _p(status), _stream()), "finite_check")
+        _ok(self._lib("elementwise").mlr_finite_check(_p(h), _p(delta), _c_float(factor), _c_int(m), _c_int(width),
+                                                      _c_int(layer), _p(status), _stream()), "finite_check")
 
     @timed("norm", _tensors_work())
-    def residual_add(self, h, delta):
+    def residual_add(self, h, delta, factor=1.0, vector=None):
+        """h += factor * delta + vector (delta, or a float vector [width], may be None)."""
         _tensor(h, "h", torch.float32, ndim=2)
-        _tensor(delta, "delta", self.dtype, tuple(h.shape))
+        if delta is not None:
+            _tensor(delta, "delta", self.dtype, tuple(h.shape))
+        if vector is not None:
+            _tensor(vector, "vector", torch.float32, (h.shape[1],))
         fn = self._lib("elementwise").mlr_residual_add
-        _ok(fn(_p(h), _p(delta), _c_size_t(h.numel()), _stream()), "residual_add")
+        _ok(fn(_p(h), _p(delta), _c_float(factor), _p(vector), _c_int(h.shape[1]), _c_size_t(h.numel()), _stream()), "residual_add")
 
     @timed("norm", _tensors_work())
     def residual_add_float(self, h, extra):
@@ -232,12 +239,12 @@ class Kernels:
         fn = self._lib("elementwise").mlr_silu_mul
         _ok(fn(_p(gate_up), _p(act), _c_int(m), _c_int(two_f // 2), _stream()), "silu_mul")
 
-    GATED_ACTS = {"silu": 0, "gelu_tanh": 1}
+    GATED_ACTS = {"silu": 0, "gelu_tanh": 1, "relu": 2}
 
     @timed("activation", _tensors_work())
     def gated_act_mul(self, gate_up, act, kind):
-        """act[m, f] = kind(gate_up[m, f]) * gate_up[m, F + f]; kind: silu, or gelu_tanh,
-        0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3)))."""
+        """act[m, f] = kind(gate_up[m, f]) * gate_up[m, F + f]; kind: silu, gelu_tanh,
+        0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3))), or relu."""
         _need(kind in self.GATED_ACTS, f"gated_act_mul: activation {kind!r} ({', '.join(self.GATED_ACTS)})")
         _tensor(gate_up, "gate_up", self.dtype, ndim=2)
         m, two_f = gate_up.shape
@@ -298,6 +305,20 @@ class Kernels:
         _tensor(out, "out", self.dtype, tuple(a.shape))
         _ok(self._lib("elementwise").mlr_scaled_sum(_p(a), _p(b), _p(out), _c_float(sa), _c_float(sb), _c_size_t(a.numel()),
                                                     _stream()), "scaled_sum")
+
+    @timed("norm", _tensors_work())
+    def normed_sum(self, a, b, wa, wb, out, sa, sb, eps):
+        """out = sa * norm(a) + sb * norm(b), norm(x) = x / sqrt(mean(x^2) + eps) * weight row by row (a weight of None: the
+        row as it is), the sum taken in 32-bit; out may be a or b."""
+        _tensor(a, "a", self.dtype, ndim=2)
+        rows, width = a.shape
+        _tensor(b, "b", self.dtype, (rows, width))
+        _tensor(out, "out", self.dtype, (rows, width))
+        for name, w in (("wa", wa), ("wb", wb)):
+            if w is not None:
+                _tensor(w, name, torch.float32, (width,))
+        _ok(self._lib("elementwise").mlr_normed_sum(_p(a), _p(b), _p(wa), _p(wb), _p(out), _c_float(sa), _c_float(sb),
+                                                    _c_int(rows), _c_int(width), _c_float(eps), _stream()), "normed_sum")
 
     # -- projections -------------------------------------------------------------------------
     @timed("gemm", _gemm_work)
@@ -388,18 +409,19 @@ class Kernels:
             "gemm_gated_clamped")
 
     @timed("gemm", _gemm_work)
-    def gemm_gated_gelu_tanh(self, a, w, out):
-        """out[M, N] = gelu_tanh(a . w[:N]^T) * (a . w[N:]^T), w = [gate; up] stacked: the tanh form of gelu fused into
-        the weight-streaming projection, up to 64 rows (bfloat16)."""
-        _need(self.dtype == torch.bfloat16 and a.shape[0] <= 64, "gemm_gated_gelu_tanh: bfloat16, up to 64 rows")
+    def gemm_gated_act(self, a, w, out, kind):
+        """out[M, N] = kind(a . w[:N]^T) * (a . w[N:]^T), w = [gate; up] stacked: the gate (gelu_tanh or relu, as
+        `gated_act_mul`'s) fused into the weight-streaming projection, up to 64 rows (bfloat16)."""
+        _need(kind in ("gelu_tanh", "relu"), f"gemm_gated_act: activation {kind!r}")
+        _need(self.dtype == torch.bfloat16 and a.shape[0] <= 64, "gemm_gated_act: bfloat16, up to 64 rows")
         _tensor(a, "a", self.dtype, ndim=2)
         _tensor(w, "w", self.dtype, ndim=2)
         m, k = a.shape
         two_n, k2 = w.shape
-        _need(k == k2 and two_n % 2 == 0, "gemm_gated_gelu_tanh: sizes do not fit")
+        _need(k == k2 and two_n % 2 == 0, "gemm_gated_act: sizes do not fit")
         _tensor(out, "out", self.dtype, (m, two_n // 2))
-        _ok(self._lib("gemm").mlr_gemm_gated_gelu_tanh(_p(a), _p(w), _p(out), _c_int(m), _c_int(two_n // 2), _c_int(k),
-                                                       _stream()), "gemm_gated_gelu_tanh")
+        _ok(self._lib("gemm").mlr_gemm_gated_act(_p(a), _p(w), _p(out), _c_int(m), _c_int(two_n // 2), _c_int(k),
+                                                 _c_int(self.GATED_ACTS[kind]), _stream()), "gemm_gated_act")
 
     @timed("gemm", _gemm_work)
     def gemm_act(self, a, w, out, kind):
@@ -826,13 +848,15 @@ class Kernels:
     @timed("norm", _tensors_work())
     def gated_part_norm(self, y, gate, weight, out, part, eps, gate_first, gate_kind="silu"):
         """y float [rows, width] in parts of `part` values, each over its root mean square, times
-        weight[i % len(weight)]; the activation of `gate` (columns of a matrix) multiplies before the norm
+        weight[i % len(weight)] (None: no weight); the activation of `gate` (columns of a matrix) multiplies before the norm
         (`gate_first`) or after it."""
         _tensor(y, "y", torch.float32, ndim=2)
         m, width = y.shape
         stride = self._columns(gate, "gate", self.dtype, m, width)
-        _tensor(weight, "weight", torch.float32, ndim=1)
-        period = weight.numel()
+        period = part
+        if weight is not None:
+            _tensor(weight, "weight", torch.float32, ndim=1)
+            period = weight.numel()
         _need(part >= 1 and width % part == 0 and period in (part, width), "gated_part_norm: sizes do not fit")
         _need(gate_kind in ("silu", "sigmoid"), "gated_part_norm: unknown gate")
         _tensor(out, "out", self.dtype, (m, width))
@@ -903,7 +927,7 @@ class Kernels:
     @timed("recurrence", _tensors_work())
     def linear_recurrence(self, q, k, v, log_decay, out, live, stage, state_offset, seg_first, seg_count, segments, slots,
                           heads, n_keys, n_values, heads_per_group=1, v_scale=None, skip=None, q_scale=1.0,
-                          write_state=True, piece_state=None, piece_decay=None, activation=None):
+                          write_state=True, piece_state=None, piece_decay=None, activation=None, rope=None, positions=None):
         """Per request of the step and head, from the live state: S_t = diag(exp(log_decay_t)) S_(t-1) + k_t (v_scale_t
         v_t)^T, out_t = S_t^T (q_scale q_t) + skip[head] v_t.  q, k: columns [rows, (heads / heads_per_group) * n_keys];
         v: columns [rows, heads * n_values]; log_decay float [rows, heads * n_keys] (a decay per key channel) or
@@ -912,8 +936,11 @@ class Kernels:
         With `piece_state` float [segments * heads * n_keys * n_values] and `piece_decay` float [segments * heads *
         n_keys]: `seg_first`/`seg_count` name PIECES of requests (a request's pieces one after the other), which run
         side by side in three passes; the result differs from the token-by-token order by 32-bit rounding.
-        log_decay float [heads]: one constant decay a head.  `activation` "silu": q, k and v pass it as they are read."""
+        log_decay float [heads]: one constant decay a head.  `activation` "silu": q, k and v pass it as they are read.
+        `rope` (float [positions, rot]: cosines | sines) with `positions` int32 [rows]: the first rot channels of every
+        head of q and k are turned as they are read, in pairs (i, i + rot / 2), in 32-bit."""
         rows = v.shape[0]
+        rot = self._turn_table(rope, positions, rows, n_keys)
         groups = heads // heads_per_group
         _need(heads >= 1 and heads_per_group >= 1 and heads % heads_per_group == 0, "linear_recurrence: heads and groups")
         _need(1 <= n_keys <= self.RECURRENCE_MAX_KEYS, f"linear_recurrence: 1..{self.RECURRENCE_MAX_KEYS} key channels a head")
@@ -956,7 +983,18 @@ class Kernels:
                _ptr(live.data_ptr() + at), _ptr(stage.data_ptr() + at), ctypes.c_long(live.stride(0)), _p(seg_first),
                _p(seg_count), _p(slots), _c_int(segments), _c_int(heads), _c_int(heads_per_group), _c_int(n_keys),
                _c_int(n_values), _c_int(1 if write_state else 0), _p(piece_state), _p(piece_decay),
-               _c_int(1 if activation == "silu" else 0), _stream()), "linear_recurrence")
+               _c_int(1 if activation == "silu" else 0), _p(rope), _p(positions if rope is not None else None), _c_int(rot),
+               _stream()), "linear_recurrence")
+
+    def _turn_table(self, rope, positions, rows, n_keys):
+        """The width of a rotation table for heads of `n_keys` channels (0: none given), checked with the positions."""
+        if rope is None:
+            return 0
+        _tensor(rope, "rope", torch.float32, ndim=2)
+        rot = rope.shape[1]
+        _need(2 <= rot <= n_keys and rot % 2 == 0, f"rope: the table's width {rot} must be even and at most {n_keys}")
+        _tensor(positions, "positions", torch.int32, (rows,))
+        return rot
 
     @timed("activation", _tensors_work())
     def channel_log_decay(self, z, bias, a_log, out, heads, n_keys):
@@ -1463,10 +1501,11 @@ class Kernels:
 
     @timed("attention")
     def sink_attention(self, q, k_pages, v_pages, block_table, slots, positions, sink, out, q_heads, kv_heads, key_dim,
-                       value_dim, page_size, scale, mask=None, mask_size=0):
+                       value_dim, page_size, scale, mask=None, mask_size=0, keep_first=0, softcap=None):
         """out[m, h] = softmax (with one more summand exp(sink[h]) in the denominator; sink None: none) over the keys
         that token m sees of q.k * scale, times v.  mask: None/"all" (positions <= its own), "window" (the last
-        mask_size positions), "chunk" (its own block of mask_size positions).  Keys are the first key_dim channels of
+        mask_size positions), "chunk" (its own block of mask_size positions); with either the request's first `keep_first`
+        positions besides.  `softcap`: a score s becomes softcap tanh(s / softcap).  Keys are the first key_dim channels of
         k_pages' rows, values the first value_dim of v_pages' rows (which may be the same tensor)."""
         _tensor(q, "q", self.dtype, ndim=2)
         rows = q.shape[0]
@@ -1489,20 +1528,33 @@ class Kernels:
             _p(q), ctypes.c_long(q.shape[1]), _p(k_pages), ctypes.c_long(k_row), _p(v_pages), ctypes.c_long(v_row),
             _p(block_table), _c_int(block_table.shape[1]), _p(slots), _p(positions), _p(sink), _p(out),
             ctypes.c_long(out.shape[1]), _c_int(rows), _c_int(q_heads), _c_int(kv_heads), _c_int(key_dim),
-            _c_int(value_dim), _c_int(page_size), _c_int(kind), _c_int(int(mask_size)), _c_float(scale), _stream()),
-            "sink_attention")
+            _c_int(value_dim), _c_int(page_size), _c_int(kind), _c_int(int(mask_size)), _c_int(self._kept(kind, keep_first)),
+            _c_float(self._cap(softcap)), _c_float(scale), _stream()), "sink_attention")
+
+    @staticmethod
+    def _kept(kind, keep_first):
+        _need(keep_first >= 0, "keep_first cannot be negative")
+        return int(keep_first) if kind != 0 else 0        # (without a mask every key is seen anyway)
+
+    @staticmethod
+    def _cap(softcap):
+        _need(softcap is None or softcap > 0, "softcap must be positive")
+        return 0.0 if softcap is None else float(softcap)
 
     SINK_TILES_BLOCKS = 2048
 
-    def sink_tiles_supported(self, key_dim, value_dim, k_row, v_row, page_size=16, mask=None, mask_size=0, max_context=0):
+    def sink_tiles_supported(self, key_dim, value_dim, k_row, v_row, page_size=16, mask=None, mask_size=0, max_context=0,
+                             keep_first=0):
         """Whether the matrix-core kernel takes these sizes: the bfloat16 engine, keys in multiples of 8 channels up to
         576, values in multiples of 16 up to 512, cache rows that start at multiples of 16 bytes, and a key range of
         one workgroup (the window or chunk and its tokens; without a mask the step's longest context) whose page ids
         fit what the kernel keeps of them."""
-        reach = max_context if self.SINK_MASKS.get(mask, 0) == 0 else mask_size + 64
+        whole = self.SINK_MASKS.get(mask, 0) == 0
+        kept = not whole and keep_first > 0
+        reach = max_context if whole else mask_size + 64 + (keep_first + 96 if kept else 0)
         return (self.dtype == torch.bfloat16 and key_dim % 8 == 0 and value_dim % 16 == 0 and key_dim <= 576
                 and value_dim <= 512 and k_row % 8 == 0 and v_row % 8 == 0
-                and reach // page_size + 2 <= self.SINK_TILES_BLOCKS)
+                and reach // page_size + (4 if kept else 2) <= self.SINK_TILES_BLOCKS)
 
     @staticmethod
     def sink_tiles_layout(q_heads, kv_heads):
@@ -1518,7 +1570,8 @@ class Kernels:
     @timed("attention")
     def sink_attention_tiles(self, q, k_pages, v_pages, block_table, slots, positions, sink, out, group_first, group_count,
                              groups, head_block, split_values, q_heads, kv_heads, key_dim, value_dim, page_size, scale,
-                             mask=None, mask_size=0, max_context=0, partial=None, split_keys=0, splits=1):
+                             mask=None, mask_size=0, max_context=0, partial=None, split_keys=0, splits=1, keep_first=0,
+                             softcap=None):
         """`sink_attention` on the matrix cores for `groups` groups of consecutive tokens of one request each (device
         vectors group_first, group_count), at most 64 / head_block tokens a group (16 / head_block with
         `split_values`).  splits > 1: a group's keys in that many ranges of `split_keys` keys (a multiple of 32), one
@@ -1529,7 +1582,7 @@ class Kernels:
         k_row = self._sink_pages(k_pages, "k_pages", kv_heads, page_size, key_dim)
         v_row = self._sink_pages(v_pages, "v_pages", kv_heads, page_size, value_dim)
         _need(mask in self.SINK_MASKS, f"mask {mask!r}: one of all, window, chunk")
-        _need(self.sink_tiles_supported(key_dim, value_dim, k_row, v_row, page_size, mask, mask_size, max_context)
+        _need(self.sink_tiles_supported(key_dim, value_dim, k_row, v_row, page_size, mask, mask_size, max_context, keep_first)
               and q.shape[1] % 8 == 0, "sink_attention_tiles: sizes that the matrix-core kernel does not take")
         kind = self.SINK_MASKS[mask]
         _need(kind == 0 or mask_size >= 1, "a window or chunk needs a positive size")
@@ -1553,7 +1606,8 @@ class Kernels:
             _p(block_table), _c_int(block_table.shape[1]), _p(slots), _p(positions), _p(sink), _p(out),
             ctypes.c_long(out.shape[1]), _p(group_first), _p(group_count), _c_int(groups), _c_int(head_block),
             _c_int(1 if split_values else 0), _c_int(q_heads), _c_int(kv_heads), _c_int(key_dim), _c_int(value_dim),
-            _c_int(page_size), _c_int(kind), _c_int(int(mask_size)), _c_int(int(max_context)), _c_float(scale),
+            _c_int(page_size), _c_int(kind), _c_int(int(mask_size)), _c_int(self._kept(kind, keep_first)),
+            _c_float(self._cap(softcap)), _c_int(int(max_context)), _c_float(scale),
             _p(partial if splits > 1 else None), _c_int(int(split_keys)), _c_int(int(splits)), _stream())
         _ok(code, "sink_attention_tiles")
 
@@ -1768,9 +1822,9 @@ class Kernels:
                                                      _p(offsets), _p(token_of), _p(row_of), _stream()), "route_sort")
 
     @timed("activation", _tensors_work())
-    def route_combine(self, y, row_of, weights, out, shared=None, shared_gate=None):
-        """out[m] = sum_i weights[m, i] * y[row_of[m * top + i]] (32-bit sums, in the order of the choices), plus
-        shared[m], which `shared_gate` (a float column [rows, 1] of a row-major matrix) multiplies by its sigmoid."""
+    def route_combine(self, y, row_of, weights, out, shared=None, shared_gate=None, ids=None, experts=0, x=None):
+        """out[m] = sum_i weights[m, i] * y[row_of[m * top + i]] (32-bit sums, in the order of the choices; with `ids`
+        [rows, top] a choice >= `experts` takes x[m] instead: an expert that gives its input back), plus shared[m], which `shared_gate` (a float column [rows, 1] of a row-major matrix) multiplies by its sigmoid."""
         _tensor(weights, "weights", torch.float32, ndim=2)
         rows, top = weights.shape
         _tensor(y, "y", self.dtype, ndim=2)
@@ -1780,10 +1834,14 @@ class Kernels:
         _need(shared is not None or shared_gate is None, "route_combine: a gate without what it gates")
         if shared is not None:
             _tensor(shared, "shared", self.dtype, (rows, y.shape[1]))
+        _need((ids is None) == (x is None), "route_combine: ids and x go together")
+        if ids is not None:
+            _tensor(ids, "ids", torch.int32, (rows, top))
+            _tensor(x, "x", self.dtype, (rows, y.shape[1]))
         gate_stride = self._columns(shared_gate, "shared_gate", torch.float32, rows, 1) if shared_gate is not None else 0
         _ok(self._lib("grouped_gemm").mlr_route_combine(
             _p(y), _p(row_of), _p(weights), _p(out), _c_int(rows), _c_int(y.shape[1]), _c_int(top), _p(shared),
-            _p(shared_gate), ctypes.c_long(gate_stride), _stream()), "route_combine")
+            _p(shared_gate), ctypes.c_long(gate_stride), _p(ids), _c_int(experts), _p(x), _stream()), "route_combine")
 
     # -- sampling ----------------------------------------------------------------------------
     def sample_scratch(self, rows):

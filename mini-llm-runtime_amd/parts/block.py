@@ -1,20 +1,24 @@
 """Arrangement of the parts in a layer.  Pre-norm residual block (src/minillm/runtime.cpp:245-337):
 h += mixer(norm1(h)); h += ffn(norm2(h)).  The residual stream h is float; every add into it is
 fused with the norm that follows, so a block hands its last output on as `pending` instead of
-adding it itself.  `norm2` and `ffn` may be missing: a layer of the first sublayer only.
+adding it itself.  `norm2` and `ffn` may be missing: a layer of the first sublayer only.  With a `residual_scale` m
+h += m * mixer(norm1(h)); h += m * ffn(norm2(h)): the factor rides in the pass that adds.
 Other arrangements: mixer and feed-forward side by side (`parallel`), norms behind the sublayers (`postnorm`), norms in
 front of AND behind each sublayer (`sandwich`)."""
 from __future__ import annotations
 
-from .registry import Complete, Handoff, build_part, register_part
+from .registry import Addend, Complete, Handoff, addend_for, build_part, register_part
 
 
 @register_part("block", "prenorm")
 class PreNormBlock:
     graph_safe = True        # forward launches kernels over the step's device vectors only
+    takes_addend = True
+
     def __init__(self, spec):
         self.norm1 = build_part("norm", spec.norm1)
         self.mixer = build_part("mixer", spec.mixer)
+        self.scale = float(getattr(spec, "residual_scale", 1.0))
         if (spec.ffn is None) != (spec.norm2 is None):
             raise ValueError("a pre-norm block has a feed-forward and its norm, or neither")
         self.norm2 = build_part("norm", spec.norm2) if spec.norm2 is not None else None
@@ -35,11 +39,14 @@ class PreNormBlock:
 
     def forward(self, ctx, h, pending, cache_id, write_cache=True, next_norm=None):
         fusable = lambda norm: norm is not None and getattr(norm, "fusable_rmsnorm", False) and norm.size == h.shape[1]
-        if (ctx.kernels.handoff_supported(h.shape[0]) and fusable(self.norm1) and fusable(self.norm2)
+        if (self.scale == 1.0 and ctx.kernels.handoff_supported(h.shape[0]) and fusable(self.norm1) and fusable(self.norm2)
                 and getattr(self.mixer, "forward_handoff", None) is not None
                 and getattr(self.ffn, "forward_handoff", None) is not None):
             # few rows: every norm is shared between the projection before it (which adds into h and leaves
             # h * weight and partial sums of squares) and the projection after it (which applies the scale)
+            if isinstance(pending, Addend):
+                pending.settle(ctx, h)
+                pending = None
             hand = pending if isinstance(pending, Handoff) and pending.norm is self.norm1 else \
                 self.norm1.prenorm(ctx, h, None if isinstance(pending, Complete) else pending)
             hand = self.mixer.forward_handoff(ctx, hand, h, self.norm2, cache_id, write_cache)
@@ -47,12 +54,15 @@ class PreNormBlock:
         if isinstance(pending, Complete):                 # h is complete already
             pending = None
         normed = ctx.workspace.get("normed", tuple(h.shape), ctx.dtype)
-        self.norm1.forward(ctx, h, pending, normed)
-        mixed = self.mixer.forward(ctx, normed, cache_id, write_cache)
+        self.norm1.forward(ctx, h, addend_for(self.norm1, ctx, h, pending), normed)
+        mixed = self._scaled(self.mixer.forward(ctx, normed, cache_id, write_cache))
         if self.ffn is None:
             return mixed                                  # (whoever norms next adds it)
-        self.norm2.forward(ctx, h, mixed, normed)
-        return self.ffn.forward(ctx, normed)
+        self.norm2.forward(ctx, h, addend_for(self.norm2, ctx, h, mixed), normed)
+        return self._scaled(self.ffn.forward(ctx, normed))
+
+    def _scaled(self, delta):
+        return delta if self.scale == 1.0 else Addend(delta, self.scale)
 
 
 @register_part("block", "parallel")

@@ -13,7 +13,7 @@ from ..config.specs import EmbedSpec, HeadSpec
 from ..weights.loader import WeightSpec
 from .registry import PartError, register_part
 
-__all__ = ["TokenEmbedding", "PairEmbedding", "LinearHead", "ScaledHead", "CappedHead", "EmbedSpec", "HeadSpec"]
+__all__ = ["TokenEmbedding", "PairEmbedding", "RunVectors", "LinearHead", "ScaledHead", "CappedHead", "EmbedSpec", "HeadSpec"]
 
 
 @register_part("embed", "token_embedding")
@@ -47,6 +47,30 @@ class TokenEmbedding:
         h = ctx.workspace.get("hidden", (ctx.n_tokens, self.spec.hidden), torch.float32)
         ctx.kernels.embed_gather(ctx.token_ids, self.weight, h, float(getattr(self.spec, "scale", 1.0)))
         return h
+
+
+@register_part("embed", "run_vectors")
+class RunVectors:
+    """Learned vectors that runs of the schedule add to the residual stream, one row of [count, hidden] each; 32-bit."""
+    graph_safe = True
+
+    def __init__(self, spec):
+        if spec.count < 1 or spec.hidden < 1:
+            raise PartError("run vectors need a count and a width")
+        self.spec = spec
+        self.weight = None
+
+    def weight_specs(self):
+        return {"weight": WeightSpec((self.spec.count, self.spec.hidden), keep_float32=True, init=("normal", 0.0, 0.3))}
+
+    def bind(self, weights):
+        self.weight = weights["weight"]
+
+    def libraries(self):
+        return ["elementwise"]
+
+    def row(self, i):
+        return self.weight[i]
 
 
 @register_part("embed", "pair_embedding")

@@ -1,6 +1,6 @@
 """SwiGLU feed-forward: out = (silu(x Wgate^T) * (x Wup^T)) Wdown^T with silu(g) = g / (1 + exp(-g))
 (src/minillm/runtime.cpp:323-336).  Gate and up are one stacked projection.  The gate's activation is the spec's:
-silu, or gelu_tanh (0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3)))); for few rows either rides on the projection,
+silu, gelu_tanh (0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3)))) or relu; for few rows each rides on the projection,
 the norm handed between projections is silu's alone."""
 from __future__ import annotations
 
@@ -14,9 +14,10 @@ from .registry import Handoff, PartError, register_part
 class SwiGluMlp:
     graph_safe = True        # forward launches kernels over the step's device vectors only
     def __init__(self, spec):
-        if spec.activation not in ("silu", "gelu_tanh"):
-            raise PartError(f"activation {spec.activation!r} is not built (silu, gelu_tanh)")
+        if spec.activation not in ("silu", "gelu_tanh", "relu"):
+            raise PartError(f"activation {spec.activation!r} is not built (silu, gelu_tanh, relu)")
         self.spec = spec
+        self.out_name = "ffn_out"                         # (a part that runs it beside others gives it a buffer of its own)
         self.gate_up = None
         self.down = None
         if spec.activation != "silu":         # the projections' fused epilogues are silu's
@@ -38,7 +39,7 @@ class SwiGluMlp:
     def workspace_plan(self, rows, dtype, limits):
         s = self.spec
         return {("act", dtype): rows * s.intermediate, ("gate_up", dtype): rows * 2 * s.intermediate,
-                ("ffn_out", dtype): rows * s.hidden}
+                (self.out_name, dtype): rows * s.hidden}
 
     def forward_handoff(self, ctx, hand, h, norm_after):
         """As `forward` on the norm that `hand` describes, its scale applied inside the first projection; the
@@ -62,8 +63,8 @@ class SwiGluMlp:
         act = ctx.workspace.get("act", (m, s.intermediate), x.dtype)
         if s.activation == "silu" and ctx.kernels.gated_silu_fused(m, s.hidden):
             ctx.kernels.gemm_gated_silu(x, self.gate_up, act)      # few rows: the activation rides on the projection
-        elif s.activation == "gelu_tanh" and m <= 64 and ctx.kernels.streams_weight(m, s.hidden):
-            ctx.kernels.gemm_gated_gelu_tanh(x, self.gate_up, act)
+        elif s.activation != "silu" and m <= 64 and ctx.kernels.streams_weight(m, s.hidden):
+            ctx.kernels.gemm_gated_act(x, self.gate_up, act, s.activation)
         else:
             gate_up = ctx.workspace.get("gate_up", (m, 2 * s.intermediate), x.dtype)
             ctx.kernels.gemm(x, self.gate_up, gate_up)
@@ -71,7 +72,7 @@ class SwiGluMlp:
                 ctx.kernels.silu_mul(gate_up, act)
             else:
                 ctx.kernels.gated_act_mul(gate_up, act, s.activation)
-        out = ctx.workspace.get("ffn_out", (m, s.hidden), x.dtype)
+        out = ctx.workspace.get(self.out_name, (m, s.hidden), x.dtype)
         ctx.kernels.gemm(act, self.down, out)
         return out
 

@@ -13,7 +13,7 @@ import torch
 
 from ..config import load_config
 from ..weights.loader import WeightSpec, load_weights
-from .registry import Complete, PartError, build_part
+from .registry import Addend, Complete, PartError, addend_for, build_part
 
 
 def build_blocks(spec):
@@ -22,12 +22,16 @@ def build_blocks(spec):
 
 def _tensor_plan(config, spec, blocks):
     """([(global name, WeightSpec, owner, local name)] for every tensor of the model, the embedding part, the
-    final norm, the head part); owner is ("embed",), ("final_norm",), ("head",) or (layer index, part name)."""
+    final norm, the head part, the run vectors or None); owner is ("embed",), ("final_norm",), ("head",), ("run_vectors",)
+    or (layer index, part name)."""
     embed = build_part("embed", spec.embed_spec())
     final = build_part("norm", spec.final_norm)
     head = build_part("head", spec.head_spec())
+    vectors = build_part("embed", spec.run_vectors) if spec.run_vectors is not None else None
     plan = []
-    for owner, part in (("embed", embed), ("final_norm", final), ("head", head)):
+    for owner, part in (("embed", embed), ("final_norm", final), ("head", head), ("run_vectors", vectors)):
+        if part is None:
+            continue
         for local, ws in part.weight_specs().items():
             plan.append((config.global_tensor_name(f"{owner}.{local}"), ws, (owner,), local))
     for i, block in enumerate(blocks):
@@ -39,7 +43,7 @@ def _tensor_plan(config, spec, blocks):
     names = [p[0] for p in plan]
     if len(set(names)) != len(names):
         raise PartError("two parts claim the same tensor name")
-    return plan, embed, final, head
+    return plan, embed, final, head, vectors
 
 
 def expected_tensors(config):
@@ -61,8 +65,10 @@ class DecoderModel:
         for run in spec.schedule:
             if not 0 <= run.layer < len(spec.layers):
                 raise PartError(f"the schedule names layer {run.layer} of {len(spec.layers)}")
+            if run.add_vector is not None and not (spec.run_vectors is not None and 0 <= run.add_vector < spec.run_vectors.count):
+                raise PartError(f"the schedule names run vector {run.add_vector}, which the model does not have")
         self.blocks = build_blocks(spec)
-        plan, self.embed, self.final_norm, self.head = _tensor_plan(config, spec, self.blocks)
+        plan, self.embed, self.final_norm, self.head, self.run_vectors = _tensor_plan(config, spec, self.blocks)
         by_owner = {}
         for name, ws, owner, local in plan:
             if name in weights:
@@ -70,6 +76,8 @@ class DecoderModel:
         self.embed.bind(by_owner.get(("embed",), {}))
         self.final_norm.bind(by_owner[("final_norm",)])
         self.head.bind(by_owner.get(("head",), {}), embed=self.embed)      # (tied: the embedding's memory, no copy)
+        if self.run_vectors is not None:
+            self.run_vectors.bind(by_owner.get(("run_vectors",), {}))
         for i, block in enumerate(self.blocks):
             for part_name, part in block.parts().items():
                 part.bind(by_owner.get((i, part_name), {}))
@@ -117,7 +125,7 @@ class DecoderModel:
         return model
 
     def _ends(self):
-        return [self.embed, self.final_norm, self.head]
+        return [self.embed, self.final_norm, self.head] + ([self.run_vectors] if self.run_vectors is not None else [])
 
     def libraries(self):
         """The kernel libraries that the parts of this model launch (each part names its own)."""
@@ -195,25 +203,42 @@ class DecoderModel:
                 raise PartError("the first run cannot add the embedding's output again")
             if extra is not None and getattr(block, "adds_extra", False):
                 more["extra"], extra = extra, None
-            if extra is not None:
+            joins = i + 1 < len(schedule) and schedule[i + 1].add_vector is not None
+            if extra is not None or joins:
                 next_norm = None                          # (the stream is not complete when this block ends)
                 if "next_block" in more:
                     more["next_block"] = None
+            if run.add_vector is not None:
+                pending = self._with_vector(pending, self.run_vectors.row(run.add_vector))
+            if not getattr(block, "takes_addend", False):
+                pending = addend_for(block, ctx, h, pending)
             pending = block.forward(ctx, h, pending, self.cache_ids[run.cache], run.write_cache, next_norm=next_norm, **more)
             if extra is not None:
-                if pending is not None and not isinstance(pending, Complete):
+                if isinstance(pending, Addend):
+                    pending.settle(ctx, h)
+                elif pending is not None and not isinstance(pending, Complete):
                     k.residual_add(h, pending)
                 k.residual_add_float(h, extra)
                 pending = None
             if isinstance(pending, Complete) and i + 1 == len(schedule):
                 pending = None                            # (h is complete)
             if status is not None:                        # h + pending is the hidden state after this run
-                k.finite_check(h, None if isinstance(pending, Complete) else pending, i, status)
+                if isinstance(pending, Addend):
+                    k.finite_check(h, pending.delta, i, status, pending.factor)
+                else:
+                    k.finite_check(h, None if isinstance(pending, Complete) else pending, i, status)
         if ctx.cache is not None and ctx.cache.has_state():
             ctx.cache.commit_state(ctx.segment_slots)     # every layer has run: the staged state becomes live
         r = 0 if want_rows is None else want_rows.numel()
         if r == 0:
             return None
         final = ctx.workspace.get("final", (r, self.spec.hidden), self.dtype)
-        self.final_norm.forward(ctx, h, pending, final, rows=want_rows, write_h=False)
+        self.final_norm.forward(ctx, h, addend_for(self.final_norm, ctx, h, pending), final, rows=want_rows, write_h=False)
         return self.head.forward(ctx, final)
+
+    @staticmethod
+    def _with_vector(pending, vector):
+        """What is still to be added to the stream, and a vector besides."""
+        if isinstance(pending, Addend):
+            return Addend(pending.delta, pending.factor, vector)
+        return Addend(None if isinstance(pending, Complete) else pending, 1.0, vector)

@@ -7,13 +7,14 @@ from __future__ import annotations
 import torch
 
 from ..weights.loader import WeightSpec
-from .registry import register_part
+from .registry import Addend, register_part
 
 
 @register_part("norm", "rmsnorm")
 class RmsNorm:
     graph_safe = True        # forward launches kernels over the step's device vectors only
     fusable_rmsnorm = True   # the projections before and after it may share this norm between them (weight, eps as here)
+    takes_addend = True      # a delta with a factor, and a vector that joins every row, ride in the norm's pass
     def __init__(self, spec):
         self.size, self.eps = spec.size, float(spec.eps)
         self.offset = float(getattr(spec, "weight_offset", 0.0))
@@ -40,7 +41,11 @@ class RmsNorm:
         return Handoff(self, x, ss)
 
     def forward(self, ctx, h, delta, out, rows=None, write_h=True):
-        ctx.kernels.add_rmsnorm(h, delta, self.weight, out, self.eps, rows=rows, write_h=write_h)
+        if isinstance(delta, Addend):
+            ctx.kernels.add_rmsnorm(h, delta.delta, self.weight, out, self.eps, rows=rows, write_h=write_h,
+                                    factor=delta.factor, vector=delta.vector)
+        else:
+            ctx.kernels.add_rmsnorm(h, delta, self.weight, out, self.eps, rows=rows, write_h=write_h)
         return out
 
 

@@ -13,7 +13,7 @@ import torch
 
 from ..cache.manager import StateSpec
 from ..weights.loader import WeightSpec, stacked
-from .registry import PartError, register_part
+from .registry import PartError, build_part, register_part
 
 WHOLE = 1 << 30          # `StepContext.token_groups(WHOLE)`: every request of the step as one group of rows
 PIECE = 128              # tokens of a piece when a step's portions run in pieces side by side
@@ -216,9 +216,11 @@ class Mamba2:
 
 @register_part("mixer", "decayed_linear_attention")
 class DecayedLinearAttention:
-    """q = act(Wq x), k = act(Wk x) (heads x head_dim), v = act(Wv x) (heads x value_dim); per head the recurrence
-    above with ONE constant decay a head on every key channel, no other factor; the heads side by side are RMS-normed
-    as one row with a weight as wide as the row, multiplied by gate(Wg x) and projected by Wo."""
+    """q = act(Wq x), k = act(Wk x) (heads x head_dim), v = act(Wv x) (heads x value_dim), q and k optionally turned by
+    their position (inside the recurrence kernel, 32-bit), k times `k_scale`; per head the recurrence above with ONE
+    constant decay a head on every key channel; the heads side by side are RMS-normed as one row with a weight as wide
+    as the row (`norm` "row"), or each head's o is divided by its own root mean square (`norm` "heads"), multiplied by
+    gate(Wg x) and projected by Wo."""
     graph_safe = True
 
     def __init__(self, spec):
@@ -229,6 +231,9 @@ class DecayedLinearAttention:
             raise PartError(f"decay: one number in (0, 1] for each of the {s.heads} heads")
         if s.activation not in (None, "silu") or s.gate not in ("sigmoid", "silu"):
             raise PartError(f"activation {s.activation!r} / gate {s.gate!r}: silu or none / sigmoid or silu")
+        if s.norm not in ("row", "heads"):
+            raise PartError(f"norm {s.norm!r}: row or heads")
+        self.position = build_part("position", s.position) if s.position is not None else None
         self.qk_width, self.v_width = s.heads * s.head_dim, s.heads * s.value_dim
         self.out_name = "mixer_out"
         self.proj = self.norm = self.o = self._log_decay = None
@@ -237,12 +242,13 @@ class DecayedLinearAttention:
         s = self.spec
         return {"q": WeightSpec((self.qk_width, s.hidden), stack="qkvg"), "k": WeightSpec((self.qk_width, s.hidden), stack="qkvg"),
                 "v": WeightSpec((self.v_width, s.hidden), stack="qkvg"), "g": WeightSpec((self.v_width, s.hidden), stack="qkvg"),
-                "o": WeightSpec((s.hidden, self.v_width)), "norm": WeightSpec((self.v_width,), keep_float32=True)}
+                "o": WeightSpec((s.hidden, self.v_width)),
+                **({"norm": WeightSpec((self.v_width,), keep_float32=True)} if s.norm == "row" else {})}
 
     def bind(self, weights):
         import math
         self.proj = stacked([weights[n] for n in ("q", "k", "v", "g")])
-        self.norm, self.o = weights["norm"], weights["o"]
+        self.norm, self.o = weights.get("norm"), weights["o"]
         # (the logarithm in 64-bit, rounded once: the kernel's exp gives the decay back to the last bit or so)
         self._log_decay = torch.tensor([math.log(float(d)) for d in self.spec.decay], dtype=torch.float32,
                                        device=self.o.device)
@@ -274,12 +280,24 @@ class DecayedLinearAttention:
         _recurrence(ctx, s.heads * s.head_dim * s.value_dim, s.heads, s.head_dim,
                     proj[:, :a], proj[:, a:b], proj[:, b:c], self._log_decay, o, ctx.cache.state_view(cache_id),
                     ctx.cache.state_stage(cache_id), 0, ctx.slots, s.heads, s.head_dim, s.value_dim,
-                    write_state=write_cache, activation=s.activation)
+                    q_scale=float(s.k_scale), write_state=write_cache, activation=s.activation, **self._turns(ctx, x.device))
         y = ws.get("recurrent_normed", (m, self.v_width), x.dtype)
-        k.gated_part_norm(o, proj[:, c:], self.norm, y, self.v_width, float(s.eps), gate_first=False, gate_kind=s.gate)
+        k.gated_part_norm(o, proj[:, c:], self.norm, y, self.v_width if s.norm == "row" else s.value_dim, float(s.eps),
+                          gate_first=False, gate_kind=s.gate)
         out = ws.get(self.out_name, (m, s.hidden), x.dtype)
         k.gemm(y, self.o, out)
         return out
+
+
+    def _turns(self, ctx, device):
+        """The rotation of q and k, as the recurrence takes it.  (`k_scale` is given to it as the factor on q: every product
+        holds one of either.)"""
+        rotation = self.position.rotation(ctx.max_positions, device) if self.position is not None else None
+        if rotation is None:
+            return {}
+        if rotation.interleaved or rotation.dim > self.spec.head_dim:
+            raise PartError("the recurrence turns a head's first channels in split-half pairs")
+        return dict(rope=rotation.table, positions=ctx.positions)
 
 
 @register_part("mixer", "delta_rule")

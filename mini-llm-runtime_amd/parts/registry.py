@@ -20,7 +20,8 @@ Interfaces (B = the tokens of a step, E = the model width, T = the engine's elem
                   `pending` may also be a `Handoff` (h is complete and the first half of a norm is
                   done); a block may return one for `next_norm`, the norm the next block starts with.
                   Any `Complete` object says that h is complete; a block that does not know its kind
-                  ignores what it carries.  A block class with `wants_next_block = True` is also given
+                  ignores what it carries.  A block may return an `Addend` (a delta with a factor); only a
+                  block with `takes_addend = True` is handed one, for the others the model adds it into h.  A block class with `wants_next_block = True` is also given
                   `next_block=` (the block that runs next, or None).
   embed           weight_specs(), bind(), libraries();  forward(ctx) -> the float residual stream [B, E] of
                   the step's tokens (ctx.token_ids);  optional table() -> the [vocab, E] matrix that a tied head
@@ -28,6 +29,7 @@ Interfaces (B = the tokens of a step, E = the model width, T = the engine's elem
   head            weight_specs(), bind(weights, embed=the embedding part), libraries();
                   forward(ctx, final) -> float logits [R, V] of the normed rows final [R, E];
                   workspace_plan(rows, logits_rows, dtype, limits).
+  norms with `takes_addend = True` take an `Addend` for `delta`.
   Optional, for steps of few rows (each falls back to forward when a part lacks it):
   norm            handoff-capable norms set `fusable_rmsnorm = True` and offer
                   prenorm(ctx, h, delta) -> Handoff.
@@ -81,6 +83,28 @@ class Rotation:
 class Complete:
     """What a block may hand to the next one instead of a pending delta: the residual stream h is complete
     (nothing is left to be added), and the object carries something that the next block may use or ignore."""
+
+
+@dataclass
+class Addend:
+    """What is still to be added to the residual stream where that is more than a plain delta: factor * delta + vector,
+    `delta` being a sublayer's output and `vector` a float row [E] that joins every token's; either may be None."""
+    delta: object
+    factor: float = 1.0
+    vector: object = None
+
+    def settle(self, ctx, h):
+        """Add it into h in a pass of its own (for a reader that does not take it into its own pass)."""
+        ctx.kernels.residual_add(h, self.delta, self.factor, self.vector)
+
+
+def addend_for(norm, ctx, h, pending):
+    """`pending` (a delta, an `Addend` or None) as `norm.forward` may be given it: what the norm does not take is added
+    into h here."""
+    if isinstance(pending, Addend) and not getattr(norm, "takes_addend", False):
+        pending.settle(ctx, h)
+        return None
+    return pending
 
 
 @dataclass

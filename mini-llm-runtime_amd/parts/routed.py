@@ -6,7 +6,9 @@ number an expert while the weights stay the plain s.  The scores may be softmax(
 a group's score its largest s.  An expert is an ungated feed-forward down(act(up(x))) or, `gated`, down(act(gate(x)) *
 up(x)), or with the activation `clamped` down(g sigmoid(slope g) (u + 1)) of the clamped g and u.  A shared expert (any
 feed-forward part) runs for every token besides and is added by the pass that sums the chosen experts, multiplied by
-sigmoid(sg . x) when `shared_gate` says so: sg is one more row of the router's product.
+sigmoid(sg . x) when `shared_gate` says so: sg is one more row of the router's product.  `identity` further router outputs
+behind the experts' stand for experts without tensors whose output is x: they are scored and chosen like the others, no
+row is multiplied for them, and the pass that sums a token's experts takes x in their place.
 
 The step's (token, expert) pairs are sorted by expert on the device, so that every expert's rows lie side by side
 and ONE launch multiplies all of them with their own weights (`Kernels.experts_gemm`, the rows of the first product
@@ -47,9 +49,11 @@ class RoutedMlp:
             raise PartError("a gate for a shared expert that is not there")
         self.correction = None
         self.fused_gate = False
-        if s.experts % s.group_count != 0 or not 1 <= s.group_keep <= s.group_count or \
-                not 1 <= s.top <= s.group_keep * (s.experts // s.group_count):
-            raise PartError(f"routing: {s.experts} experts in {s.group_count} groups of which {s.group_keep} stay cannot "
+        self.identity = int(getattr(s, "identity", 0))
+        self.choices = s.experts + self.identity         # what a token chooses among
+        if self.identity < 0 or self.choices % s.group_count != 0 or not 1 <= s.group_keep <= s.group_count or \
+                not 1 <= s.top <= s.group_keep * (self.choices // s.group_count):
+            raise PartError(f"routing: {self.choices} experts in {s.group_count} groups of which {s.group_keep} stay cannot "
                             f"give {s.top} choices")
         self.router = self.up = self.down = None
 
@@ -58,14 +62,14 @@ class RoutedMlp:
         # (a matrix like the others: its products with the layer's input are exact in 32 bits, and so are their sums'
         # partial results up to rounding: the logits are an ordinary product with float output)
         gate = bool(s.shared_gate)
-        specs = {"router": WeightSpec((s.experts, s.hidden), init=("normal", 0.0, 0.05), stack="route" if gate else None)}
+        specs = {"router": WeightSpec((self.choices, s.hidden), init=("normal", 0.0, 0.05), stack="route" if gate else None)}
         if gate:                                # (one more row of the router's product)
             specs["shared.sg"] = WeightSpec((1, s.hidden), init=("normal", 0.0, 0.05), stack="route")
         if self.shared is not None:
             for local, ws in self.shared.weight_specs().items():
                 specs[f"shared.{local}"] = replace(ws, stack=f"shared.{ws.stack}") if ws.stack is not None else ws
         if getattr(s, "correction", False):
-            specs["correction"] = WeightSpec((s.experts,), keep_float32=True, init=("normal", 0.0, 0.05))
+            specs["correction"] = WeightSpec((self.choices,), keep_float32=True, init=("normal", 0.0, 0.05))
         for e in range(s.experts):
             if self.gated:                      # (an expert's gate and up side by side: one product gives both)
                 specs[f"e{e}.gate"] = WeightSpec((s.intermediate, s.hidden), stack="up")
@@ -106,9 +110,9 @@ class RoutedMlp:
         s = self.spec
         pairs = rows * s.top
         return {**(self.shared.workspace_plan(rows, dtype, limits) if self.shared is not None else {}),
-                ("route_logits", torch.float32): rows * (s.experts + (1 if s.shared_gate else 0)), ("route_ids", torch.int32): pairs,
+                ("route_logits", torch.float32): rows * (self.choices + (1 if s.shared_gate else 0)), ("route_ids", torch.int32): pairs,
                 ("route_weights", torch.float32): pairs,
-                ("route_offsets", torch.int32): s.experts + 1, ("route_token", torch.int32): pairs,
+                ("route_offsets", torch.int32): self.choices + 1, ("route_token", torch.int32): pairs,
                 ("route_row", torch.int32): pairs, ("route_act", dtype): pairs * s.intermediate,
                 **({("route_gate_up", dtype): pairs * 2 * s.intermediate} if self.gated else {}),
                 ("route_y", dtype): pairs * s.hidden, ("ffn_out", dtype): rows * s.hidden}
@@ -120,15 +124,16 @@ class RoutedMlp:
         pairs = m * s.top
         ids = ws.get("route_ids", (m, s.top), torch.int32)
         weights = ws.get("route_weights", (m, s.top), torch.float32)
-        offsets = ws.get("route_offsets", (s.experts + 1,), torch.int32)
+        offsets = ws.get("route_offsets", (self.choices + 1,), torch.int32)
         token_of = ws.get("route_token", (pairs,), torch.int32)
         row_of = ws.get("route_row", (pairs,), torch.int32)
         logits = ws.get("route_logits", (m, self.router.shape[0]), torch.float32)
         k.gemm(x, self.router, logits)                   # 32-bit sums of the engine's element type's products
         k.router_topk(logits, ids, weights, s.group_count, s.group_keep, correction=self.correction,
                       renormalize=bool(s.renormalize), scale=float(getattr(s, "route_scale", 1.0)), score=s.score,
-                      group_score=s.group_score, experts=s.experts)
-        k.route_sort(ids, s.experts, offsets, token_of, row_of)
+                      group_score=s.group_score, experts=self.choices)
+        k.route_sort(ids, self.choices, offsets, token_of, row_of)
+        offsets = offsets[:s.experts + 1]                # (the pairs of experts without tensors lie behind the others')
         act = ws.get("route_act", (pairs, s.intermediate), x.dtype)
         if self.fused_gate:
             k.experts_gemm(x, self.up, act, offsets, gather=token_of, act="gated_" + s.activation, limit=float(s.limit or 0.0),
@@ -145,9 +150,10 @@ class RoutedMlp:
         y = ws.get("route_y", (pairs, s.hidden), x.dtype)
         k.experts_gemm(act, self.down, y, offsets)
         out = ws.get("ffn_out", (m, s.hidden), x.dtype)
+        more = dict(ids=ids, experts=s.experts, x=x) if self.identity else {}
         if self.shared is None:
-            k.route_combine(y, row_of, weights, out)
+            k.route_combine(y, row_of, weights, out, **more)
         else:
             k.route_combine(y, row_of, weights, out, shared=self.shared.forward(ctx, x),
-                            shared_gate=logits[:, s.experts:] if s.shared_gate else None)
+                            shared_gate=logits[:, self.choices:] if s.shared_gate else None, **more)
         return out

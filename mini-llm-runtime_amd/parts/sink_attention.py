@@ -1,7 +1,7 @@
 """Two mixers whose softmax has a sink -- one more summand exp(sink[head]) in the denominator, a learned number a
 head that stands for no key and brings no value -- and whose queries see the keys that a mask rule names: the last
-`size` positions (`window`) or the positions of the query's own block of `size` (`chunk`), counted from the
-request's first token.
+`size` positions (`window`; with `keep_first` the request's first tokens besides) or the positions of the query's own
+block of `size` (`chunk`), counted from the request's first token.  Scores may be capped, c tanh(score / c).
 
 `SinkAttention`: grouped-query attention with query/key and value sizes of their own, optional biases on q, k, v,
 a norm per head of q and k before the rotation (or after it; with a weight shared by the heads or without one), a
@@ -32,6 +32,8 @@ def _mask_of(spec):
         return None, 0
     if spec.mask.kind not in ("window", "chunk") or spec.mask.size < 1:
         raise PartError(f"mask {spec.mask.kind!r} of size {spec.mask.size}: window or chunk, of a positive size")
+    if spec.mask.keep_first < 0 or (spec.mask.keep_first > 0 and spec.mask.kind != "window"):
+        raise PartError("a window may keep a request's first tokens")
     return spec.mask.kind, int(spec.mask.size)
 
 
@@ -60,13 +62,15 @@ def _groups_plan(rows, q_heads, kv_heads, value_dim):
             ("sink_partial", torch.float32): min(PARTIAL_CAP, Kernels.sink_partial_numel(rows, small_tokens, q_heads, value_dim, MOST_RANGES))}
 
 
-def _key_ranges(ctx, groups, tokens, workgroups, q_heads, value_dim, mask, mask_size):
+def _key_ranges(ctx, groups, tokens, workgroups, q_heads, value_dim, mask, mask_size, keep_first=0):
     """(keys a range, ranges, room for their shares) for a launch over `groups` groups of single tokens or short portions
     that has `workgroups` workgroups without ranges: where those do not fill the GPU, a group's keys (its window or
     chunk; without a mask the step's longest context) are dealt out to several workgroups, as many as reach
     `target_workgroups`, none narrower than RANGE_KEYS, and no more than their shares have room for."""
     k = ctx.kernels
     reach = (mask_size if mask == "chunk" else mask_size + tokens - 1) if mask is not None else ctx.max_context
+    if mask is not None and keep_first > 0:
+        reach += -(-keep_first // 32) * 32
     reach = min(reach, ctx.max_context + 31) + 31             # (ranges start at the first tile, which may start earlier)
     most = max(1, min(MOST_RANGES, -(-reach // RANGE_KEYS), -(-ctx.target_workgroups // max(1, workgroups))))
     room = ctx.workspace.get("sink_partial", (min(PARTIAL_CAP, k.sink_partial_numel(groups, tokens, q_heads, value_dim, most)),),
@@ -78,14 +82,15 @@ def _key_ranges(ctx, groups, tokens, workgroups, q_heads, value_dim, mask, mask_
     return keys, -(-reach // keys), room
 
 
-def attend(ctx, q, k_pages, v_pages, view, sink, out, q_heads, kv_heads, key_dim, value_dim, scale, mask, mask_size):
+def attend(ctx, q, k_pages, v_pages, view, sink, out, q_heads, kv_heads, key_dim, value_dim, scale, mask, mask_size,
+           keep_first=0, softcap=None):
     """Every token of the step over the keys it sees.  The bfloat16 engine on the matrix cores where they take the
     sizes (prompt portions in workgroups of 64 columns, single tokens and short portions in workgroups of 16 whose
     wavefronts share the value channels); else, and in the float engine, one wavefront a (token, head), whose sums
     follow from the token's position alone."""
     k = ctx.kernels
     if k.sink_tiles_supported(key_dim, value_dim, k_pages.shape[3], v_pages.shape[3], view.page_size, mask, mask_size,
-                              ctx.max_positions) and q.shape[1] % 8 == 0:
+                              ctx.max_positions, keep_first) and q.shape[1] % 8 == 0:
         big_heads, big_tokens, small_heads, small_tokens = k.sink_tiles_layout(q_heads, kv_heads)
         small, big, _ = ctx.token_groups(small_tokens, max(1, big_tokens // small_tokens))
         for (first, count, n), heads, split in ((big, big_heads, False), (small, small_heads, True)):
@@ -94,13 +99,15 @@ def attend(ctx, q, k_pages, v_pages, view, sink, out, q_heads, kv_heads, key_dim
             keys, ranges, room = (0, 1, None)
             if split:
                 per_group = kv_heads * -(-(q_heads // kv_heads) // heads)
-                keys, ranges, room = _key_ranges(ctx, n, small_tokens, n * per_group, q_heads, value_dim, mask, mask_size)
+                keys, ranges, room = _key_ranges(ctx, n, small_tokens, n * per_group, q_heads, value_dim, mask, mask_size,
+                                                 keep_first)
             k.sink_attention_tiles(q, k_pages, v_pages, view.block_table, ctx.slots, ctx.positions, sink, out, first,
                                    count, n, heads, split, q_heads, kv_heads, key_dim, value_dim, view.page_size,
-                                   scale, mask, mask_size, ctx.max_positions, partial=room, split_keys=keys, splits=ranges)
+                                   scale, mask, mask_size, ctx.max_positions, partial=room, split_keys=keys, splits=ranges,
+                                   keep_first=keep_first, softcap=softcap)
         return
     k.sink_attention(q, k_pages, v_pages, view.block_table, ctx.slots, ctx.positions, sink, out, q_heads, kv_heads,
-                     key_dim, value_dim, view.page_size, scale, mask, mask_size)
+                     key_dim, value_dim, view.page_size, scale, mask, mask_size, keep_first, softcap)
 
 
 @register_part("mixer", "sink_attention")
@@ -112,6 +119,9 @@ class SinkAttention:
         if s.q_heads % s.kv_heads != 0:
             raise PartError(f"q_heads {s.q_heads} is no multiple of kv_heads {s.kv_heads}")
         self.mask, self.mask_size = _mask_of(s)
+        self.keep_first = s.mask.keep_first if s.mask is not None else 0
+        if s.softcap is not None and not s.softcap > 0:
+            raise PartError("softcap must be positive")
         if s.qk_norm is not None and s.qk_norm.size != s.head_dim:
             raise PartError("the q/k norm must span one head")
         self.position = build_part("position", s.position) if s.position is not None else None
@@ -151,7 +161,7 @@ class SinkAttention:
     def cache_spec(self):
         s = self.spec
         return PagedSpec((("k", (s.kv_heads, PAGE, s.head_dim)), ("v", (s.kv_heads, PAGE, s.value_dim))),
-                         self.mask_size if self.mask is not None else None)
+                         self.mask_size if self.mask is not None else None, keep_first=self.keep_first)
 
     def libraries(self):
         return ["gemm", "sink_attention", "elementwise"]
@@ -179,7 +189,7 @@ class SinkAttention:
                         s.head_dim, s.value_dim, view.page_size, write_cache, norm=self.norm_order, interleaved=interleaved)
         attn = ctx.workspace.get("attn", (m, self.o_width), x.dtype)
         attend(ctx, q, k_pages, v_pages, view, self.sink, attn, s.q_heads, s.kv_heads, s.head_dim, s.value_dim,
-               float(s.scale), self.mask, self.mask_size)
+               float(s.scale), self.mask, self.mask_size, self.keep_first, s.softcap)
         if s.gate is not None:
             k.gate_mul(attn, proj[:, qkv_width:], attn, s.gate)
         out = ctx.workspace.get(self.out_name, (m, s.hidden), x.dtype)

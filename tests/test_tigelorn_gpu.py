@@ -458,7 +458,7 @@ def test_the_gelu_gate_fused_into_the_projection(rows):
     a = rounded(rng.normal(size=(rows, inner)), torch.bfloat16)
     w = rounded(rng.normal(size=(2 * n, inner)) * 0.2, torch.bfloat16)
     out = torch.empty(rows, n, dtype=torch.bfloat16, device="cuda")
-    k.gemm_gated_gelu_tanh(a, w, out)
+    k.gemm_gated_act(a, w, out, "gelu_tanh")
     want = P.gated_ffn(back(a), {"gate": back(w)[:n], "up": back(w)[n:], "down": np.eye(n)})
     np.testing.assert_allclose(back(out), want, atol=1e-2 * np.abs(want).max(), rtol=1e-2)
 
