@@ -32,6 +32,9 @@ many gigabytes).  Every runner is built with the product's own defaults.  One JS
   * --only nuvorax: the same for Nuvorax models (attention whose heads' weights are mixed, over turned values, beside a
     dense feed-forward and a mixture of clamped experts with a shared expert in turn), beside a Pamunex model of equal
     sizes.
+  * --only sagopel: the same for Sagopel models (linear attention with a constant decay a head, and windowed attention
+    beside retention, with a dense feed-forward and mixtures of gated experts some of which give their input back; two of
+    the six layers run twice), beside a Tigelorn model of equal sizes.
 """
 import argparse
 import json
@@ -801,16 +804,95 @@ class NuvoraxBench(Bench):
                     frac=round(step_bytes / (seconds / steps) / HBM_PEAK, 5)), step_bytes, report
 
 
+# `--only sagopel`: layer sizes that resemble a real model's, for a Sagopel model of six layers -- linear attention with a
+# constant decay a head, or windowed attention (the first 64 tokens kept) beside retention -- of which the third and the
+# fourth run twice (eight runs a token), the first beside a dense feed-forward, the others beside a mixture of sixteen gated
+# experts and four identities of which a token uses four (an expert has an eighth of the dense inner size) and a shared
+# expert (half of it), and for the closest model the engine had before: a Tigelorn model of the same width, feed-forward,
+# heads and runs.
+SAGOPEL_SIZES = {
+    "2k": dict(width=2048, ff=5632, vocab=32000, layers=8, heads=16, kv_heads=4, window=1024, keep=64),
+    "4k": dict(width=4096, ff=12288, vocab=32000, layers=8, heads=32, kv_heads=8, window=1024, keep=64),
+}
+
+
+class SagopelBench(Bench):
+    """A Sagopel model of SAGOPEL_SIZES[size] with random weights drawn on the GPU."""
+    EXPERTS, IDENTITY, TOP = 16, 4, 4
+
+    def __init__(self, size, args):
+        import torch
+        from mini_llm_runtime_amd.api import parse_dtype
+        from mini_llm_runtime_amd.config import config_from_dict
+        from mini_llm_runtime_amd.parts import DecoderModel, expected_tensors
+        from mini_llm_runtime_amd.weights import random_tensors_on_device
+        d = SAGOPEL_SIZES[size]
+        self.torch, self.args, self.size = torch, args, size
+        self.dtype = parse_dtype(args.dtype)
+        self.tag = "bf16" if self.dtype == torch.bfloat16 else "fp32"
+        h, w, ff = d["heads"], d["width"], d["ff"]
+        decay = [1.0 - 2.0 ** -(2 + 6 * i / (h - 1)) for i in range(h)]
+        rot = dict(dims=64, base=1000000.0)
+        linear = dict(heads=h, dim=128, vdim=128, decay=decay)
+        left = dict(heads=h, kv_heads=d["kv_heads"], dim=128, vdim=128, scale=128 ** -0.5, softcap=50.0, rot=rot,
+                    mask=dict(size=d["window"], keep_first=d["keep"]))
+        dense = dict(kind="dense", ff=ff)
+        moe = dict(kind="moe", expert=dict(ff=ff // 8), shared=dict(ff=ff // 2),
+                   router=dict(experts=self.EXPERTS, identity=self.IDENTITY, top=self.TOP))
+        lightning = lambda mlp: dict(type="lightning", mixer=linear, mlp=mlp)
+        parallel = dict(type="parallel", mixer=dict(left=left, right=dict(linear, rot=dict(rot, dims=128))), mlp=moe)
+        layers = [lightning(dense), lightning(moe), parallel, lightning(moe), parallel, lightning(moe)]
+        self.cfg = config_from_dict(dict(architecture="Sagopel", vocab=d["vocab"], width=w, norm=dict(eps=1e-5), residual_mult=0.4,
+                                         loop=dict(start=2, stop=4, times=2), layers=layers))
+        self.model = DecoderModel(self.cfg, random_tensors_on_device(expected_tensors(self.cfg), 0, self.dtype, "cuda"),
+                                  self.dtype, "cuda:0")
+        self.weights_from = "drawn on the GPU"
+        self.layers = self.full_layers = d["layers"]
+        self.elem = 2 if self.dtype == torch.bfloat16 else 4
+        runs = [layers[i] for i, _ in self.cfg.run_order()]
+        n_par, n_moe = (sum(1 for r in runs if r[key] is part) for key, part in (("mixer", parallel["mixer"]), ("mlp", moe)))
+        n = len(runs)
+        linear_w, left_w = 5 * w * h * 128, 2 * w * h * 128 + w * d["kv_heads"] * 256
+        shared = 3 * w * (ff // 2)
+        # (a layer that runs twice is read twice)
+        self.common = n * linear_w + n_par * left_w + (n - n_moe) * 3 * w * ff + n_moe * (shared + (self.EXPERTS + self.IDENTITY) * w)
+        self.expert, self.n_moe = 3 * w * (ff // 8), n_moe
+        self.with_tensors = self.TOP * self.EXPERTS / (self.EXPERTS + self.IDENTITY)      # of a token's choices, about
+        self.matrix_params = self.common + n_moe * self.with_tensors * self.expert
+        self.weight_bytes = (self.common + n_moe * self.EXPERTS * self.expert + d["vocab"] * w) * self.elem   # (of the table a row a token)
+        self.window_row_bytes = n_par * d["kv_heads"] * 256 * self.elem
+        self.state_bytes = n * h * 128 * 128 * 4 * 2
+        self.kv_bytes_per_token = 0                  # (see decode_point)
+        seen = lambda t: sum(min(p + 1, d["window"] + d["keep"]) for p in range(t))
+        self.attention_flops = lambda t: n_par * 2.0 * seen(t) * h * 256 + n * 2 * 2.0 * t * h * 128 * 128
+        self.vocab = d["vocab"]
+        self.g = torch.Generator().manual_seed(0)
+
+    def prefill_flops(self, t):
+        d = SAGOPEL_SIZES[self.size]
+        return 2.0 * t * self.matrix_params + self.attention_flops(t) + 2.0 * d["vocab"] * d["width"]
+
+    def decode_point(self, batch, steps, warmup, context=None):
+        d = SAGOPEL_SIZES[self.size]
+        seconds, mean_context, report = self.decode(batch, steps, warmup, context)
+        touched = self.EXPERTS * (1.0 - (1.0 - self.with_tensors / self.EXPERTS) ** batch)      # experts that a step's tokens choose, about
+        weights = (self.common + self.n_moe * touched * self.expert + d["vocab"] * d["width"]) * self.elem
+        step_bytes = weights + batch * (min(mean_context, d["window"] + d["keep"]) * self.window_row_bytes + self.state_bytes)
+        return dict(tok_s=round(batch * steps / seconds, 1), ms=round(seconds / steps * 1e3, 4),
+                    frac=round(step_bytes / (seconds / steps) / HBM_PEAK, 5)), step_bytes, report
+
+
 def design_block(args):
     """Prefill (2048 tokens in one step) and decode (batch 8 and 64 behind --context tokens) of a design's sizes
     beside the closest model the engine had before it (a Qwen3 dense model of equal width, heads, feed-forward and
-    layers; for Tigelorn a Taletar model, for Budorax a Tigelorn model, for Nuvorax a Pamunex model of equal sizes); then
+    layers; for Tigelorn a Taletar model, for Budorax and Sagopel a Tigelorn model, for Nuvorax a Pamunex model of equal sizes); then
     the same steps once more with events around every launch: milliseconds per kernel class."""
     import copy
     out = {}
     design = getattr(args, "design", "taletar")
     table, make_design = {"pamunex": (PAMUNEX_SIZES, PamunexBench), "tigelorn": (TIGELORN_SIZES, TigelornBench),
-                          "budorax": (BUDORAX_SIZES, BudoraxBench), "nuvorax": (NUVORAX_SIZES, NuvoraxBench)}.get(design, (DESIGN_SIZES, TaletarBench))
+                          "budorax": (BUDORAX_SIZES, BudoraxBench), "nuvorax": (NUVORAX_SIZES, NuvoraxBench),
+                          "sagopel": (SAGOPEL_SIZES, SagopelBench)}.get(design, (DESIGN_SIZES, TaletarBench))
     for size in (args.design_sizes.split(",") if args.design_sizes else list(table)):
         d = table[size]
         dense = (d["layers"], dict(hidden_size=d["width"], num_attention_heads=d["heads"], num_key_value_heads=d["kv_heads"],
@@ -819,7 +901,7 @@ def design_block(args):
                                    tie_word_embeddings=False))
         block = {}
         beside = ("taletar", lambda a: TaletarBench(size, a)) if design == "tigelorn" else \
-            ("tigelorn", lambda a: TigelornBench(size, a)) if design == "budorax" else \
+            ("tigelorn", lambda a: TigelornBench(size, a)) if design in ("budorax", "sagopel") else \
             ("pamunex", lambda a: PamunexBench(size, a)) if design == "nuvorax" else \
             ("qwen3_dense", lambda a: Bench(size, 0, a, sizes=dense))
         for name, make in ((design, lambda a: make_design(size, a)), beside):
@@ -864,12 +946,12 @@ def main():
     ap.add_argument("--warm-up", type=int, default=0,
                     help="--only engine: 1 captures the decoding steps (Engine.warm_up) before the first burst")
     ap.add_argument("--only", default="all", choices=["all", "decode", "prefill", "prompt", "engine", "mixed", "taletar", "pamunex", "tigelorn", "budorax",
-                                                         "nuvorax"],
+                                                         "nuvorax", "sagopel"],
                     help="profiling aid: run just the decode steps, just the prefill or just the mixed step; prompt: one "
                          "prompt of --context tokens in portions of 2048; engine: the "
                          "scheduler over a burst of requests (3 x batch requests of 512 prompt and 128 output tokens, "
                          "batch slots), printed as one line of its own")
-    ap.add_argument("--design-sizes", default="", help="--only taletar / pamunex / tigelorn / budorax / nuvorax: which of its sizes (2k, 4k; default both)")
+    ap.add_argument("--design-sizes", default="", help="--only taletar / pamunex / tigelorn / budorax / nuvorax / sagopel: which of its sizes (2k, 4k; default both)")
     ap.add_argument("--library", type=int, default=1,
                     help="0: every matrix product on the hand-written kernels, none in the vendor library")
     ap.add_argument("--split-keys", type=int, default=256, help="the smallest range of keys of one attention workgroup")
@@ -893,7 +975,7 @@ def main():
     if not args.tune:
         from mini_llm_runtime_amd.kernels import build
         build.load("library_gemm").mlr_library_gemm_tuning(0)
-    if args.only in ("taletar", "pamunex", "tigelorn", "budorax", "nuvorax"):
+    if args.only in ("taletar", "pamunex", "tigelorn", "budorax", "nuvorax", "sagopel"):
         args.design = args.only
         print(json.dumps({f"{args.only}_sizes": design_block(args), "context": args.context, "dtype": args.dtype}))
         return 0

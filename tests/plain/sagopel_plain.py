@@ -132,6 +132,19 @@ def retention(x, w, cfg, eps):
     return (o * silu(x @ w["g"].T)) @ w["o"].T
 
 
+def retention_margin(x, w, cfg, rounding=2.0 ** -9):
+    """[T]: the smallest of a token's heads' outputs (root mean square), in units of what rounding q, k and v (relative, per
+    element) may move it by: a head whose output nearly cancels is brought to size one all the same."""
+    T = x.shape[0]
+    H, D, V = cfg["heads"], cfg["dim"], cfg["vdim"]
+    pos = np.arange(T)
+    q, k = (rotate((x @ w[n].T).reshape(T, H, D), pos, cfg["rot"]["dims"], cfg["rot"]["base"]) for n in "qk")
+    v = (x @ w["v"].T).reshape(T, H, V)
+    size = lambda a: np.sqrt(np.mean(a * a, axis=1))
+    return np.min([size(decayed_sum(q[:, h], k[:, h], v[:, h], cfg["decay"][h]))
+                   / (rounding * size(decayed_sum(abs(q[:, h]), abs(k[:, h]), abs(v[:, h]), cfg["decay"][h]))) for h in range(H)], axis=0)
+
+
 def two_mixers(x, w, cfg, eps):
     """Half the sum of two mixers' outputs, each normed over the model's width first."""
     left = window_attention(x, sub(w, "left"), cfg["left"], eps)
@@ -157,17 +170,19 @@ def route(x, w, router):
     return order, np.take_along_axis(s, order, axis=1)
 
 
-def route_margin(x, w, cfg):
-    """How far a token's choice is from another one: the gap between the last chosen and the first not chosen, over a
-    bound on what rounding x to bfloat16 moves it by (infinite where every expert is chosen)."""
-    router = cfg["router"]
-    s = softmax_rows(x @ w["router"].T)
-    c = np.sort(s + w["correction"], axis=1)[:, ::-1]
-    top = router["top"]
-    if top >= c.shape[1]:
+def route_margin(x, w, cfg, rounding=2.0 ** -8):
+    """[T]: how far each token's choice is from another one, in units of what rounding x (relative, per element) may move
+    a choice score: the gap between the last output chosen and the best one left (infinite where every one is chosen)."""
+    top = cfg["router"]["top"]
+    z = x @ w["router"].T
+    if top >= z.shape[1]:
         return np.full(x.shape[0], np.inf)
-    move = 2.0 ** -9 * np.sqrt((x ** 2).sum(axis=1)) * np.sqrt((w["router"] ** 2).sum(axis=1)).max()
-    return (c[:, top - 1] - c[:, top]) / (move * s.max(axis=1) + 1e-30)
+    s = softmax_rows(z)
+    c = s + w["correction"]
+    moved = (rounding * np.sqrt((x * x) @ (w["router"] ** 2).T)).max(axis=1) + 1e-300
+    order = np.argsort(-c, axis=1, kind="stable")
+    at = lambda a, i: np.take_along_axis(a, order[:, i:i + 1], axis=1)[:, 0]
+    return (at(c, top - 1) - at(c, top)) / (moved * (at(s, top - 1) + at(s, top)) + 1e-300)
 
 
 def moe_ffn(x, w, cfg):
@@ -196,9 +211,10 @@ def run_order(config):
     return order + [(i, None) for i in range(stop, n)]
 
 
-def forward(config, weights, tokens, streams=None, routes=None):
+def forward(config, weights, tokens, streams=None, margins=None):
     """Logits [T, vocab] of one sequence from position 0.  `weights`: {tensor name: float64 array}.
-    `streams`, a list, receives the residual stream after every layer run; `routes` the routing margins of every mixture."""
+    `streams`, a list, receives the residual stream after every layer run; `margins` the tokens' margins at every mixture and
+    every retention."""
     eps, m = config["norm"]["eps"], config["residual_mult"]
     x = weights["embed"][np.asarray(tokens)]
     for i, step in run_order(config):
@@ -206,12 +222,15 @@ def forward(config, weights, tokens, streams=None, routes=None):
         if step is not None:
             x = x + weights["loop.step"][step]
         mix = MIXERS[layer["type"]]
-        x = x + m * mix(rms_norm(x, weights[f"l{i}.norm1"], eps), sub(weights, f"l{i}.mix"), layer["mixer"], eps)
+        h, w = rms_norm(x, weights[f"l{i}.norm1"], eps), sub(weights, f"l{i}.mix")
+        if layer["type"] == "parallel" and margins is not None:
+            margins.append(retention_margin(h, sub(w, "right"), layer["mixer"]["right"]))
+        x = x + m * mix(h, w, layer["mixer"], eps)
         mlp = layer.get("mlp")
         if mlp is not None:
             h, w = rms_norm(x, weights[f"l{i}.norm2"], eps), sub(weights, f"l{i}.mlp")
-            if mlp["kind"] == "moe" and routes is not None:
-                routes.append(route_margin(h, w, mlp))
+            if mlp["kind"] == "moe" and margins is not None:
+                margins.append(route_margin(h, w, mlp))
             x = x + m * (gated_ffn(h, w, relu) if mlp["kind"] == "dense" else moe_ffn(h, w, mlp))
         if streams is not None:
             streams.append(x.copy())
@@ -240,11 +259,27 @@ class PlainSagopel:
         forward(self.cfg, self.tensors, tokens, streams=out)
         return np.stack(out)
 
-    def routing_margins(self, tokens):
-        """The smallest routing margin of every token over the mixtures (None: the model has none)."""
+    def margins(self, tokens):
+        """The smallest margin of every token over the mixtures and retentions (None: the model has none)."""
         out = []
-        forward(self.cfg, self.tensors, tokens, routes=out)
+        forward(self.cfg, self.tensors, tokens, margins=out)
         return np.min(out, axis=0) if out else None
+
+    def decisive(self, tokens, rng, least=40.0, tries=400):
+        """`tokens` with every position that is a close call (a margin below `least`: another choice of experts, or a head of
+        retention that nearly cancels) drawn again, until none is left: no comparison with an engine that rounds then
+        rests on a close call.  (A position's margins depend on the
+        tokens up to it only, so what lies before the first close call stays as it is.)"""
+        tokens = list(tokens)
+        vocab = self.tensors["embed"].shape[0]
+        for _ in range(tries):
+            margins = self.margins(tokens)
+            near = [] if margins is None else np.nonzero(margins < least)[0]
+            if len(near) == 0:
+                return tokens
+            for t in near:
+                tokens[int(t)] = int(rng.integers(0, vocab))
+        raise ValueError("no decisive sequence found")
 
     def greedy(self, prompt, n):
         tokens, out = list(prompt), []

@@ -110,6 +110,28 @@ def test_window_gives_pages_back_when_passed():
     b.check()
 
 
+@pytest.mark.parametrize("keep", [1, 4, 5, 11])
+def test_a_window_may_keep_the_first_tokens(keep):
+    b = PageBook(2, 1000)
+    b.add_group(4, 9, 6, keep)
+    for _ in range(2):                                                           # (the slot and its pages are used again)
+        s = b.acquire_slot()
+        length = 0
+        for n in [3, 5, 1, 1, 1, 7, 2, 1, 1, 1, 1, 9, 2, 8, 1]:
+            b.commit([s], [n])
+            length += n
+            b.retire([s])
+            row = b.table()[s]
+            for blk in range((length + 3) // 4):
+                needed = blk * 4 < keep or (blk + 1) * 4 > max(0, length - 6 + 1)
+                assert (row[blk] >= 0) == needed, (length, blk)
+            assert b.free_pages() == 9 - sum(1 for p in row if p >= 0)
+            b.check()
+        b.release_slot(s)
+        assert b.free_pages() == 9
+        b.check()
+
+
 def test_two_groups_with_different_needs():
     b = PageBook(3, 512)
     full = b.add_group(16, 10, None)
