@@ -48,6 +48,7 @@ HIP_LIBRARIES = {
     "head_mix_attention": (["head_mix_attention.hip"], ["common.h"], True),
     "grouped_gemm": (["grouped_gemm.hip"], ["common.h"], True),
     "attention_tiles": (["attention_tiles.hip"], [], False),      # bfloat16 only by nature
+    "recurrence_chunks": (["recurrence_chunks.hip"], ["common.h"], False),      # likewise
     "sampling": (["sampling.hip"], ["no_alloc.h"], False),
     "library_gemm": (["library_gemm.hip"], [], False, ["-lhipblaslt"]),      # host code around hipBLASLt
 }

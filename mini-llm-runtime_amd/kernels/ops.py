@@ -986,6 +986,53 @@ class Kernels:
                _c_int(1 if activation == "silu" else 0), _p(rope), _p(positions if rope is not None else None), _c_int(rot),
                _stream()), "linear_recurrence")
 
+    CHUNKED_MAX_KEYS = 128        # key channels a head of the recurrence in chunks
+
+    def decayed_chunks_supported(self, q, k, v, n_keys, n_values, rot):
+        """Whether `decayed_recurrence_chunks` takes these operands: the bfloat16 engine, up to 128 key channels a head in
+        multiples of 8, value channels in multiples of 16, a rotation of a multiple of 16 channels, rows and heads that start
+        at multiples of 16 bytes."""
+        return (self.dtype == torch.bfloat16 and n_keys % 8 == 0 and n_keys <= self.CHUNKED_MAX_KEYS and n_values % 16 == 0
+                and rot % 16 == 0 and all(t.stride(0) % 8 == 0 and t.data_ptr() % 16 == 0 for t in (q, k, v)))
+
+    @timed("recurrence", _tensors_work())
+    def decayed_recurrence_chunks(self, q, k, v, log_decay, out, live, stage, state_offset, seg_first, seg_count, segments, slots,
+                                  chunk_first, chunk_count, chunks, chunk, chunk_state, heads, n_keys, n_values,
+                                  heads_per_group=1, q_scale=1.0, write_state=True, activation=None, rope=None, positions=None):
+        """`linear_recurrence` with log_decay float [heads] on the matrix cores, for the many rows of prompt portions: the
+        requests' rows in `chunks` chunks of at most `chunk` tokens (a multiple of 64; a request's chunks one after the
+        other, the requests in the order of seg_first), `chunk_state` float [chunks * heads * n_keys * n_values] their
+        states.  The result differs from the token-by-token order by 32-bit rounding."""
+        rows = v.shape[0]
+        groups = heads // heads_per_group
+        _need(heads >= 1 and heads_per_group >= 1 and heads % heads_per_group == 0, "decayed_recurrence_chunks: heads and groups")
+        rot = self._turn_table(rope, positions, rows, n_keys)
+        qs = self._columns(q, "q", self.dtype, rows, groups * n_keys)
+        ks = self._columns(k, "k", self.dtype, rows, groups * n_keys)
+        vs = self._columns(v, "v", self.dtype, rows, heads * n_values)
+        _need(self.decayed_chunks_supported(q, k, v, n_keys, n_values, rot), "decayed_recurrence_chunks: sizes that the kernel does not take")
+        _need(activation in (None, "silu"), f"decayed_recurrence_chunks: activation {activation!r}")
+        _need(chunk >= 64 and chunk % 64 == 0 and segments * heads <= 65535, "decayed_recurrence_chunks: chunks in multiples of 64 tokens, "
+              "and no more requests and heads than the grid takes")
+        _tensor(log_decay, "log_decay", torch.float32, (heads,))
+        _tensor(out, "out", torch.float32, (rows, heads * n_values))
+        self._check_state(live, stage, state_offset, heads * n_keys * n_values)
+        for name, t, n in (("seg_first", seg_first, segments), ("seg_count", seg_count, segments), ("chunk_first", chunk_first, chunks),
+                           ("chunk_count", chunk_count, chunks)):
+            _tensor(t, name, torch.int32, (n,))
+        _tensor(slots, "slots", torch.int32, (rows,))
+        _tensor(chunk_state, "chunk_state", torch.float32, ndim=1)
+        _need(chunk_state.numel() >= chunks * heads * n_keys * n_values and chunk_state.data_ptr() % 16 == 0,
+              "decayed_recurrence_chunks: the states' buffer is too small")
+        at = state_offset * 4
+        _ok(self._lib("recurrence_chunks").mlr_decayed_recurrence_chunks(
+            _p(q), ctypes.c_long(qs), _p(k), ctypes.c_long(ks), _p(v), ctypes.c_long(vs), _p(log_decay), _c_float(q_scale),
+            _c_int(1 if activation == "silu" else 0), _p(rope), _p(positions if rope is not None else None), _c_int(rot), _p(out),
+            _ptr(live.data_ptr() + at), _ptr(stage.data_ptr() + at), ctypes.c_long(live.stride(0)), _p(slots), _p(seg_first),
+            _p(seg_count), _c_int(segments), _p(chunk_first), _p(chunk_count), _c_int(chunks), _c_int(chunk), _p(chunk_state),
+            _c_int(heads), _c_int(heads_per_group), _c_int(n_keys), _c_int(n_values), _c_int(1 if write_state else 0), _stream()),
+            "decayed_recurrence_chunks")
+
     def _turn_table(self, rope, positions, rows, n_keys):
         """The width of a rotation table for heads of `n_keys` channels (0: none given), checked with the positions."""
         if rope is None:

@@ -20,8 +20,9 @@ PIECE = 128              # tokens of a piece when a step's portions run in piece
 PIECES_FROM = 512        # rows of a step from which they do (the bfloat16 engine)
 PIECE_FLOATS = 64 << 20  # floats that the pieces' states may take; a step with more runs token by token
 DELTA_CHUNK = 32         # tokens of a chunk of the delta rule (the kernel's `delta_chunk_tokens()`)
-CHUNKS_FROM = 64         # rows of a step from which the delta rule runs in chunks (the bfloat16 engine), where the
-                         # step's requests bring eight tokens each or more (single tokens stay with the walk)
+CHUNKS_FROM = 64         # rows of a step from which the delta rule, and the recurrence with a constant decay, run in chunks
+                         # (the bfloat16 engine), where the step's requests bring eight tokens each or more (single tokens
+                         # stay with the walk)
 
 
 def _requests(ctx):
@@ -258,14 +259,28 @@ class DecayedLinearAttention:
         return StateSpec((s.heads * s.head_dim * s.value_dim,), torch.float32)
 
     def libraries(self):
-        return ["gemm", "recurrence", "elementwise"]
+        chunks = ["recurrence_chunks"] if self.proj is not None and self.proj.dtype == torch.bfloat16 else []
+        return ["gemm", "recurrence", "elementwise"] + chunks
+
+    def _chunks_plan(self, rows, dtype, limits):
+        """Scratch memory of the recurrence in chunks for a step of at most `rows` tokens: every request of the step may add
+        a ragged chunk."""
+        state = self.spec.heads * self.spec.head_dim * self.spec.value_dim
+        plan = _pieces_plan(rows, state, self.spec.heads, self.spec.head_dim)
+        if dtype != torch.bfloat16 or rows < CHUNKS_FROM:
+            return plan
+        chunks = rows // PIECE + min(rows // 8, int((limits or {}).get("max_slots") or rows))
+        for key, count in ((("recurrent_pieces", torch.float32), min(chunks, max(1, PIECE_FLOATS // state)) * state),
+                           ((f"token_groups_{PIECE}_0", torch.int32), 2 * chunks + 2)):
+            plan[key] = max(plan.get(key, 0), count)
+        return plan
 
     def workspace_plan(self, rows, dtype, limits):
         s = self.spec
         return {("decayed_proj", dtype): rows * (2 * self.qk_width + 2 * self.v_width),
                 ("recurrent_out", torch.float32): rows * self.v_width, ("recurrent_normed", dtype): rows * self.v_width,
                 (self.out_name, dtype): rows * s.hidden, (f"token_groups_{WHOLE}_0", torch.int32): 2 * rows + 2,
-                **_pieces_plan(rows, s.heads * s.head_dim * s.value_dim, s.heads, s.head_dim)}
+                **self._chunks_plan(rows, dtype, limits)}
 
     def forward(self, ctx, x, cache_id, write_cache=True):
         s = self.spec
@@ -277,10 +292,22 @@ class DecayedLinearAttention:
         a, b = self.qk_width, 2 * self.qk_width
         c = b + self.v_width
         o = ws.get("recurrent_out", (m, self.v_width), torch.float32)
-        _recurrence(ctx, s.heads * s.head_dim * s.value_dim, s.heads, s.head_dim,
-                    proj[:, :a], proj[:, a:b], proj[:, b:c], self._log_decay, o, ctx.cache.state_view(cache_id),
-                    ctx.cache.state_stage(cache_id), 0, ctx.slots, s.heads, s.head_dim, s.value_dim,
-                    q_scale=float(s.k_scale), write_state=write_cache, activation=s.activation, **self._turns(ctx, x.device))
+        q, kk, v = proj[:, :a], proj[:, a:b], proj[:, b:c]
+        live, stage = ctx.cache.state_view(cache_id), ctx.cache.state_stage(cache_id)
+        turns = self._turns(ctx, x.device)
+        more = dict(q_scale=float(s.k_scale), write_state=write_cache, activation=s.activation, **turns)
+        state = s.heads * s.head_dim * s.value_dim
+        if m >= max(CHUNKS_FROM, 8 * len(ctx.segments)) and (m // PIECE + len(ctx.segments)) * state <= PIECE_FLOATS and \
+                len(ctx.segments) * s.heads <= 65535 and \
+                k.decayed_chunks_supported(q, kk, v, s.head_dim, s.value_dim, turns["rope"].shape[1] if turns else 0):
+            first, count, n = _requests(ctx)
+            (c_first, c_count, c_n), _, _ = ctx.token_groups(PIECE, 0)
+            k.decayed_recurrence_chunks(q, kk, v, self._log_decay, o, live, stage, 0, first, count, n, ctx.slots, c_first, c_count, c_n,
+                                        PIECE, ws.get("recurrent_pieces", (c_n * state,), torch.float32), s.heads, s.head_dim,
+                                        s.value_dim, **more)
+        else:
+            _recurrence(ctx, state, s.heads, s.head_dim, q, kk, v, self._log_decay, o, live, stage, 0, ctx.slots, s.heads, s.head_dim,
+                        s.value_dim, **more)
         y = ws.get("recurrent_normed", (m, self.v_width), x.dtype)
         k.gated_part_norm(o, proj[:, c:], self.norm, y, self.v_width if s.norm == "row" else s.value_dim, float(s.eps),
                           gate_first=False, gate_kind=s.gate)

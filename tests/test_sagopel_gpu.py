@@ -339,6 +339,33 @@ def test_the_recurrence_turns_its_queries_and_keys(dtype_name, silu, heads, keys
         check_recurrence(case, out, stage, 6e-5)
 
 
+@pytest.mark.parametrize("silu", [False, True])
+@pytest.mark.parametrize("heads,keys,values,rot", [(3, 24, 48, 16), (2, 128, 128, 128), (4, 64, 32, 0), (1, 8, 16, 0), (5, 96, 144, 64), (2, 40, 272, 32),
+                                                   (6, 48, 80, 48), (1, 112, 64, 112), (2, 16, 16, 16)])
+def test_the_recurrence_in_chunks_on_the_matrix_cores(silu, heads, keys, values, rot):
+    """Requests shorter and longer than a chunk, ends around blocks of 64 rows, single tokens between them, from states that
+    are not zero; decays from none at all to 0.03 a token.  What differs from 32-bit arithmetic is rounding, not bfloat16."""
+    from mini_llm_runtime_amd.kernels import Kernels
+    k = Kernels(torch.bfloat16)
+    for chunk, lengths in ((128, [37, 1, 128, 300, 64, 2, 129, 65]), (64, [200, 63, 1]), (192, [1, 500, 192])):
+        case = recurrence_case(k, torch.bfloat16, heads, keys, values, rot, silu, lengths, seed=keys + values + chunk)
+        args = case["args"]
+        if args[0].stride(0) % 8:                                      # (rows that start at multiples of 16 bytes)
+            wide = torch.zeros((case["n"], -(-args[0].stride(0) // 8) * 8), dtype=torch.bfloat16, device="cuda")
+            a, b, c = heads * keys, 2 * heads * keys, 2 * heads * keys + heads * values
+            for lo, hi, t in ((0, a, args[0]), (a, b, args[1]), (b, c, args[2])):
+                wide[:, lo:hi] = t
+            args = (wide[:, :a], wide[:, a:b], wide[:, b:c], args[3])
+        cut = [(f + i, min(chunk, n - i)) for f, n in zip(case["first"], case["count"]) for i in range(0, n, chunk)]
+        out = torch.full((case["n"], heads * values), float("nan"), device="cuda")
+        stage = torch.full_like(case["live"], float("nan"))
+        scratch = torch.full((len(cut) * heads * keys * values,), float("nan"), device="cuda")
+        k.decayed_recurrence_chunks(*args, out, case["live"], stage, 0, ints(case["first"]), ints(case["count"]), len(lengths), case["slots"],
+                                    ints([f for f, _ in cut]), ints([n for _, n in cut]), len(cut), chunk, scratch, heads, keys, values,
+                                    **case["more"])
+        check_recurrence(case, out, stage, 6e-5 if rot else 1e-5)      # (an angle near 1000 carries 32-bit rounding of 6e-5)
+
+
 def paged(x, page, dtype, seed=0):
     """[T, G, D] of ONE request in row-major pages that lie in a shuffled order, NaN where nothing was written; (pages, block
     table [1, blocks])."""
