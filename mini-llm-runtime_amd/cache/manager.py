@@ -368,6 +368,11 @@ class CacheManager:
             if isinstance(spec, StateSpec):
                 self._states[cid] = torch.zeros((max_slots + 1, *spec.shape), dtype=spec.dtype, device=self.device)
                 self._staged[cid] = torch.zeros_like(self._states[cid])
+        self._state_rows = [t[0].numel() * t.element_size() for t in self._states.values()]
+        self._state_entries = None       # device int64 [entries, 3]: both slabs' addresses and the bytes of a row
+        if self._states and self.device.type == "cuda":
+            self._state_entries = torch.tensor([[live.data_ptr(), self._staged[cid].data_ptr(), size] for (cid, live), size
+                                                in zip(self._states.items(), self._state_rows)], dtype=torch.int64, device=self.device)
 
     # -- views for the parts ---------------------------------------------------------------------
     def paged_view(self, cache_id):
@@ -397,10 +402,13 @@ class CacheManager:
     def has_state(self):
         return bool(self._states)
 
-    def commit_state(self, segment_slots):
+    def commit_state(self, segment_slots, kernels=None):
         """The staged rows of the step's requests (`segment_slots`: device integer vector, one slot per
-        entry of the batch) become live.  Device work only, so a captured step holds it.  The scratch
-        request's state starts every step at zero."""
+        entry of the batch) become live, in one launch of `kernels` for all entries.  Device work only, so a
+        captured step holds it.  The scratch request's state starts every step at zero."""
+        if kernels is not None and self._state_entries is not None and segment_slots.dtype == torch.int32:
+            kernels.state_commit(self._state_entries, max(self._state_rows), segment_slots, self.max_slots)
+            return
         index = segment_slots.long()
         for cid, live in self._states.items():
             live.index_copy_(0, index, self._staged[cid].index_select(0, index))

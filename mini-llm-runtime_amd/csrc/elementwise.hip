@@ -1020,6 +1020,30 @@ static int launch_gated(const void* gate_up, void* act, int rows, int inter, hip
     return (int)hipGetLastError();
 }
 
+// The staged state of a step's requests becomes live, every entry's in one launch: row slots[s] of the entry's live slab
+// takes the staged row (zeros for the scratch request).  entries[3 e]: the live slab, the staged slab, bytes a row.  One
+// workgroup moves COMMIT_BYTES of a row; rows of a multiple of 16 bytes in 16-byte accesses.
+#define COMMIT_BYTES 16384
+__global__ __launch_bounds__(256) void state_commit_kernel(const int64_t* __restrict__ entries, const int32_t* __restrict__ slots,
+                                                           int scratch_slot) {
+    const int64_t* entry = entries + 3 * blockIdx.z;
+    const int64_t row = entry[2], from = (int64_t)blockIdx.x * COMMIT_BYTES, to = min(from + COMMIT_BYTES, row);
+    const int slot = slots[blockIdx.y];
+    char* live = reinterpret_cast<char*>(entry[0]) + slot * row;
+    const char* stage = reinterpret_cast<const char*>(entry[1]) + slot * row;
+    const bool clear = slot == scratch_slot;
+    if (row % 16 == 0) {
+        const vec16 zero = {{0, 0, 0, 0}};
+#pragma unroll
+        for (int i = 0; i < COMMIT_BYTES / (256 * 16); ++i) {
+            const int64_t at = from + (i * 256 + threadIdx.x) * 16;
+            if (at < to) *reinterpret_cast<vec16*>(live + at) = clear ? zero : *reinterpret_cast<const vec16*>(stage + at);
+        }
+        return;
+    }
+    for (int64_t at = from + threadIdx.x; at < to; at += 256) live[at] = clear ? 0 : stage[at];
+}
+
 // Whether every pointer given (null ones aside) allows 16-byte accesses.
 template <class... P> static bool aligned16(P... pointers) {
     return (((uintptr_t)pointers % 16 == 0) && ...);
@@ -1133,6 +1157,15 @@ int mlr_rmsnorm_columns(const void* x, long x_stride, const float* weight, void*
 int mlr_scaled_sum(const void* a, const void* b, void* out, float sa, float sb, size_t count, hipStream_t stream) {
     if (count == 0) return 0;
     scaled_sum_kernel<<<grid_for(count, 256), 256, 0, stream>>>((const elem_t*)a, (const elem_t*)b, (elem_t*)out, sa, sb, count);
+    return (int)hipGetLastError();
+}
+
+int mlr_state_commit(const int64_t* entries, int n_entries, long long most_bytes, const int32_t* slots, int n_slots,
+                     int scratch_slot, hipStream_t stream) {
+    if (n_entries <= 0 || n_slots <= 0 || most_bytes <= 0) return 0;
+    if (n_entries > 65535 || n_slots > 65535) return -1;
+    const unsigned parts = (unsigned)((most_bytes + COMMIT_BYTES - 1) / COMMIT_BYTES);
+    state_commit_kernel<<<dim3(parts, n_slots, n_entries), 256, 0, stream>>>(entries, slots, scratch_slot);
     return (int)hipGetLastError();
 }
 

@@ -11,7 +11,7 @@
 // 32-bit operands on matrix cores that multiply bfloat16: an operand is the sum of three bfloat16 numbers of 8 significant
 // bits each, which holds a 32-bit number's 24 bits whole; a product is the six (or three, where the other operand is
 // bfloat16 as it comes) products of parts whose orders add up to less than three, summed in 32-bit: what is left out lies
-// below 2^-24 of the product.  Decays, activations and rotations are 32-bit too.
+// below 2^-22 of the product.  Decays, activations and rotations are 32-bit too.
 #define MLR_BF16 1
 #include "common.h"
 
@@ -42,7 +42,9 @@ struct ChunkArgs {
     float q_scale;
 };
 
-__device__ __forceinline__ float silu_of(float x) { return x / (1.0f + expf(-x)); }
+#define LOG2E 1.4426950408889634f
+// (the exponential and reciprocal instructions: 32-bit, each within a unit of the last place or so)
+__device__ __forceinline__ float silu_of(float x) { return x * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-LOG2E * x)); }
 
 // Eight channels of a row from channel `ch` on, through the activation and the rotation (pairs (i, i + rot_dim / 2)).
 __device__ __forceinline__ void row_channels(const ChunkArgs& a, const __bf16* head_row, size_t row, int ch, float (&x)[8]) {
@@ -70,18 +72,25 @@ __device__ __forceinline__ void row_channels(const ChunkArgs& a, const __bf16* h
     }
 }
 
-// x as the sum of bfloat16 numbers, part[0] + part[1] + part[2] (the last two only where asked for).
+// x as a sum of bfloat16 numbers: a part is the upper half of what the parts before it leave (cut off, so each holds the
+// next eight significant bits); P 1: x holds bfloat16 numbers.
 template <int P> __device__ __forceinline__ void parts_of(const float (&x)[8], bf16x8 (&part)[P]) {
+    u32x4 w[P];
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-        float rest = x[e];
+    for (int c = 0; c < 4; ++c) {
+        float lo = x[2 * c], hi = x[2 * c + 1];
 #pragma unroll
         for (int p = 0; p < P; ++p) {
-            const __bf16 b = (__bf16)rest;
-            part[p][e] = b;
-            rest -= (float)b;
+            const uint32_t a = __float_as_uint(lo), b = __float_as_uint(hi);
+            w[p][c] = __builtin_amdgcn_perm(b, a, 0x07060302u);          // the upper halves of both
+            if (p + 1 < P) {
+                lo -= __uint_as_float(a & 0xffff0000u);
+                hi -= __uint_as_float(b & 0xffff0000u);
+            }
         }
     }
+#pragma unroll
+    for (int p = 0; p < P; ++p) part[p] = __builtin_bit_cast(bf16x8, w[p]);
 }
 
 // Eight channels of one token into [part][channel][TP]: the lane beside holds the token beside, so a lane takes the other's
@@ -130,7 +139,7 @@ __global__ __launch_bounds__(THREADS) void chunk_write_kernel(ChunkArgs a) {
     const int first = a.chunk_first[chunk], count = a.chunk_count[chunk];
     const int v_cols = min(VB, V - v0), vt = v_cols >> 4;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, i16 = lane & 15, b = lane >> 4;
-    const float lam = a.log_decay[head];
+    const float lam = a.log_decay[head] * LOG2E;
     const int shares = 8 / nt, my_nt = wave % nt, share = wave / nt;
     floatx4 acc[8];
 #pragma unroll
@@ -143,7 +152,7 @@ __global__ __launch_bounds__(THREADS) void chunk_write_kernel(ChunkArgs a) {
             if (t0 + token < count && ch < N) {
                 const size_t row = (size_t)(first + t0 + token);
                 row_channels(a, a.k + row * a.k_stride + (head / a.heads_per_group) * N, row, ch, x);
-                const float f = expf(lam * (float)(count - 1 - t0 - token));
+                const float f = __builtin_amdgcn_exp2f(lam * (float)(count - 1 - t0 - token));
 #pragma unroll
                 for (int e = 0; e < 8; ++e) x[e] *= f;
             }
@@ -200,7 +209,7 @@ __global__ __launch_bounds__(256) void chunk_states_kernel(ChunkArgs a) {
     const size_t at = (size_t)slot * a.state_stride + ((size_t)head * a.N + n) * a.V + v;
     const size_t per = (size_t)a.heads * a.N * a.V;
     float* p = a.chunk_state + (size_t)chunk0 * per + ((size_t)head * a.V + v) * a.N + n;
-    const float lam = a.log_decay[head];
+    const float lam = a.log_decay[head] * LOG2E;
     float S = a.live[at];
     for (int c0 = 0; c0 < chunks; c0 += STATE_AHEAD) {
         float add[STATE_AHEAD];
@@ -210,7 +219,7 @@ __global__ __launch_bounds__(256) void chunk_states_kernel(ChunkArgs a) {
         for (int i = 0; i < STATE_AHEAD; ++i) {
             if (c0 + i < chunks) {
                 p[(size_t)(c0 + i) * per] = S;
-                S = expf(lam * (float)a.chunk_count[chunk0 + c0 + i]) * S + add[i];
+                S = __builtin_amdgcn_exp2f(lam * (float)a.chunk_count[chunk0 + c0 + i]) * S + add[i];
             }
         }
     }
@@ -235,7 +244,7 @@ __global__ __launch_bounds__(THREADS) void chunk_read_kernel(ChunkArgs a, int bl
     const int rows = min(BT, count - block * BT);
     const int v_cols = min(VB, V - v0), vt = v_cols >> 4;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, i16 = lane & 15, b = lane >> 4;
-    const float lam = a.log_decay[head];
+    const float lam = a.log_decay[head] * LOG2E;
     const int qk_head = head / a.heads_per_group;
     // this wavefront's value channels and rows: with few value channels several wavefronts share 16 of them and deal the rows out
     const int shares = vt > 4 ? 1 : vt > 2 ? 2 : 4, my_vt = wave / shares, share = wave % shares, tiles = 4 / shares;
@@ -254,9 +263,9 @@ __global__ __launch_bounds__(THREADS) void chunk_read_kernel(ChunkArgs a, int bl
     }
     // 64 rows of q or k into [part][row][pitch], zeros past the rows there are and past the key channels
     auto put_rows = [&](const __bf16* base, long stride, int row0, int present, float factor, __bf16* dst) {
-        const int per = n_steps * 4;                                    // eight-channel pieces of a row
-        for (int i = tid; i < BT * per; i += THREADS) {
-            const int r = i / per, ch = (i % per) * 8;
+        for (int i = tid; i < BT * (MAX_CHUNK_KEYS / 8); i += THREADS) {
+            const int r = i / (MAX_CHUNK_KEYS / 8), ch = (i % (MAX_CHUNK_KEYS / 8)) * 8;
+            if (ch >= n_steps * 32) continue;
             float x[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
             if (r < present && ch < N) {
                 const size_t row = (size_t)(row0 + r);
@@ -294,7 +303,7 @@ __global__ __launch_bounds__(THREADS) void chunk_read_kernel(ChunkArgs a, int bl
         }
 #pragma unroll
         for (int j = 0; j < 4; ++j)
-            if (j < tiles) acc[j] *= expf(lam * (float)(block * BT + (share + shares * j) * 16 + i16 + 1));
+            if (j < tiles) acc[j] *= __builtin_amdgcn_exp2f(lam * (float)(block * BT + (share + shares * j) * 16 + i16 + 1));
     }
     const int row_tile = wave & 3, key_half = wave >> 2;                 // of the scores
     const int key_row = key_half * 32 + 8 * (i16 >> 2) + (i16 & 3);      // (and key_row + 4)
@@ -332,7 +341,7 @@ __global__ __launch_bounds__(THREADS) void chunk_read_kernel(ChunkArgs a, int bl
 #pragma unroll
             for (int e = 0; e < 8; ++e) {
                 const float s = e < 4 ? s_lo[e] : s_hi[e - 4];
-                w[e] = behind - e >= 0 ? s * expf(lam * (float)(behind - e)) : 0.f;
+                w[e] = behind - e >= 0 ? s * __builtin_amdgcn_exp2f(lam * (float)(behind - e)) : 0.f;
             }
             bf16x8 part[PARTS];
             parts_of<PARTS>(w, part);

@@ -866,6 +866,17 @@ class Kernels:
                _stream()), "gated_part_norm")
 
     # -- mixers with a state of fixed size ------------------------------------------------------------
+    @timed("state")
+    def state_commit(self, entries, row_bytes, slots, scratch_slot):
+        """Row slots[s] of every entry's live slab takes the staged slab's row (zeros where it is `scratch_slot`).  entries:
+        int64 [n, 3] on the device, the addresses of an entry's two slabs and the bytes of a row; row_bytes: the most of
+        those."""
+        _tensor(entries, "entries", torch.int64, ndim=2)
+        _tensor(slots, "slots", torch.int32, ndim=1)
+        _need(entries.shape[1] == 3 and entries.shape[0] <= 65535 and slots.numel() <= 65535, "state_commit: too many entries or requests")
+        _ok(self._lib("elementwise").mlr_state_commit(_p(entries), _c_int(entries.shape[0]), ctypes.c_longlong(row_bytes), _p(slots),
+                                                      _c_int(slots.numel()), _c_int(scratch_slot), _stream()), "state_commit")
+
     CONV_MAX_TAPS = 8
     RECURRENCE_MAX_KEYS = 256
 

@@ -228,7 +228,7 @@ class DecoderModel:
                 else:
                     k.finite_check(h, None if isinstance(pending, Complete) else pending, i, status)
         if ctx.cache is not None and ctx.cache.has_state():
-            ctx.cache.commit_state(ctx.segment_slots)     # every layer has run: the staged state becomes live
+            ctx.cache.commit_state(ctx.segment_slots, k)     # every layer has run: the staged state becomes live
         r = 0 if want_rows is None else want_rows.numel()
         if r == 0:
             return None

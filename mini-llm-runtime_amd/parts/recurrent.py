@@ -20,9 +20,9 @@ PIECE = 128              # tokens of a piece when a step's portions run in piece
 PIECES_FROM = 512        # rows of a step from which they do (the bfloat16 engine)
 PIECE_FLOATS = 64 << 20  # floats that the pieces' states may take; a step with more runs token by token
 DELTA_CHUNK = 32         # tokens of a chunk of the delta rule (the kernel's `delta_chunk_tokens()`)
-CHUNKS_FROM = 64         # rows of a step from which the delta rule, and the recurrence with a constant decay, run in chunks
-                         # (the bfloat16 engine), where the step's requests bring eight tokens each or more (single tokens
-                         # stay with the walk)
+CHUNKS_FROM = 64         # rows of a step from which the delta rule runs in chunks (the bfloat16 engine), where the
+                         # step's requests bring eight tokens each or more (single tokens stay with the walk)
+SHORT = 32               # rows up to which a request's constant-decay recurrence stays with the walk (longer ones in chunks)
 
 
 def _requests(ctx):
@@ -267,11 +267,12 @@ class DecayedLinearAttention:
         a ragged chunk."""
         state = self.spec.heads * self.spec.head_dim * self.spec.value_dim
         plan = _pieces_plan(rows, state, self.spec.heads, self.spec.head_dim)
-        if dtype != torch.bfloat16 or rows < CHUNKS_FROM:
+        if dtype != torch.bfloat16 or rows <= SHORT:
             return plan
-        chunks = rows // PIECE + min(rows // 8, int((limits or {}).get("max_slots") or rows))
+        chunks = rows // PIECE + min(rows // (SHORT + 1), int((limits or {}).get("max_slots") or rows))
         for key, count in ((("recurrent_pieces", torch.float32), min(chunks, max(1, PIECE_FLOATS // state)) * state),
-                           ((f"token_groups_{PIECE}_0", torch.int32), 2 * chunks + 2)):
+                           ((f"token_groups_{SHORT}_{PIECE // SHORT}", torch.int32), 2 * rows + 2),
+                           ((f"token_groups_{SHORT}_{WHOLE // SHORT}", torch.int32), 2 * rows + 2)):
             plan[key] = max(plan.get(key, 0), count)
         return plan
 
@@ -297,14 +298,17 @@ class DecayedLinearAttention:
         turns = self._turns(ctx, x.device)
         more = dict(q_scale=float(s.k_scale), write_state=write_cache, activation=s.activation, **turns)
         state = s.heads * s.head_dim * s.value_dim
-        if m >= max(CHUNKS_FROM, 8 * len(ctx.segments)) and (m // PIECE + len(ctx.segments)) * state <= PIECE_FLOATS and \
-                len(ctx.segments) * s.heads <= 65535 and \
+        if m > SHORT and (m // PIECE + m // (SHORT + 1)) * state <= PIECE_FLOATS and len(ctx.segments) * s.heads <= 65535 and \
                 k.decayed_chunks_supported(q, kk, v, s.head_dim, s.value_dim, turns["rope"].shape[1] if turns else 0):
-            first, count, n = _requests(ctx)
-            (c_first, c_count, c_n), _, _ = ctx.token_groups(PIECE, 0)
-            k.decayed_recurrence_chunks(q, kk, v, self._log_decay, o, live, stage, 0, first, count, n, ctx.slots, c_first, c_count, c_n,
-                                        PIECE, ws.get("recurrent_pieces", (c_n * state,), torch.float32), s.heads, s.head_dim,
-                                        s.value_dim, **more)
+            # long portions in chunks on the matrix cores, single tokens and short portions of the same step by the walk
+            few, (c_first, c_count, c_n), _ = ctx.token_groups(SHORT, PIECE // SHORT)
+            _, (first, count, n), _ = ctx.token_groups(SHORT, WHOLE // SHORT)
+            if n:
+                k.decayed_recurrence_chunks(q, kk, v, self._log_decay, o, live, stage, 0, first, count, n, ctx.slots, c_first, c_count,
+                                            c_n, PIECE, ws.get("recurrent_pieces", (c_n * state,), torch.float32), s.heads,
+                                            s.head_dim, s.value_dim, **more)
+            if few[2]:
+                k.linear_recurrence(q, kk, v, self._log_decay, o, live, stage, 0, *few, ctx.slots, s.heads, s.head_dim, s.value_dim, **more)
         else:
             _recurrence(ctx, state, s.heads, s.head_dim, q, kk, v, self._log_decay, o, live, stage, 0, ctx.slots, s.heads, s.head_dim,
                         s.value_dim, **more)

@@ -532,6 +532,28 @@ def test_experts_that_give_their_input_back(dtype_name, rows, experts, identity,
     assert identity == 0 or (ids >= experts).any()
 
 
+@pytest.mark.parametrize("shapes", [[(5,)], [(3, 8), (4096,), (7,), (4100,)], [(1,), (9000,)]])
+def test_staged_states_become_live_in_one_launch(shapes):
+    from mini_llm_runtime_amd.cache import CacheManager, StateSpec
+    from mini_llm_runtime_amd.kernels import Kernels
+    k = Kernels(torch.float32)
+    specs = [StateSpec(shape, torch.int32 if i == 2 else torch.float32) for i, shape in enumerate(shapes)]
+    cache = CacheManager(specs, torch.float32, "cuda", 8, 64, 5, 64)
+    g = torch.Generator().manual_seed(3)
+    for slots in ([3], [0, 4, 2], [1, 5, 0]):                          # (the last holds the scratch request)
+        want = {}
+        for cid in cache._states:
+            for t in (cache._states[cid], cache._staged[cid]):
+                t.copy_(torch.randint(-1000, 1000, t.shape, generator=g).to(t.dtype))
+            want[cid] = cache._states[cid].clone()
+            want[cid][slots] = cache._staged[cid][slots]
+            if 5 in slots:
+                want[cid][5] = 0
+        cache.commit_state(ints(slots), k)
+        for cid in want:
+            assert torch.equal(cache._states[cid], want[cid])
+
+
 # ---- one mechanism a model ----------------------------------------------------------------------------------------
 ALONE = dict(heads=1, dim=2, vdim=2, decay=[0.5], rot=dict(dims=2, base=10.0))
 ONE_LAYER = {
