@@ -367,38 +367,89 @@ __global__ void scaled_sum_kernel(const elem_t* __restrict__ a, const elem_t* __
         out[i] = from_float<elem_t>(sa * to_float(a[i]) + sb * to_float(b[i]));
 }
 
+// VEC weights from channel c on, ones without any (16-byte accesses where VEC is more than one).
+template <int VEC> __device__ __forceinline__ void row_weights(const float* w, int c, float* out) {
+    if (w == nullptr) {
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) out[e] = 1.f;
+    } else if (VEC > 1) {
+#pragma unroll
+        for (int e = 0; e < VEC; e += 4) *reinterpret_cast<float4*>(out + e) = *reinterpret_cast<const float4*>(w + c + e);
+    } else {
+        out[0] = w[c];
+    }
+}
+
 // out[m] = sa * norm(a[m]) + sb * norm(b[m]): two sublayers' rows, each over its own root mean square times a weight as wide
-// as the row (a null weight: the row as it is, not normed), added in 32-bit.  One workgroup a row; VEC: MLR_VEC values in
-// one access, or 1.
+// as the row (a null weight: the row as it is, not normed), added in 32-bit.  One workgroup a row, which it keeps in
+// registers up to 256 * VEC * SUM_CHUNKS values (wider rows are read again); VEC: MLR_VEC values in one access, or 1.
+#define SUM_CHUNKS 4
 template <int VEC>
-__global__ __launch_bounds__(256) void normed_sum_kernel(const elem_t* __restrict__ a, const elem_t* __restrict__ b,
-                                                         const float* __restrict__ wa, const float* __restrict__ wb,
-                                                         elem_t* __restrict__ out, float sa, float sb, int width, float eps) {
-    __shared__ float scratch[16];
+__global__ __launch_bounds__(256) void normed_sum_kernel(const elem_t* a, const elem_t* b, const float* __restrict__ wa,
+                                                         const float* __restrict__ wb, elem_t* out, float sa, float sb, int width,
+                                                         float eps) {
+    __shared__ float scratch[8];
     const elem_t* arow = a + (size_t)blockIdx.x * width;
     const elem_t* brow = b + (size_t)blockIdx.x * width;
-    float suma = 0.f, sumb = 0.f;
-    for (int c = threadIdx.x * VEC; c < width; c += 256 * VEC) {
-        float x[MLR_VEC], y[MLR_VEC];
-        if (VEC > 1) { load_vec(arow + c, x); load_vec(brow + c, y); }
-        else { x[0] = to_float(arow[c]); y[0] = to_float(brow[c]); }
-#pragma unroll
-        for (int e = 0; e < VEC; ++e) { suma += x[e] * x[e]; sumb += y[e] * y[e]; }
-    }
-    suma = block_sum(suma, scratch);
-    sumb = block_sum(sumb, scratch);
-    const float fa = wa ? sa / sqrtf(suma / (float)width + eps) : sa, fb = wb ? sb / sqrtf(sumb / (float)width + eps) : sb;
     elem_t* orow = out + (size_t)blockIdx.x * width;
-    for (int c = threadIdx.x * VEC; c < width; c += 256 * VEC) {
-        float x[MLR_VEC], y[MLR_VEC];
-        if (VEC > 1) { load_vec(arow + c, x); load_vec(brow + c, y); }
-        else { x[0] = to_float(arow[c]); y[0] = to_float(brow[c]); }
+    auto read = [&](int c, float* x, float* y) {
+        if (VEC > 1) {
+            load_vec(arow + c, x);
+            load_vec(brow + c, y);
+        } else {
+            x[0] = to_float(arow[c]);
+            y[0] = to_float(brow[c]);
+        }
+    };
+    float x[SUM_CHUNKS][MLR_VEC], y[SUM_CHUNKS][MLR_VEC];
+    float suma = 0.f, sumb = 0.f;
+    const bool kept = width <= 256 * VEC * SUM_CHUNKS;
 #pragma unroll
-        for (int e = 0; e < VEC; ++e)
-            x[e] = (x[e] * fa) * (wa ? wa[c + e] : 1.f) + (y[e] * fb) * (wb ? wb[c + e] : 1.f);
-        if (VEC > 1) store_vec(orow + c, x);
-        else orow[c] = from_float<elem_t>(x[0]);
+    for (int i = 0; i < SUM_CHUNKS; ++i) {
+        const int c = (threadIdx.x + 256 * i) * VEC;
+        if (c < width) {
+            read(c, x[i], y[i]);
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) { suma += x[i][e] * x[i][e]; sumb += y[i][e] * y[i][e]; }
+        }
     }
+    if (!kept)
+        for (int c = (threadIdx.x + 256 * SUM_CHUNKS) * VEC; c < width; c += 256 * VEC) {
+            float u[MLR_VEC], v[MLR_VEC];
+            read(c, u, v);
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) { suma += u[e] * u[e]; sumb += v[e] * v[e]; }
+        }
+    suma = wave_sum(suma);
+    sumb = wave_sum(sumb);
+    if ((threadIdx.x & 63) == 0) {
+        scratch[threadIdx.x >> 6] = suma;
+        scratch[4 + (threadIdx.x >> 6)] = sumb;
+    }
+    __syncthreads();
+    suma = (scratch[0] + scratch[1]) + (scratch[2] + scratch[3]);
+    sumb = (scratch[4] + scratch[5]) + (scratch[6] + scratch[7]);
+    const float fa = wa ? sa / sqrtf(suma / (float)width + eps) : sa, fb = wb ? sb / sqrtf(sumb / (float)width + eps) : sb;
+    auto write = [&](int c, const float* u, const float* v) {
+        float o[MLR_VEC], fw[MLR_VEC], gw[MLR_VEC];
+        row_weights<VEC>(wa, c, fw);
+        row_weights<VEC>(wb, c, gw);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) o[e] = (u[e] * fa) * fw[e] + (v[e] * fb) * gw[e];
+        if (VEC > 1) store_vec(orow + c, o);
+        else orow[c] = from_float<elem_t>(o[0]);
+    };
+#pragma unroll
+    for (int i = 0; i < SUM_CHUNKS; ++i) {
+        const int c = (threadIdx.x + 256 * i) * VEC;
+        if (c < width) write(c, x[i], y[i]);
+    }
+    if (!kept)
+        for (int c = (threadIdx.x + 256 * SUM_CHUNKS) * VEC; c < width; c += 256 * VEC) {      // (this thread's own elements of out)
+            float u[MLR_VEC], v[MLR_VEC];
+            read(c, u, v);
+            write(c, u, v);
+        }
 }
 
 // The first half of an RMSNorm whose scale is applied by the projection that follows (few rows): x = h + delta
@@ -682,6 +733,60 @@ __global__ __launch_bounds__(256) void gated_part_norm_vec_kernel(const float* _
             for (int e = 0; e < 8; ++e) o[e] = ((v[e] * scale) * (weight ? weight[(c + e) % period] : 1.f)) * gt[e];
         }
         store_vec(out + m * width + c, o);
+    }
+}
+
+// The same with a part's values kept in registers between the sum and the result (one read of y and of the gate): `group`
+// neighbouring lanes (a power of two up to 64) serve a part, or with BLOCK a whole workgroup; a lane takes eight values at
+// a time, at most PART_CHUNKS times.
+#define PART_CHUNKS 4
+template <bool BLOCK>
+__global__ __launch_bounds__(256) void gated_part_norm_reg_kernel(const float* __restrict__ y, const elem_t* __restrict__ gate,
+                                                                  long gate_stride, const float* __restrict__ weight,
+                                                                  elem_t* __restrict__ out, int rows, int width, int part,
+                                                                  int period, float eps, int gate_first, int gate_kind, int group) {
+    __shared__ float scratch[16];
+    const int lanes = BLOCK ? 256 : group, lane = threadIdx.x & (lanes - 1);
+    const size_t unit = ((size_t)blockIdx.x * 256 + threadIdx.x) / lanes;
+    const int parts = width / part;
+    const bool live = unit < (size_t)rows * parts;
+    const size_t m = live ? unit / parts : 0;
+    const int c0 = live ? (int)(unit % parts) * part : 0;
+    float v[PART_CHUNKS][8], g[PART_CHUNKS][8];
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < PART_CHUNKS; ++i) {
+        const int c = (lane + lanes * i) * 8;
+        if (live && c < part) {
+            const float* p = y + m * width + c0 + c;
+            const float4 lo = *reinterpret_cast<const float4*>(p), hi = *reinterpret_cast<const float4*>(p + 4);
+            v[i][0] = lo.x; v[i][1] = lo.y; v[i][2] = lo.z; v[i][3] = lo.w; v[i][4] = hi.x; v[i][5] = hi.y; v[i][6] = hi.z; v[i][7] = hi.w;
+            load_vec(gate + m * gate_stride + c0 + c, g[i]);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                const float sg = 1.0f / (1.0f + expf(-g[i][e]));
+                g[i][e] = gate_kind == 0 ? g[i][e] * sg : sg;
+                if (gate_first) v[i][e] *= g[i][e];
+                sum += v[i][e] * v[i][e];
+            }
+        }
+    }
+    if (BLOCK) sum = block_sum(sum, scratch);
+    else for (int d = 1; d < group; d <<= 1) sum += __shfl_xor(sum, d, MLR_WAVE);
+    const float scale = 1.0f / sqrtf(sum / (float)part + eps);
+#pragma unroll
+    for (int i = 0; i < PART_CHUNKS; ++i) {
+        const int c = (lane + lanes * i) * 8;
+        if (live && c < part) {
+            float o[8], w[8];
+            row_weights<8>(weight, (c0 + c) % period, w);      // (period is a multiple of 8: eight neighbours do not wrap)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                o[e] = (v[i][e] * scale) * w[e];
+                if (!gate_first) o[e] *= g[i][e];
+            }
+            store_vec(out + m * width + c0 + c, o);
+        }
     }
 }
 #endif
@@ -1172,7 +1277,7 @@ int mlr_state_commit(const int64_t* entries, int n_entries, long long most_bytes
 int mlr_normed_sum(const void* a, const void* b, const float* wa, const float* wb, void* out, float sa, float sb, int rows,
                    int width, float eps, hipStream_t stream) {
     if (rows <= 0) return 0;
-    if (MLR_BF16 && width % MLR_VEC == 0 && aligned16(a, b, out))
+    if (MLR_BF16 && width % MLR_VEC == 0 && aligned16(a, b, out, wa, wb))
         normed_sum_kernel<MLR_VEC><<<rows, 256, 0, stream>>>((const elem_t*)a, (const elem_t*)b, wa, wb, (elem_t*)out, sa, sb, width, eps);
     else
         normed_sum_kernel<1><<<rows, 256, 0, stream>>>((const elem_t*)a, (const elem_t*)b, wa, wb, (elem_t*)out, sa, sb, width, eps);
@@ -1223,6 +1328,20 @@ int mlr_gated_part_norm(const float* y, const void* gate, long gate_stride, cons
 #if MLR_BF16
     // (16-byte accesses: parts, the gate's rows and its first column at multiples of 8 elements)
     if (part % 8 == 0 && gate_stride % 8 == 0 && ((uintptr_t)gate) % 16 == 0 && units < (1u << 31)) {
+        if (part <= 256 * 8 * PART_CHUNKS && period % 8 == 0 && aligned16(weight, y, out)) {
+            const bool block = part > 64 * 8 * 2;
+            int group = 2;
+            while (group < 64 && group * 8 < part) group *= 2;
+            const size_t threads = units * (block ? 256 : group);
+            const unsigned grid = (unsigned)((threads + 255) / 256);
+            if (block)
+                gated_part_norm_reg_kernel<true><<<grid, 256, 0, stream>>>(y, (const elem_t*)gate, gate_stride, weight, (elem_t*)out, rows,
+                                                                           width, part, period, eps, gate_first, gate_kind, 256);
+            else
+                gated_part_norm_reg_kernel<false><<<grid, 256, 0, stream>>>(y, (const elem_t*)gate, gate_stride, weight, (elem_t*)out, rows,
+                                                                            width, part, period, eps, gate_first, gate_kind, group);
+            return (int)hipGetLastError();
+        }
         if (part >= 2048)
             gated_part_norm_vec_kernel<4><<<(unsigned)units, 256, 0, stream>>>(y, (const elem_t*)gate, gate_stride, weight,
                                                                               (elem_t*)out, rows, width, part, period, eps,

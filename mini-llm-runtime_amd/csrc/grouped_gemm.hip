@@ -264,6 +264,193 @@ __global__ __launch_bounds__(256) void grouped_gemm_kernel(GroupedArgs g) {
         }
     }
 }
+
+// Experts with many rows each (inner sizes in multiples of 64): 32 x 32 tiles of v_mfma_f32_32x32x16_bf16 out of LDS blocks
+// of 64 k, double-buffered, two further blocks on their way from memory in registers.  A workgroup of WM x WN wavefronts,
+// each TM x TN tiles, owns 32 WM TM sorted rows of one expert and 32 WN TN of its weight's rows.  The weight is the
+// instruction's first operand, so a lane ends up with four consecutive columns of one row (lane = 32 h + i: row i of either
+// operand, k slots 8 h .. 8 h + 7; result column i, rows 8 q + 4 h + r in register 4 q + r); with gate and up rows in turn,
+// 16 and 16, a gate and its up projection lie in one lane, eight registers apart.
+// The workgroups' tiles are counted expert by expert, within one a strip of the weight for all of the expert's rows first;
+// every XCD takes a contiguous range of those there are, so a strip is fetched into one L2.
+typedef __attribute__((__vector_size__(16 * sizeof(float)))) float floatx16;
+#define EB_K 64
+#define EB_PITCH (EB_K + 8)
+
+template <int WM, int WN, int TM, int TN>
+__global__ __launch_bounds__(64 * WM * WN) void experts_wide_kernel(GroupedArgs g) {
+    constexpr int BM = 32 * WM * TM, BN = 32 * WN * TN, THREADS = 64 * WM * WN, ROWS = BM + BN;
+    constexpr int STEP = THREADS / 8, PT = ROWS / STEP, PW = BN / STEP;      // 16-byte pieces a thread stages, of them weight
+    static_assert(ROWS % STEP == 0 && BN % STEP == 0, "the staged pieces must divide among the threads");
+    extern __shared__ __attribute__((aligned(16))) __bf16 eb_lds[];
+    const int t = threadIdx.x, lane = t & 63, wave = t >> 6;
+    const int li = lane & 31, h = lane >> 5, wm = wave / WN, wn = wave % WN;
+    // which tile: every wavefront counts the experts' tiles, a lane an expert, 64 experts at a time
+    const int cols = (g.N + BN - 1) / BN;
+    int total = 0;
+    for (int e0 = 0; e0 < g.groups; e0 += 64) {
+        const int e = e0 + lane;
+        int n = e < g.groups ? (g.offsets[e + 1] - g.offsets[e] + BM - 1) / BM : 0;
+        for (int d = 1; d < 64; d <<= 1) n += __shfl_xor(n, d, MLR_WAVE);
+        total += n * cols;
+    }
+    const int share = (total + 7) / 8;
+    const int tile = (int)(blockIdx.x % 8) * share + (int)(blockIdx.x / 8);
+    if ((int)(blockIdx.x / 8) >= share || tile >= total) return;
+    int group = -1, row0 = 0, row_end = 0, col = 0;
+    for (int e0 = 0, before = 0; e0 < g.groups && group < 0; e0 += 64) {
+        const int e = e0 + lane;
+        const int first = e < g.groups ? g.offsets[e] : 0, count = e < g.groups ? g.offsets[e + 1] - first : 0;
+        const int tiles = (count + BM - 1) / BM * cols;
+        int upto = tiles;                                                     // tiles of the experts up to this lane's
+        for (int d = 1; d < 64; d <<= 1) {
+            const int o = __shfl_up(upto, d, MLR_WAVE);
+            if (lane >= d) upto += o;
+        }
+        const int mine = tile - before - (upto - tiles);
+        const unsigned long long here = __ballot(mine >= 0 && mine < tiles);
+        if (here) {
+            const int src = __ffsll((long long)here) - 1;
+            group = e0 + src;
+            const int at = __shfl(mine, src, MLR_WAVE), f = __shfl(first, src, MLR_WAVE), n = __shfl(count, src, MLR_WAVE);
+            const int row_tiles = (n + BM - 1) / BM;
+            col = at / row_tiles;
+            row0 = f + (at % row_tiles) * BM;
+            row_end = f + n;
+        }
+        before += __shfl(upto, 63, MLR_WAVE);
+    }
+    group = __builtin_amdgcn_readfirstlane(group);
+    if (group < 0) return;
+    const int n0 = col * BN, K = g.K, blocks = K / EB_K;
+    const __bf16* w = g.w + (size_t)group * g.w_group;
+    uint32_t src[PT];
+    const int dst0 = (t >> 3) * EB_PITCH + (t & 7) * 8;
+#pragma unroll
+    for (int i = 0; i < PT; ++i) {
+        const int row = (t >> 3) + STEP * i, kc = (t & 7) * 8;
+        if (i < PW) {
+            src[i] = (uint32_t)min(n0 + row, g.N - 1) * (uint32_t)K + kc;
+        } else {
+            const int m = min(row0 + row - BN, row_end - 1);
+            src[i] = (uint32_t)(g.gather ? g.gather[m] : m) * (uint32_t)g.lda + kc;
+        }
+    }
+    bf16x8 stage0[PT], stage1[PT];
+    auto fetch = [&](int kb, bf16x8 (&stage)[PT]) {                           // (blocks past the end fetch the last one again)
+        const size_t k = (size_t)min(kb, blocks - 1) * EB_K;
+#pragma unroll
+        for (int i = 0; i < PT; ++i) stage[i] = *reinterpret_cast<const bf16x8*>((i < PW ? w : g.a) + k + src[i]);
+    };
+    auto stash = [&](int buf, const bf16x8 (&stage)[PT]) {
+        __bf16* base = eb_lds + (size_t)buf * ROWS * EB_PITCH;
+#pragma unroll
+        for (int i = 0; i < PT; ++i) *reinterpret_cast<bf16x8*>(base + dst0 + i * STEP * EB_PITCH) = stage[i];
+    };
+    floatx16 acc[TN][TM];
+#pragma unroll
+    for (int j = 0; j < TN; ++j)
+#pragma unroll
+        for (int i = 0; i < TM; ++i)
+#pragma unroll
+            for (int e = 0; e < 16; ++e) acc[j][i][e] = 0.f;
+    auto products = [&](int buf) {
+        const __bf16* base = eb_lds + (size_t)buf * ROWS * EB_PITCH;
+        const __bf16* wb = base + (wn * TN * 32 + li) * EB_PITCH + 8 * h;
+        const __bf16* ab = base + (BN + wm * TM * 32 + li) * EB_PITCH + 8 * h;
+        bf16x8 wf[2][TN], af[2][TM];                                          // the next k step's operands are asked for first
+        auto operands = [&](int ks, int set) {
+#pragma unroll
+            for (int j = 0; j < TN; ++j) wf[set][j] = *reinterpret_cast<const bf16x8*>(wb + j * 32 * EB_PITCH + 16 * ks);
+#pragma unroll
+            for (int i = 0; i < TM; ++i) af[set][i] = *reinterpret_cast<const bf16x8*>(ab + i * 32 * EB_PITCH + 16 * ks);
+        };
+        operands(0, 0);
+#pragma unroll
+        for (int ks = 0; ks < EB_K / 16; ++ks) {
+            if (ks + 1 < EB_K / 16) operands(ks + 1, (ks + 1) & 1);
+#pragma unroll
+            for (int j = 0; j < TN; ++j)
+#pragma unroll
+                for (int i = 0; i < TM; ++i)
+                    acc[j][i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(wf[ks & 1][j], af[ks & 1][i], acc[j][i], 0, 0, 0);
+        }
+    };
+    fetch(0, stage0);
+    fetch(1, stage1);
+    stash(0, stage0);
+    fetch(2, stage0);
+    __syncthreads();
+    int kb = 0;
+#pragma unroll 1
+    for (; kb + 2 <= blocks; kb += 2) {                                       // two blocks a turn: the stages keep their names
+        products(0);
+        stash(1, stage1);
+        fetch(kb + 3, stage1);
+        __syncthreads();
+        products(1);
+        stash(0, stage0);
+        fetch(kb + 4, stage0);
+        __syncthreads();
+    }
+    if (kb < blocks) products(0);
+    // results leave through a piece of LDS of the wavefront's own, as rows of 16-byte pieces
+    const bool halves = gated_form(g.act);
+    constexpr int OPITCH = TN * 32 + 8, ROWS_W = TM * 32;
+    static_assert((size_t)WM * WN * ROWS_W * OPITCH <= 2 * (size_t)ROWS * EB_PITCH, "the output tiles must fit the LDS");
+    __syncthreads();                                                          // every wavefront has read its last operands
+    __bf16* mine = eb_lds + (size_t)wave * ROWS_W * OPITCH;
+    typedef __attribute__((__vector_size__(4 * sizeof(__bf16)))) __bf16 bf16x4;
+#pragma unroll
+    for (int i = 0; i < TM; ++i)
+#pragma unroll
+        for (int j = 0; j < TN; ++j)
+#pragma unroll
+            for (int q = 0; q < 4; ++q) {
+                float y[4];
+                if (halves) {
+                    if (q >= 2) continue;
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) y[r] = gated(acc[j][i][4 * q + r], acc[j][i][4 * q + 8 + r], g);
+                } else {
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) y[r] = activate(acc[j][i][4 * q + r], g.act);
+                }
+                *reinterpret_cast<bf16x4*>(mine + (i * 32 + li) * OPITCH + j * (halves ? 16 : 32) + 8 * q + 4 * h) =
+                    bf16x4{(__bf16)y[0], (__bf16)y[1], (__bf16)y[2], (__bf16)y[3]};
+            }
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+    const int width = halves ? TN * 16 : TN * 32, pieces = width / 8, n_out = halves ? g.N / 2 : g.N;
+    const int out_n0 = (halves ? n0 / 2 : n0) + wn * width, out_m0 = row0 + wm * TM * 32;
+    for (int c = lane; c < ROWS_W * pieces; c += 64) {
+        const int row = c / pieces, piece = c % pieces, m = out_m0 + row, n = out_n0 + 8 * piece;
+        if (m >= row_end || n >= n_out) continue;
+        const bf16x8 v = *reinterpret_cast<const bf16x8*>(mine + row * OPITCH + 8 * piece);
+        __bf16* o = (__bf16*)g.out + (size_t)m * g.ldo + n;
+        if (n + 8 <= n_out && g.ldo % 8 == 0) {
+            *reinterpret_cast<bf16x8*>(o) = v;
+        } else {
+#pragma unroll
+            for (int e = 0; e < 8; ++e)
+                if (n + e < n_out) o[e] = v[e];
+        }
+    }
+}
+
+template <int WM, int WN, int TM, int TN>
+static int launch_experts_wide(const GroupedArgs& g, hipStream_t stream) {
+    constexpr int BM = 32 * WM * TM, BN = 32 * WN * TN;
+    constexpr size_t lds = 2 * (size_t)(BM + BN) * EB_PITCH * sizeof(__bf16);
+    static const hipError_t allowed = hipFuncSetAttribute(reinterpret_cast<const void*>(&experts_wide_kernel<WM, WN, TM, TN>),
+                                                          hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    if (allowed != hipSuccess) return (int)allowed;
+    const long tiles = ((long)(g.M + BM - 1) / BM + g.groups) * ((g.N + BN - 1) / BN) + 8;      // (at most, and a multiple of 8)
+    if (tiles > 0x7ffffff0L) return -2;
+    experts_wide_kernel<WM, WN, TM, TN><<<(unsigned)((tiles + 7) / 8 * 8), 64 * WM * WN, lds, stream>>>(g);
+    return (int)hipGetLastError();
+}
 #endif
 
 // ---------------------------------------------------------------------------------------------------------
@@ -482,6 +669,10 @@ int mlr_grouped_gemm(const void* a, long lda, long a_group, const void* w, long 
 #if MLR_BF16
     // experts with many rows each: the large tile (310 -> 340 TFLOP/s at 2048 tokens of width 2048, 390 -> 420 at width
     // 4096; the products a head, with inner sizes of 128 to 512, are faster on the small one)
+    const bool aligned = ((reinterpret_cast<uintptr_t>(a) | reinterpret_cast<uintptr_t>(w) | reinterpret_cast<uintptr_t>(out)) & 15) == 0;
+    if (offsets != nullptr && (long)M >= 128L * groups && N >= 128 && K % EB_K == 0 && lda % 8 == 0 && w_group % 8 == 0 && aligned &&
+        !out_float && (unsigned long long)M * lda < (1ull << 32) && (unsigned long long)N * K < (1ull << 32))
+        return launch_experts_wide<2, 2, 2, 2>(g, stream);
     if (offsets != nullptr && (long)M >= 256L * groups && N >= 128) {
         const int row_tiles = (M + 127) / 128 + (offsets ? groups : 0);
         if (row_tiles > 65535 || groups > 65535) return -2;

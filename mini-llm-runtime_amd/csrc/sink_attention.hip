@@ -258,6 +258,11 @@ __device__ __forceinline__ void turn_eight(float (&x)[8], int li, int half_lanes
     }
 }
 
+__device__ __forceinline__ void eight_floats(const float* p, float (&x)[8]) {
+    *reinterpret_cast<float4*>(x) = *reinterpret_cast<const float4*>(p);
+    *reinterpret_cast<float4*>(x + 4) = *reinterpret_cast<const float4*>(p + 4);
+}
+
 __global__ __launch_bounds__(256) void sink_qkv_prep_vec_kernel(
     const elem_t* __restrict__ proj, long ld, const float* __restrict__ bias, elem_t* __restrict__ q_out,
     elem_t* __restrict__ k_pages, long k_row, elem_t* __restrict__ v_pages, long v_row,
@@ -279,9 +284,12 @@ __global__ __launch_bounds__(256) void sink_qkv_prep_vec_kernel(
     for (int e = 0; e < 8; ++e) x[e] = 0.f;
     if (ok) {
         load_vec(proj + (size_t)m * ld + off, x);
-        if (bias != nullptr)
+        if (bias != nullptr) {
+            float add[8];
+            eight_floats(bias + off, add);
 #pragma unroll
-            for (int e = 0; e < 8; ++e) x[e] += bias[off + e];
+            for (int e = 0; e < 8; ++e) x[e] += add[e];
+        }
     }
     if (!value && norm_mode == 1) {
         float sum = 0.f;
@@ -290,8 +298,10 @@ __global__ __launch_bounds__(256) void sink_qkv_prep_vec_kernel(
         for (int d = 1; d < lanes; d <<= 1) sum += __shfl_xor(sum, d, MLR_WAVE);
         const float r = 1.0f / sqrtf(sum / (float)key_dim + eps);
         const float* w = unit < q_heads ? q_norm_w : k_norm_w;
+        float f[8] = {1.f, 1.f, 1.f, 1.f, 1.f, 1.f, 1.f, 1.f};
+        if (w != nullptr) eight_floats(w + li * 8, f);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) x[e] = (x[e] * r) * (w != nullptr ? w[li * 8 + e] : 1.0f);
+        for (int e = 0; e < 8; ++e) x[e] = (x[e] * r) * f[e];
     }
     if (value) {
         if (v_rope != nullptr) turn_eight(x, li, v_lanes >> 1, v_rope + (size_t)pos * value_dim, value_dim);
@@ -779,7 +789,7 @@ int mlr_sink_qkv_prep(const void* proj, long ld, const float* bias, void* q_out,
     if (norm_mode < 2 && eight_lanes(key_dim) && eight_lanes(value_dim) && ld % 8 == 0 && k_row % 8 == 0 &&
         (v_transposed || v_row % 8 == 0) && (rope == nullptr || (!interleaved && rot_dim % 16 == 0 && aligned(rope))) &&
         (v_rope == nullptr || (!v_interleaved && value_dim % 16 == 0 && aligned(v_rope))) && aligned(proj) && aligned(q_out) &&
-        aligned(k_pages) && aligned(v_pages)) {
+        aligned(k_pages) && aligned(v_pages) && aligned(bias) && aligned(q_norm_w) && aligned(k_norm_w)) {
         const int v_start = ((q_heads + kv_heads) * (key_dim / 8) + 63) / 64 * 64;
         const bool values_apart = v_transposed && rows >= 64 && write_cache && kv_heads <= 65535;
         const int threads = values_apart ? v_start : v_start + kv_heads * (value_dim / 8);

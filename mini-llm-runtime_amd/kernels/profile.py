@@ -15,7 +15,7 @@ import functools
 
 import torch
 
-CLASSES = ("embed", "norm", "gemm", "rope_kv", "attention", "conv", "recurrence", "activation", "sampler", "check")
+CLASSES = ("embed", "norm", "gemm", "rope_kv", "attention", "conv", "recurrence", "state", "activation", "sampler", "check")
 
 
 class Profiler:

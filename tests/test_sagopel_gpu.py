@@ -204,7 +204,7 @@ def test_a_delta_with_a_factor_and_a_vector_ride_in_the_norms_pass(dtype_name, r
 
 
 @pytest.mark.parametrize("dtype_name", DTYPES)
-@pytest.mark.parametrize("rows,width", [(5, 24), (3, 37), (70, 128), (2, 1), (9, 4104)])
+@pytest.mark.parametrize("rows,width", [(5, 24), (3, 37), (70, 128), (2, 1), (9, 4104), (3, 9000), (2, 8195)])
 def test_two_rows_are_normed_apart_and_added(dtype_name, rows, width):
     from mini_llm_runtime_amd.kernels import Kernels
     dtype = DTYPES[dtype_name]
@@ -245,7 +245,7 @@ def test_the_relu_gate(dtype_name, rows, hidden, inter):
 
 
 @pytest.mark.parametrize("dtype_name", DTYPES)
-@pytest.mark.parametrize("heads,values", [(3, 20), (2, 64), (1, 8), (6, 32)])
+@pytest.mark.parametrize("heads,values", [(3, 20), (2, 64), (1, 8), (6, 32), (5, 24), (3, 136), (2, 1024), (1, 1032), (1, 4096), (1, 9000), (2, 512)])
 def test_heads_over_their_own_root_mean_square_without_a_weight(dtype_name, heads, values):
     from mini_llm_runtime_amd.kernels import Kernels
     dtype = DTYPES[dtype_name]
@@ -530,6 +530,42 @@ def test_experts_that_give_their_input_back(dtype_name, rows, experts, identity,
     assert err.max() <= (2e-5 if dtype_name == "float32" else 3e-2) * np.abs(want).max(), err.max()
     ids, _ = P.route(back(x), w64, cfg["router"])
     assert identity == 0 or (ids >= experts).any()
+
+
+@pytest.mark.parametrize("K,N", [(64, 128), (128, 352), (192, 136), (704, 256), (320, 1408), (64, 130)])
+@pytest.mark.parametrize("counts", [[700, 0, 1, 333, 128, 129], [900], [0, 640, 300, 0], [257] * 9 + [0] * 60 + [6000]])
+def test_products_of_experts_with_many_rows(counts, K, N):
+    """Uneven experts, empty ones among them, rows that belong to none behind the others'; every activation, rows gathered
+    and in place, against products in 32-bit."""
+    from mini_llm_runtime_amd.kernels import Kernels
+    k = Kernels(torch.bfloat16)
+    g = torch.Generator(device="cuda").manual_seed(K + N)
+    draw = lambda *shape: torch.randn(shape, generator=g, device="cuda").to(torch.bfloat16)
+    experts, rows, tail = len(counts), sum(counts), 37
+    tokens = rows // 2 + 5
+    x, w = draw(tokens, K), draw(experts, N, K) * K ** -0.5
+    gather = torch.randint(0, tokens, (rows + tail,), generator=g, device="cuda", dtype=torch.int32)
+    offsets = ints(np.concatenate([[0], np.cumsum(counts)]).tolist())
+    gathered = x[gather.long()]
+    want = torch.zeros((rows + tail, N), device="cuda")
+    for e, (lo, n) in enumerate(zip(np.cumsum([0] + counts), counts)):
+        want[lo:lo + n] = gathered[lo:lo + n].float() @ w[e].float().t()
+    for act, apply in ((None, lambda z: z), ("relu_squared", lambda z: torch.relu(z) ** 2), ("gelu_erf", torch.nn.functional.gelu)):
+        for source, rows_of in ((x, gather), (gathered.contiguous(), None)):
+            out = torch.full((rows + tail, N), float("nan"), dtype=torch.bfloat16, device="cuda")
+            k.experts_gemm(source, w, out, offsets, gather=rows_of, act=act)
+            torch.testing.assert_close(out[:rows].float(), apply(want[:rows]), rtol=2e-2, atol=1e-2)
+            assert torch.isnan(out[rows:].float()).all()               # (rows of no expert are not touched)
+    if N % 32 == 0:
+        both = want.view(rows + tail, N // 32, 2, 16)
+        gate, up = both[:, :, 0].reshape(-1, N // 2), both[:, :, 1].reshape(-1, N // 2)
+        clamped = lambda z, u: torch.clamp(z, max=0.8) * torch.sigmoid(1.5 * torch.clamp(z, max=0.8)) * (torch.clamp(u, -0.8, 0.8) + 1.0)
+        for act, y in (("gated_silu", torch.nn.functional.silu(gate) * up), ("gated_clamped", clamped(gate, up)),
+                       ("gated_gelu_tanh", torch.nn.functional.gelu(gate, approximate="tanh") * up)):
+            out = torch.full((rows + tail, N // 2), float("nan"), dtype=torch.bfloat16, device="cuda")
+            k.experts_gemm(x, w, out, offsets, gather=gather, act=act, limit=0.8, slope=1.5)
+            torch.testing.assert_close(out[:rows].float(), y[:rows], rtol=2e-2, atol=1e-2)
+            assert torch.isnan(out[rows:].float()).all()
 
 
 @pytest.mark.parametrize("shapes", [[(5,)], [(3, 8), (4096,), (7,), (4100,)], [(1,), (9000,)]])
